@@ -1,0 +1,263 @@
+// Prompt attention over a paged cache: grouped heads, chunked causal mask,
+// optional sink in the softmax denominator, separate key and value widths.
+//
+// The kv loop walks cache pages (64 keys), so a tile of keys is one
+// contiguous block per kv head whatever the prompt's cut.  Row i of a tile
+// sits at absolute position pos0 + i and sees keys from the start of its
+// own chunk to itself; only pages between the first row's chunk start and
+// the last row are visited.
+//
+// Scores, the running maximum and sum and the weights are float.  In bf16
+// mode the weights enter the value product as two bf16 parts, which keeps
+// 16 significand bits of them.
+
+#include "lm.h"
+#include "tile.h"
+
+#include <type_traits>
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+
+// One wave per (row, head) vector: RMS norm over `dim` for q heads (in
+// place) and k heads (into the cache), plain copy for v heads.
+template <bool F32>
+__global__ void __launch_bounds__(256)
+attn_prep_kernel(AttnArgs a, const int* __restrict__ pos,
+                 const int* __restrict__ slot, int row0, int n) {
+  using N = Num<F32>;
+  using E = typename N::E;
+  const int heads = a.H + 2 * a.G;
+  const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (unit >= (long)n * heads) return;
+  const int l = threadIdx.x & 63;
+  const int row = row0 + (int)(unit / heads);
+  const int hd = (int)(unit % heads);
+  const int s = slot[row];
+  if (s < 0) return;
+  const int p = pos[row];
+  E* base = (E*)a.qkv + (long)row * a.ld;
+
+  if (hd >= a.H + a.G) {           // value head
+    const int g = hd - a.H - a.G;
+    const E* src = base + (long)(a.H + a.G) * a.dim + (long)g * a.vdim;
+    const long page = a.table[(long)s * a.max_pages + p / LM_PAGE];
+    E* dst = (E*)a.vc + ((page * a.G + g) * LM_PAGE + p % LM_PAGE) * a.vdim;
+    for (int c = l; c < a.vdim; c += 64) dst[c] = src[c];
+    return;
+  }
+  E* src = base + (long)hd * a.dim;
+  const void* w = hd < a.H ? a.qw : a.kw;
+  float v[4];
+  float q = 0.f;
+  #pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = i * 64 + l;
+    v[i] = c < a.dim ? N::up(src[c]) : 0.f;
+    q += v[i] * v[i];
+  }
+  const float inv = w ? 1.0f / sqrtf(wave_reduce_sum(q) / (float)a.dim + a.eps) : 1.f;
+  E* dst = src;
+  if (hd >= a.H) {
+    const int g = hd - a.H;
+    const long page = a.table[(long)s * a.max_pages + p / LM_PAGE];
+    dst = (E*)a.kc + ((page * a.G + g) * LM_PAGE + p % LM_PAGE) * a.dim;
+  }
+  #pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = i * 64 + l;
+    if (c < a.dim)
+      dst[c] = N::down(w ? v[i] * inv * N::up(((const E*)w)[c]) : v[i]);
+  }
+}
+
+// 4 waves, 16 query rows each; one query head per block.
+template <bool F32, int DK, int DV>
+__global__ void __launch_bounds__(256)
+attn_prefill_kernel(AttnArgs a, const int4* __restrict__ tiles) {
+  using N = Num<F32>;
+  using E = typename N::E;
+  constexpr int LDK = DK + N::PAD;
+  constexpr int LDJ = LM_PAGE + N::PAD;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  E* Ks = (E*)smem;                       // [64][LDK]
+  E* Vt = Ks + LM_PAGE * LDK;             // [DV][LDJ]  values, transposed
+  E* Pb = Vt + DV * LDJ;                  // [PARTS][64][LDJ]
+  const Split<F32> P{Pb, Pb + LM_TILE * LDJ};
+
+  const int4 t = tiles[blockIdx.x];       // first row, rows, pos0, slot
+  const int h = blockIdx.y, g = h / (a.H / a.G);
+  const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
+  const int lr = l & 15, lg = l >> 4;
+  const bool aligned = a.dim % 8 == 0 && a.vdim % 8 == 0;
+
+  // this wave's 16 q rows as A fragments
+  typename N::Frag qf[DK / 32];
+  {
+    const int r = 16 * w + lr;
+    const E* qrow = (const E*)a.qkv + (long)(t.x + min(r, t.y - 1)) * a.ld + (long)h * a.dim;
+    #pragma unroll
+    for (int kb = 0; kb < DK / 32; ++kb) {
+      float v[8];
+      const int c = kb * 32 + lg * 8;
+      load8<F32>(qrow + c, a.dim - c, aligned, v);
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        if constexpr (F32) qf[kb].v[i] = v[i];
+        else qf[kb][i] = N::down(v[i]);
+      }
+    }
+  }
+
+  const float scale2 = a.scale * LOG2E;   // softmax in base 2
+  int cs[4], ip[4];                       // chunk start, position per row
+  float m[4], lsum[4];
+  f32x4 o[DV / 16];
+  #pragma unroll
+  for (int i = 0; i < DV / 16; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  #pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int row = 16 * w + 4 * lg + r;
+    ip[r] = t.z + min(row, t.y - 1);
+    cs[r] = a.size ? ip[r] - ip[r] % a.size : 0;
+    m[r] = a.sink ? N::up(((const E*)a.sink)[h]) * LOG2E : -1e30f;
+    lsum[r] = a.sink ? 1.f : 0.f;
+  }
+
+  const int p_last = t.z + t.y - 1;
+  const int j_first = a.size ? t.z - t.z % a.size : 0;
+  const int* tab = a.table + (long)t.w * a.max_pages;
+  for (int pg = j_first / LM_PAGE; pg <= p_last / LM_PAGE; ++pg) {
+    const long page = tab[pg];
+    const E* kp = (const E*)a.kc + (page * a.G + g) * LM_PAGE * a.dim;
+    const E* vp = (const E*)a.vc + (page * a.G + g) * LM_PAGE * a.vdim;
+    const int j0 = pg * LM_PAGE;
+    __syncthreads();                      // the last tile's reads are over
+    for (int u = tid; u < LM_PAGE * (DK / 8); u += 256) {
+      const int j = u / (DK / 8), c = (u % (DK / 8)) * 8;
+      float v[8];
+      const bool ok = j0 + j >= j_first && j0 + j <= p_last;
+      load8<F32>(kp + (long)j * a.dim + c, ok ? a.dim - c : 0, aligned, v);
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) Ks[j * LDK + c + i] = N::down(v[i]);
+    }
+    for (int u = tid; u < LM_PAGE * (DV / 8); u += 256) {
+      const int j = u % LM_PAGE, c = (u / LM_PAGE) * 8;
+      float v[8];
+      const bool ok = j0 + j >= j_first && j0 + j <= p_last;
+      load8<F32>(vp + (long)j * a.vdim + c, ok ? a.vdim - c : 0, aligned, v);
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) Vt[(c + i) * LDJ + j] = N::down(v[i]);
+    }
+    __syncthreads();
+
+    f32x4 s[4];
+    #pragma unroll
+    for (int ct = 0; ct < 4; ++ct) {
+      s[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
+      #pragma unroll
+      for (int kb = 0; kb < DK / 32; ++kb)
+        s[ct] = N::mma(qf[kb], N::load(Ks + (ct * 16 + lr) * LDK, kb * 32 + lg * 8), s[ct]);
+    }
+    float mx[4] = {-1e30f, -1e30f, -1e30f, -1e30f};
+    #pragma unroll
+    for (int ct = 0; ct < 4; ++ct)
+      #pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = j0 + ct * 16 + lr;
+        const bool see = j <= ip[r] && j >= cs[r];
+        s[ct][r] = see ? s[ct][r] * scale2 : -1e30f;
+        mx[r] = fmaxf(mx[r], s[ct][r]);
+      }
+    #pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float mn = fmaxf(m[r], max16(mx[r]));
+      const float al = exp2f(m[r] - mn);
+      m[r] = mn;
+      float ps = 0.f;
+      #pragma unroll
+      for (int ct = 0; ct < 4; ++ct) {
+        // a row that has seen no key yet has mn = -1e30: its weights are 0
+        const float e = s[ct][r] > -1e29f ? exp2f(s[ct][r] - mn) : 0.f;
+        ps += e;
+        P.put((16 * w + 4 * lg + r) * LDJ + ct * 16 + lr, e);
+      }
+      lsum[r] = lsum[r] * al + sum16(ps);
+      #pragma unroll
+      for (int i = 0; i < DV / 16; ++i) o[i][r] *= al;
+    }
+    // P rows are written and read by the same wave; order its LDS ops
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    #pragma unroll
+    for (int kb = 0; kb < LM_PAGE / 32; ++kb) {
+      const auto pf = P.load((16 * w + lr) * LDJ, kb * 32 + lg * 8);
+      #pragma unroll
+      for (int i = 0; i < DV / 16; ++i)
+        o[i] = mma_sp<F32>(pf, N::load(Vt + (i * 16 + lr) * LDJ, kb * 32 + lg * 8), o[i]);
+    }
+  }
+
+  #pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int row = 16 * w + 4 * lg + r;
+    if (row >= t.y) continue;
+    const float inv = lsum[r] > 0.f ? 1.0f / lsum[r] : 0.f;
+    E* dst = (E*)a.out + (long)(t.x + row) * a.H * a.vdim + (long)h * a.vdim;
+    #pragma unroll
+    for (int i = 0; i < DV / 16; ++i)
+      if (i * 16 + lr < a.vdim) dst[i * 16 + lr] = N::down(o[i][r] * inv);
+  }
+}
+
+template <bool F32, int DK, int DV>
+void launch_prefill(const AttnArgs& a, const int4* tiles, int n_tiles,
+                    hipStream_t st) {
+  using N = Num<F32>;
+  constexpr int LDJ = LM_PAGE + N::PAD;
+  constexpr size_t lds = sizeof(typename N::E) *
+      (LM_PAGE * (DK + N::PAD) + DV * LDJ + Split<F32>::PARTS * LM_TILE * LDJ);
+  static_assert(lds <= 160 * 1024, "exceeds the CU's LDS");
+  static const hipError_t attr = hipFuncSetAttribute(
+      (const void*)attn_prefill_kernel<F32, DK, DV>,
+      hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+  (void)attr;
+  hipLaunchKernelGGL((attn_prefill_kernel<F32, DK, DV>), dim3(n_tiles, a.H),
+                     dim3(256), lds, st, a, tiles);
+}
+
+template <bool F32, int DK>
+void pick_dv(const AttnArgs& a, const int4* tiles, int n, hipStream_t st) {
+  if (a.vdim <= 64) launch_prefill<F32, DK, 64>(a, tiles, n, st);
+  else if (a.vdim <= 128) launch_prefill<F32, DK, 128>(a, tiles, n, st);
+  else launch_prefill<F32, DK, 256>(a, tiles, n, st);
+}
+
+template <bool F32>
+void pick_dk(const AttnArgs& a, const int4* tiles, int n, hipStream_t st) {
+  if (a.dim <= 64) pick_dv<F32, 64>(a, tiles, n, st);
+  else if (a.dim <= 128) pick_dv<F32, 128>(a, tiles, n, st);
+  else pick_dv<F32, 256>(a, tiles, n, st);
+}
+
+}  // namespace
+
+void lm_attn_prep(const AttnArgs& a, const int* pos, const int* slot, int row0,
+                  int n, bool f32, hipStream_t stream) {
+  if (n <= 0) return;
+  const long units = (long)n * (a.H + 2 * a.G);
+  const dim3 grid((units + 3) / 4);
+  if (f32)
+    hipLaunchKernelGGL((attn_prep_kernel<true>), grid, dim3(256), 0, stream, a, pos, slot, row0, n);
+  else
+    hipLaunchKernelGGL((attn_prep_kernel<false>), grid, dim3(256), 0, stream, a, pos, slot, row0, n);
+}
+
+void lm_attn_prefill(const AttnArgs& a, const int4* tiles, int n_tiles,
+                     bool f32, hipStream_t stream) {
+  if (n_tiles <= 0) return;
+  if (f32) pick_dk<true>(a, tiles, n_tiles, stream);
+  else pick_dk<false>(a, tiles, n_tiles, stream);
+}

@@ -1,0 +1,290 @@
+// Decode attention: one new token per row against its paged cache, all
+// query heads of a kv head in one block so keys and values are read once.
+//
+// The block norms q (every split needs it) and, in the split that holds
+// the new token, norms k and appends k and v to the cache; the new key is
+// scored from registers, so no other block waits for that write.
+// LPK lanes share one key (8 elements each), 64/LPK keys go through a wave
+// at a time and each lane group keeps its own running softmax; groups,
+// waves and splits merge at the end.  The sink joins the last merge.
+
+#include "lm.h"
+#include "tile.h"
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr float NEG = -1e30f;
+
+template <int LPK>
+DEVINL float group_sum(float v) {
+  #pragma unroll
+  for (int o = 1; o < LPK; o <<= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+
+// 8 elements, normed over the lane group and rounded to the cache's type
+template <bool F32, int LPK>
+DEVINL void head_norm(float* v, const void* w, int c, int dim, float eps) {
+  using N = Num<F32>;
+  float q = 0.f;
+  #pragma unroll
+  for (int i = 0; i < 8; ++i) q += v[i] * v[i];
+  q = group_sum<LPK>(q);
+  if (!w) return;
+  const float inv = 1.0f / sqrtf(q / (float)dim + eps);
+  #pragma unroll
+  for (int i = 0; i < 8; ++i)
+    if (c + i < dim)
+      v[i] = N::up(N::down(v[i] * inv * N::up(((const typename N::E*)w)[c + i])));
+}
+
+template <bool F32, int LPK, int HGC>
+__global__ void __launch_bounds__(256)
+attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
+                   const int* __restrict__ slot, int nsplit,
+                   float* __restrict__ ws) {
+  using N = Num<F32>;
+  using E = typename N::E;
+  constexpr int KPW = 64 / LPK;      // keys per wave and pass
+  constexpr int KB = 4;              // passes in flight
+  __shared__ float acc_s[4][HGC][LPK * 8];
+  __shared__ float m_s[4][HGC], l_s[4][HGC];
+
+  const int split = blockIdx.x, row = blockIdx.z;
+  const int hg = a.H / a.G, nhc = (hg + HGC - 1) / HGC;
+  const int g = blockIdx.y / nhc, hc = blockIdx.y % nhc;
+  const int nh = min(HGC, hg - hc * HGC);     // heads of this block
+  const int h0 = g * hg + hc * HGC;
+  const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
+  const int grp = l / LPK, c = (l % LPK) * 8;
+  const bool aligned = a.dim % 8 == 0 && a.vdim % 8 == 0;
+  E* out = (E*)a.out + (long)row * a.H * a.vdim;
+
+  const int s = slot[row];
+  if (s < 0) {                        // idle row: a defined, unused output
+    if (split == 0)
+      for (int i = tid; i < nh * a.vdim; i += 256)
+        out[(long)h0 * a.vdim + i] = N::down(0.f);
+    if (nsplit > 1)
+      for (int i = tid; i < nh * (a.vdim + 2); i += 256)
+        ws[(((long)row * a.H + h0 + i / (a.vdim + 2)) * nsplit + split) *
+               (a.vdim + 2) + i % (a.vdim + 2)] = 0.f;
+    return;
+  }
+  const int p = pos[row];
+  const int cs = a.size ? p - p % a.size : 0;
+  const int nkeys = p - cs + 1;
+  const int per = (nkeys + nsplit - 1) / nsplit;
+  const int jb = cs + split * per;
+  const int je = min(jb + per, p + 1);        // may be <= jb: empty split
+  const bool has_new = jb <= p && je == p + 1;
+  const int* tab = a.table + (long)s * a.max_pages;
+  const E* qkv = (const E*)a.qkv + (long)row * a.ld;
+
+  float q[HGC][8], acc[HGC][8], m[HGC], ls[HGC];
+  const float scale2 = a.scale * LOG2E;
+  #pragma unroll
+  for (int i = 0; i < HGC; ++i) {
+    load8<F32>(qkv + (long)(h0 + min(i, nh - 1)) * a.dim + c, a.dim - c, aligned, q[i]);
+    head_norm<F32, LPK>(q[i], a.qw, c, a.dim, a.eps);
+    m[i] = NEG;
+    ls[i] = 0.f;
+    #pragma unroll
+    for (int j = 0; j < 8; ++j) acc[i][j] = 0.f;
+  }
+
+  auto fold = [&](const float (&k)[KB][8], const float (&v)[KB][8],
+                  const bool (&ok)[KB]) {
+    #pragma unroll
+    for (int i = 0; i < HGC; ++i) {
+      float sc[KB], mx = m[i];
+      #pragma unroll
+      for (int u = 0; u < KB; ++u) {
+        float d = 0.f;
+        #pragma unroll
+        for (int j = 0; j < 8; ++j) d = fmaf(q[i][j], k[u][j], d);
+        d = group_sum<LPK>(d) * scale2;
+        sc[u] = ok[u] ? d : NEG;
+        mx = fmaxf(mx, sc[u]);
+      }
+      const float al = exp2f(m[i] - mx);
+      m[i] = mx;
+      float e[KB], es = 0.f;
+      #pragma unroll
+      for (int u = 0; u < KB; ++u) {
+        e[u] = ok[u] ? exp2f(sc[u] - mx) : 0.f;
+        es += e[u];
+      }
+      ls[i] = ls[i] * al + es;
+      #pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        float t = acc[i][j] * al;
+        #pragma unroll
+        for (int u = 0; u < KB; ++u) t = fmaf(e[u], v[u][j], t);
+        acc[i][j] = t;
+      }
+    }
+  };
+
+  const int jc = min(je, p);                  // cached keys end here
+  for (int j0 = jb; j0 < jc; j0 += 4 * KPW * KB) {
+    float k[KB][8], v[KB][8];
+    bool ok[KB];
+    #pragma unroll
+    for (int u = 0; u < KB; ++u) {
+      const int j = j0 + (u * 4 + w) * KPW + grp;
+      ok[u] = j < jc;
+      long kb = 0, vb = 0;
+      if (ok[u]) {
+        const long cell = ((long)tab[j / LM_PAGE] * a.G + g) * LM_PAGE + j % LM_PAGE;
+        kb = cell * a.dim + c;
+        vb = cell * a.vdim + c;
+      }
+      load8<F32>((const E*)a.kc + kb, ok[u] ? a.dim - c : 0, aligned, k[u]);
+      load8<F32>((const E*)a.vc + vb, ok[u] ? a.vdim - c : 0, aligned, v[u]);
+    }
+    fold(k, v, ok);
+  }
+  if (has_new && w == 0) {
+    float k[KB][8], v[KB][8];
+    bool ok[KB];
+    #pragma unroll
+    for (int u = 0; u < KB; ++u) {
+      ok[u] = u == 0 && grp == 0;
+      #pragma unroll
+      for (int j = 0; j < 8; ++j) k[u][j] = v[u][j] = 0.f;
+    }
+    load8<F32>(qkv + (long)(a.H + g) * a.dim + c, a.dim - c, aligned, k[0]);
+    load8<F32>(qkv + (long)(a.H + a.G) * a.dim + (long)g * a.vdim + c,
+               a.vdim - c, aligned, v[0]);
+    head_norm<F32, LPK>(k[0], a.kw, c, a.dim, a.eps);
+    if (grp == 0 && hc == 0) {
+      const long cell = ((long)tab[p / LM_PAGE] * a.G + g) * LM_PAGE + p % LM_PAGE;
+      E* kd = (E*)a.kc + cell * a.dim + c;
+      E* vd = (E*)a.vc + cell * a.vdim + c;
+      #pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        if (c + j < a.dim) kd[j] = N::down(k[0][j]);
+        if (c + j < a.vdim) vd[j] = N::down(v[0][j]);
+      }
+    }
+    fold(k, v, ok);
+  }
+
+  // lane groups of a wave, then the four waves
+  #pragma unroll
+  for (int i = 0; i < HGC; ++i) {
+    #pragma unroll
+    for (int o = LPK; o < 64; o <<= 1) {
+      const float mo = __shfl_xor(m[i], o, 64), lo = __shfl_xor(ls[i], o, 64);
+      const float mn = fmaxf(m[i], mo);
+      const float x = exp2f(m[i] - mn), y = exp2f(mo - mn);
+      ls[i] = ls[i] * x + lo * y;
+      #pragma unroll
+      for (int j = 0; j < 8; ++j)
+        acc[i][j] = acc[i][j] * x + __shfl_xor(acc[i][j], o, 64) * y;
+      m[i] = mn;
+    }
+    if (grp == 0) {
+      #pragma unroll
+      for (int j = 0; j < 8; ++j) acc_s[w][i][c + j] = acc[i][j];
+      if (l == 0) {
+        m_s[w][i] = m[i];
+        l_s[w][i] = ls[i];
+      }
+    }
+  }
+  __syncthreads();
+  for (int t = tid; t < nh * a.vdim; t += 256) {
+    const int i = t / a.vdim, d = t % a.vdim;
+    float mn = NEG;
+    #pragma unroll
+    for (int x = 0; x < 4; ++x) mn = fmaxf(mn, m_s[x][i]);
+    float lt = 0.f, av = 0.f;
+    #pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      const float f = exp2f(m_s[x][i] - mn);
+      lt += l_s[x][i] * f;
+      av += acc_s[x][i][d] * f;
+    }
+    if (nsplit == 1) {
+      if (a.sink) {
+        const float sk = N::up(((const E*)a.sink)[h0 + i]) * LOG2E;
+        const float mt = fmaxf(mn, sk);
+        const float f = exp2f(mn - mt);
+        lt = lt * f + exp2f(sk - mt);
+        av *= f;
+      }
+      out[(long)(h0 + i) * a.vdim + d] = N::down(av / lt);
+    } else {
+      float* o = ws + (((long)row * a.H + h0 + i) * nsplit + split) * (a.vdim + 2);
+      o[2 + d] = av;
+      if (d == 0) {
+        o[0] = mn;
+        o[1] = lt;
+      }
+    }
+  }
+}
+
+template <bool F32>
+__global__ void __launch_bounds__(256)
+attn_combine_kernel(AttnArgs a, const int* __restrict__ slot, int nsplit,
+                    const float* __restrict__ ws) {
+  using N = Num<F32>;
+  using E = typename N::E;
+  const int h = blockIdx.x, row = blockIdx.y;
+  if (slot[row] < 0) return;
+  const float* p = ws + ((long)row * a.H + h) * nsplit * (a.vdim + 2);
+  const int st = a.vdim + 2;
+  float mn = a.sink ? N::up(((const E*)a.sink)[h]) * LOG2E : NEG;
+  float lt = 0.f;
+  const float m0 = mn;
+  for (int i = 0; i < nsplit; ++i) mn = fmaxf(mn, p[i * st]);
+  if (a.sink) lt = exp2f(m0 - mn);
+  for (int i = 0; i < nsplit; ++i) lt += p[i * st + 1] * exp2f(p[i * st] - mn);
+  for (int d = threadIdx.x; d < a.vdim; d += 256) {
+    float av = 0.f;
+    for (int i = 0; i < nsplit; ++i)
+      av += p[i * st + 2 + d] * exp2f(p[i * st] - mn);
+    ((E*)a.out)[((long)row * a.H + h) * a.vdim + d] = N::down(av / lt);
+  }
+}
+
+template <bool F32, int LPK>
+void pick_heads(const AttnArgs& a, const int* pos, const int* slot, int R,
+                int nsplit, float* ws, hipStream_t st) {
+  const int hg = a.H / a.G;
+  #define AD_GO(HGC)                                                           \
+    hipLaunchKernelGGL((attn_decode_kernel<F32, LPK, HGC>),                    \
+                       dim3(nsplit, a.G * ((hg + HGC - 1) / HGC), R),          \
+                       dim3(256), 0, st, a, pos, slot, nsplit, ws)
+  if (hg == 1) AD_GO(1);
+  else if (hg == 2) AD_GO(2);
+  else AD_GO(4);
+  #undef AD_GO
+}
+
+template <bool F32>
+void run_decode(const AttnArgs& a, const int* pos, const int* slot, int R,
+                int nsplit, float* ws, hipStream_t st) {
+  const int d = std::max(a.dim, a.vdim);
+  if (d <= 32) pick_heads<F32, 4>(a, pos, slot, R, nsplit, ws, st);
+  else if (d <= 64) pick_heads<F32, 8>(a, pos, slot, R, nsplit, ws, st);
+  else if (d <= 128) pick_heads<F32, 16>(a, pos, slot, R, nsplit, ws, st);
+  else pick_heads<F32, 32>(a, pos, slot, R, nsplit, ws, st);
+  if (nsplit > 1)
+    hipLaunchKernelGGL((attn_combine_kernel<F32>), dim3(a.H, R),
+                       dim3(a.vdim <= 64 ? 64 : a.vdim <= 128 ? 128 : 256), 0,
+                       st, a, slot, nsplit, ws);
+}
+
+}  // namespace
+
+void lm_attn_decode(const AttnArgs& a, const int* pos, const int* slot, int R,
+                    int nsplit, float* ws, bool f32, hipStream_t stream) {
+  if (R <= 0) return;
+  if (f32) run_decode<true>(a, pos, slot, R, nsplit, ws, stream);
+  else run_decode<false>(a, pos, slot, R, nsplit, ws, stream);
+}

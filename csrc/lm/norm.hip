@@ -1,0 +1,262 @@
+// Residual-stream kernels: the stream x stays float in HBM and is touched
+// once per sublayer.  One launch applies the norm after a sublayer, adds
+// it to the stream and produces the next sublayer's normed input:
+//     x <- x + mult * LN(y; post)        h <- LN(x; next)
+// so a layer costs two reads and one write of x instead of four passes.
+//
+// Rows up to 2048 wide take one wave each (4 rows a block, shuffles
+// only); wider rows take a 4-wave block.  Row values stay in registers
+// between the mean and the variance pass.
+
+#include "lm.h"
+#include "tile.h"
+
+namespace {
+
+template <int VEC> struct Pack { float v[VEC]; };
+
+template <bool F32, int VEC>
+DEVINL Pack<VEC> ldv(const void* base, long i) {
+  Pack<VEC> p;
+  if constexpr (F32) {
+    const float* s = (const float*)base + i;
+    if constexpr (VEC == 4) *(f32x4*)p.v = *(const f32x4*)s;
+    else p.v[0] = s[0];
+  } else {
+    const short* s = (const short*)base + i;
+    if constexpr (VEC == 4) {
+      const bf16x4 t = *(const bf16x4*)s;
+      #pragma unroll
+      for (int j = 0; j < 4; ++j) p.v[j] = bf2f(t[j]);
+    } else {
+      p.v[0] = bf2f(s[0]);
+    }
+  }
+  return p;
+}
+
+template <bool F32, int VEC>
+DEVINL void stv(void* base, long i, const Pack<VEC>& p) {
+  if constexpr (F32) {
+    float* s = (float*)base + i;
+    if constexpr (VEC == 4) *(f32x4*)s = *(const f32x4*)p.v;
+    else s[0] = p.v[0];
+  } else {
+    short* s = (short*)base + i;
+    if constexpr (VEC == 4) {
+      bf16x4 t;
+      #pragma unroll
+      for (int j = 0; j < 4; ++j) t[j] = cvt_bf16(p.v[j]);
+      *(bf16x4*)s = t;
+    } else {
+      s[0] = cvt_bf16(p.v[0]);
+    }
+  }
+}
+
+template <int TPR>
+DEVINL float row_sum(float v, float* red) {
+  v = wave_reduce_sum(v);
+  if constexpr (TPR == 256) {
+    const int w = threadIdx.x >> 6;
+    __syncthreads();             // the previous use of red is over
+    if ((threadIdx.x & 63) == 0) red[w] = v;
+    __syncthreads();
+    v = red[0] + red[1] + red[2] + red[3];
+  }
+  return v;
+}
+
+template <int TPR, int VEC, int NV>
+DEVINL void layer_norm_rows(Pack<VEC> (&v)[NV], int tid, int W, float eps,
+                            float* red) {
+  float s = 0.f;
+  #pragma unroll
+  for (int i = 0; i < NV; ++i)
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) s += v[i].v[j];  // lanes past W hold 0
+  const float mean = row_sum<TPR>(s, red) / (float)W;
+  float q = 0.f;
+  #pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const bool ok = (i * TPR + tid) * VEC < W;
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float d = v[i].v[j] - mean;
+      v[i].v[j] = d;
+      q += ok ? d * d : 0.f;
+    }
+  }
+  const float inv = 1.0f / sqrtf(row_sum<TPR>(q, red) / (float)W + eps);
+  #pragma unroll
+  for (int i = 0; i < NV; ++i)
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) v[i].v[j] *= inv;
+}
+
+struct NormArgs {
+  const long* tokens;   // embedding form: x <- embed[token]
+  const void* embed;
+  long vocab;
+  float* x;
+  const void* y;        // sublayer output or null
+  const void* pw;       // its norm (null: y is added as it is)
+  const void* pb;
+  float mult;
+  const void* nw;       // next norm or null
+  const void* nb;
+  void* h;
+  const int* rows;      // null: identity; else h[r] comes from x[rows[r]]
+  int T, W;
+  float eps;
+  bool store_x;
+};
+
+template <bool F32, int TPR, int VEC, int NV>
+__global__ void __launch_bounds__(256)
+residual_norm_kernel(NormArgs a) {
+  __shared__ float red[4];
+  constexpr int RPB = 256 / TPR;
+  const int tid = threadIdx.x % TPR;
+  const int out_row = blockIdx.x * RPB + threadIdx.x / TPR;
+  if (out_row >= a.T) return;     // whole wave (TPR 64) or whole block
+  const long row = a.rows ? a.rows[out_row] : out_row;
+  const int W = a.W;
+
+  Pack<VEC> x[NV];
+  if (a.tokens) {
+    const long tok = a.tokens[row];
+    const bool ok = tok >= 0 && tok < a.vocab;
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      x[i] = Pack<VEC>{};
+      if (c < W && ok) x[i] = ldv<F32, VEC>(a.embed, tok * W + c);
+      if (c < W) stv<true, VEC>(a.x, row * W + c, x[i]);
+    }
+  } else {
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      x[i] = Pack<VEC>{};
+      if (c < W) x[i] = ldv<true, VEC>(a.x, row * W + c);
+    }
+  }
+  if (a.y) {
+    Pack<VEC> y[NV];
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      y[i] = Pack<VEC>{};
+      if (c < W) y[i] = ldv<F32, VEC>(a.y, row * W + c);
+    }
+    if (a.pw) layer_norm_rows<TPR, VEC, NV>(y, tid, W, a.eps, red);
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      if (c < W) {
+        if (a.pw) {
+          const Pack<VEC> w = ldv<F32, VEC>(a.pw, c);
+          Pack<VEC> b{};
+          if (a.pb) b = ldv<F32, VEC>(a.pb, c);
+          #pragma unroll
+          for (int j = 0; j < VEC; ++j)
+            y[i].v[j] = y[i].v[j] * w.v[j] + b.v[j];
+        }
+        #pragma unroll
+        for (int j = 0; j < VEC; ++j) x[i].v[j] += a.mult * y[i].v[j];
+        if (a.store_x) stv<true, VEC>(a.x, row * W + c, x[i]);
+      }
+    }
+  }
+  if (a.nw) {
+    layer_norm_rows<TPR, VEC, NV>(x, tid, W, a.eps, red);
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      if (c < W) {
+        const Pack<VEC> w = ldv<F32, VEC>(a.nw, c);
+        Pack<VEC> b{};
+        if (a.nb) b = ldv<F32, VEC>(a.nb, c);
+        #pragma unroll
+        for (int j = 0; j < VEC; ++j)
+          x[i].v[j] = x[i].v[j] * w.v[j] + b.v[j];
+        stv<F32, VEC>(a.h, (long)out_row * W + c, x[i]);
+      }
+    }
+  }
+}
+
+template <bool F32, int VEC>
+void launch_norm(const NormArgs& a, hipStream_t st) {
+  #define LN_GO(TPR, NV)                                                       \
+    hipLaunchKernelGGL((residual_norm_kernel<F32, TPR, VEC, NV>),              \
+                       dim3((a.T * TPR + 255) / 256), dim3(256), 0, st, a)
+  if (a.W <= 64 * VEC) LN_GO(64, 1);
+  else if (a.W <= 128 * VEC) LN_GO(64, 2);
+  else if (a.W <= 256 * VEC) LN_GO(64, 4);
+  else if (a.W <= 512 * VEC) LN_GO(64, 8);
+  else if (a.W <= 1024 * VEC) LN_GO(256, 4);
+  else if (a.W <= 2048 * VEC) LN_GO(256, 8);
+  else LN_GO(256, 16);            // up to 4096 * VEC (checked by the caller)
+  #undef LN_GO
+}
+
+void dispatch_norm(const NormArgs& a, bool f32, hipStream_t st) {
+  if (a.T <= 0) return;
+  const bool v4 = a.W % 4 == 0;
+  if (f32) v4 ? launch_norm<true, 4>(a, st) : launch_norm<true, 1>(a, st);
+  else v4 ? launch_norm<false, 4>(a, st) : launch_norm<false, 1>(a, st);
+}
+
+template <bool F32>
+__global__ void __launch_bounds__(256)
+gelu_erf_kernel(const void* in, void* out, long n4, long n) {
+  const long step = grid_stride();
+  auto f = [](float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); };
+  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n4; i += step) {
+    Pack<4> p = ldv<F32, 4>(in, i * 4);
+    #pragma unroll
+    for (int j = 0; j < 4; ++j) p.v[j] = f(p.v[j]);
+    stv<F32, 4>(out, i * 4, p);
+  }
+  const long tail = n4 * 4 + (long)blockIdx.x * 256 + threadIdx.x;
+  if (tail < n) {
+    Pack<1> p = ldv<F32, 1>(in, tail);
+    p.v[0] = f(p.v[0]);
+    stv<F32, 1>(out, tail, p);
+  }
+}
+
+}  // namespace
+
+void lm_embed_norm(const long* tokens, const void* embed, float* x,
+                   const void* w, const void* b, void* h, int T, int W,
+                   long vocab, float eps, bool f32, hipStream_t stream) {
+  NormArgs a{};
+  a.tokens = tokens; a.embed = embed; a.vocab = vocab;
+  a.x = x; a.nw = w; a.nb = b; a.h = h; a.T = T; a.W = W; a.eps = eps;
+  dispatch_norm(a, f32, stream);
+}
+
+void lm_residual_norm(float* x, const void* y, const void* pw, const void* pb,
+                      float mult, const void* nw, const void* nb, void* h,
+                      const int* rows, int T, int W, float eps, bool store_x,
+                      bool f32, hipStream_t stream) {
+  NormArgs a{};
+  a.x = x; a.y = y; a.pw = pw; a.pb = pb; a.mult = mult;
+  a.nw = nw; a.nb = nb; a.h = h; a.rows = rows; a.T = T; a.W = W; a.eps = eps;
+  a.store_x = store_x;
+  dispatch_norm(a, f32, stream);
+}
+
+void lm_gelu_erf(const void* in, void* out, long n, bool f32,
+                 hipStream_t stream) {
+  if (n <= 0) return;
+  const long n4 = n / 4;
+  const dim3 grid(capped_blocks(std::max<long>(n4, 256), 256, 4096));
+  if (f32)
+    hipLaunchKernelGGL((gelu_erf_kernel<true>), grid, dim3(256), 0, stream, in, out, n4, n);
+  else
+    hipLaunchKernelGGL((gelu_erf_kernel<false>), grid, dim3(256), 0, stream, in, out, n4, n);
+}

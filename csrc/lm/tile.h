@@ -1,0 +1,129 @@
+// Element access and 16x16 MFMA tiles for the serving kernels, in two
+// precisions behind one interface:
+//   Num<false>  bf16 operands, float accumulation (v_mfma 16x16x32)
+//   Num<true>   float operands throughout         (v_mfma 16x16x4)
+// A fragment is 8 consecutive k-values of one row per lane in both: lane
+// l holds row l%16, k = 8*(l/16) .. +7 of a 32-wide k-block.  The float
+// form issues 8 MFMAs that walk those 8 values; every lane group then
+// contributes its own k's, and A and B use the same assignment, so the
+// sum over the block is the same set of products.
+// Accumulator layout: lane l holds rows 4*(l/16)+r (r = 0..3), col l%16.
+#pragma once
+
+#include "../device.h"
+
+DEVINL short cvt_bf16(float f) {  // RNE, one VALU op on gfx950
+  return __builtin_bit_cast(short, (__bf16)f);
+}
+
+template <bool F32> struct Num;
+
+template <> struct Num<false> {
+  using E = short;
+  using Frag = bf16x8;
+  static constexpr int PAD = 8;
+  static DEVINL float up(E v) { return bf2f(v); }
+  static DEVINL E down(float v) { return cvt_bf16(v); }
+  static DEVINL Frag load(const E* row, int k) { return *(const Frag*)(row + k); }
+  static DEVINL f32x4 mma(const Frag& a, const Frag& b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+        __builtin_bit_cast(__attribute__((ext_vector_type(8))) __bf16, a),
+        __builtin_bit_cast(__attribute__((ext_vector_type(8))) __bf16, b), c,
+        0, 0, 0);
+  }
+};
+
+template <> struct Num<true> {
+  using E = float;
+  struct Frag { float v[8]; };
+  static constexpr int PAD = 4;
+  static DEVINL float up(E v) { return v; }
+  static DEVINL E down(float v) { return v; }
+  static DEVINL Frag load(const E* row, int k) {
+    Frag f;
+    *(f32x4*)f.v = *(const f32x4*)(row + k);
+    *(f32x4*)(f.v + 4) = *(const f32x4*)(row + k + 4);
+    return f;
+  }
+  static DEVINL f32x4 mma(const Frag& a, const Frag& b, f32x4 c) {
+    #pragma unroll
+    for (int i = 0; i < 8; ++i)
+      c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.v[i], b.v[i], c, 0, 0, 0);
+    return c;
+  }
+};
+
+// 8 consecutive elements as floats; entries at or past `valid` are 0.
+// `aligned` promises 16-byte aligned rows whose lengths are multiples of 8.
+template <bool F32>
+DEVINL void load8(const typename Num<F32>::E* p, int valid, bool aligned,
+                  float* out) {
+  if (valid <= 0) {
+    #pragma unroll
+    for (int i = 0; i < 8; ++i) out[i] = 0.f;
+  } else if (aligned) {
+    if constexpr (F32) {
+      *(f32x4*)out = *(const f32x4*)p;
+      *(f32x4*)(out + 4) = *(const f32x4*)(p + 4);
+    } else {
+      const bf16x8 t = *(const bf16x8*)p;
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) out[i] = bf2f(t[i]);
+    }
+  } else {
+    #pragma unroll
+    for (int i = 0; i < 8; ++i) out[i] = i < valid ? Num<F32>::up(p[i]) : 0.f;
+  }
+}
+
+// Operand kept at (nearly) float precision in LDS.  In bf16 mode a value
+// is the sum of two bf16 (16 significand bits) and a product is three
+// MFMAs; in float mode it is the value itself.
+template <bool F32> struct Split {
+  using N = Num<F32>;
+  using E = typename N::E;
+  E* hi;
+  E* lo;
+  static constexpr int PARTS = F32 ? 1 : 2;
+  struct Frag { typename N::Frag hi, lo; };
+  DEVINL void put(int i, float v) const {
+    const E h = N::down(v);
+    hi[i] = h;
+    if constexpr (!F32) lo[i] = N::down(v - N::up(h));
+  }
+  DEVINL Frag load(int row_off, int k) const {
+    Frag f;
+    f.hi = N::load(hi + row_off, k);
+    if constexpr (!F32) f.lo = N::load(lo + row_off, k);
+    return f;
+  }
+};
+
+// split x split
+template <bool F32>
+DEVINL f32x4 mma_ss(const typename Split<F32>::Frag& a,
+                    const typename Split<F32>::Frag& b, f32x4 c) {
+  if constexpr (!F32) {
+    c = Num<F32>::mma(a.lo, b.hi, c);
+    c = Num<F32>::mma(a.hi, b.lo, c);
+  }
+  return Num<F32>::mma(a.hi, b.hi, c);
+}
+// split x plain
+template <bool F32>
+DEVINL f32x4 mma_sp(const typename Split<F32>::Frag& a,
+                    const typename Num<F32>::Frag& b, f32x4 c) {
+  if constexpr (!F32) c = Num<F32>::mma(a.lo, b, c);
+  return Num<F32>::mma(a.hi, b, c);
+}
+
+DEVINL float sum16(float v) {  // over the 16 lanes that share l/16
+  #pragma unroll
+  for (int o = 1; o < 16; o <<= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+DEVINL float max16(float v) {
+  #pragma unroll
+  for (int o = 1; o < 16; o <<= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
+  return v;
+}

@@ -25,7 +25,11 @@ SCHEMA_VERSION = 1
 
 @dataclass
 class ModelConfig:
-    name: str = "mlp"  # mlp | resnet50 | gpt2 | llama3_8b | llama (custom dims)
+    # mlp | resnet50 | gpt2 | llama3_8b | llama (custom dims) | lasezen
+    name: str = "mlp"
+    # a model folder: config.json (its "architecture" picks the name and
+    # fills the fields below) beside model.safetensors
+    dir: str = ""
     # MLP
     in_dim: int = 256
     hidden_dim: int = 512
@@ -65,6 +69,13 @@ class ModelConfig:
     # its activations (trades ~1 extra block fwd for O(1) activation
     # memory per block); LM families only, no-op in eval
     act_ckpt: bool = False
+    # mixer-stack models: one entry per layer ({"type", "mixer", "mlp"}),
+    # the span of layers that runs `times` times in a row
+    # ({"start", "stop", "times"}), and the factor of every sublayer's
+    # contribution to the residual stream
+    layers: List[Any] = field(default_factory=list)
+    loop: Optional[Dict[str, int]] = None
+    residual_mult: float = 1.0
 
 
 @dataclass
@@ -260,9 +271,34 @@ def load_config(path: Optional[str] = None, overrides: Optional[List[str]] = Non
     return cfg
 
 
+def _lasezen_fields(d: Dict[str, Any]) -> Dict[str, Any]:
+    return {"name": "lasezen", "vocab_size": d["vocab"],
+            "d_model": d["width"], "n_layers": len(d["layers"]),
+            "norm_eps": d["norm"]["eps"], "layers": d["layers"],
+            "loop": d.get("loop"), "residual_mult": d["residual_mult"]}
+
+
+# config.json "architecture" -> reader of that file's keys
+ARCHITECTURES = {"Lasezen": _lasezen_fields}
+
+
+def read_model_dir(path: str) -> Dict[str, Any]:
+    """ModelConfig fields of a model folder's config.json."""
+    with open(os.path.join(path, "config.json")) as fh:
+        d = json.load(fh)
+    arch = d.get("architecture")
+    if arch not in ARCHITECTURES:
+        raise ValueError(f"{path}: unknown architecture {arch!r} (known: "
+                         f"{', '.join(sorted(ARCHITECTURES))})")
+    return ARCHITECTURES[arch](d)
+
+
 def _apply_model_preset(cfg: TrainConfig) -> None:
     """Fill model dims for named presets unless the user overrode them."""
     m = cfg.model
+    if m.dir:
+        for k, v in read_model_dir(m.dir).items():
+            setattr(m, k, v)
     if m.name == "gpt2":
         if m.d_ff is None:
             m.d_ff = 4 * m.d_model

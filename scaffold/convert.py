@@ -26,6 +26,7 @@ import torch
 
 from .models.gpt2 import GPT2
 from .models.llama import Llama
+from .models.stack import MixerStack
 
 
 def _strip_prefix(sd: Dict[str, torch.Tensor], prefix: str) -> Dict[str, torch.Tensor]:
@@ -327,3 +328,67 @@ def to_hf_mixtral(model: Llama) -> Dict[str, torch.Tensor]:
         out[h + "mlp.experts.gate_up_proj"] = ups
         out[h + "mlp.experts.down_proj"] = downs
     return out
+
+
+# ---- mixer-stack checkpoints ------------------------------------------
+def _stack_tensors(model: MixerStack):
+    """(checkpoint name, destination, first row, rows) of every tensor of
+    a mixer-stack model; projections that share an input are one packed
+    matrix in the module and separate tensors in a checkpoint."""
+    def norm(name, mod):
+        return [(name, mod.weight, 0, mod.weight.shape[0]),
+                (name + ".b", mod.bias, 0, mod.bias.shape[0])]
+
+    out = [("embed", model.embed.weight, 0, model.embed.weight.shape[0])]
+    for i, blk in enumerate(model.blocks):
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            if hasattr(blk, n):
+                out += norm(f"l{i}.{n}", getattr(blk, n))
+        out += [(f"l{i}.mix.{n}", t, a, b) for n, t, a, b in blk.mixer.packed()]
+        if blk.ff is not None:
+            out += [(f"l{i}.mlp.{n}", t, a, b) for n, t, a, b in blk.ff.packed()]
+    out += norm("final.norm", model.norm_f)
+    out.append(("head", model.lm_head.weight, 0, model.lm_head.weight.shape[0]))
+    return out
+
+
+def load_stack(model: MixerStack, sd: Dict[str, torch.Tensor]) -> None:
+    """Copy a mixer-stack checkpoint into the model; every tensor of the
+    model must be there with its shape, and nothing else."""
+    want = _stack_tensors(model)
+    names = {n for n, *_ in want}
+    if names != set(sd):
+        raise KeyError(f"missing {sorted(names - set(sd))}, unexpected "
+                       f"{sorted(set(sd) - names)}")
+    with torch.no_grad():
+        for n, t, a, rows in want:
+            dst = t[a:a + rows]
+            if dst.shape != sd[n].shape:
+                raise ValueError(f"{n}: shape {tuple(sd[n].shape)}, expected "
+                                 f"{tuple(dst.shape)}")
+            dst.copy_(sd[n])
+
+
+def to_stack(model: MixerStack) -> Dict[str, torch.Tensor]:
+    """Inverse of load_stack."""
+    return {n: t[a:a + rows].detach().cpu().clone()
+            for n, t, a, rows in _stack_tensors(model)}
+
+
+def load_model_dir(path: str, dtype=None, device="cpu", overrides=()
+                   ) -> torch.nn.Module:
+    """Build and load the model of a folder (config.json and
+    model.safetensors); the class follows config.json."""
+    import os
+
+    import safetensors.torch as st
+
+    from .config import load_config
+    from .models import build_model
+
+    cfg = load_config(None, [f"model.dir={path}", *overrides])
+    with torch.device("meta"):
+        model = build_model(cfg)
+    model = model.to_empty(device="cpu")
+    load_stack(model, st.load_file(os.path.join(path, "model.safetensors")))
+    return model.to(device=device, dtype=dtype).eval()

@@ -6,8 +6,9 @@ attention op on GPU) while recording K/V; each decode step attends the
 single new query against the cache.  The decode GEMVs take the library
 path — the hand decode_gemv kernel measured below hipBLASLt in-graph
 and is parked behind SCAFFOLD_DECODE_GEMV=1 (NOTES r2 serving ladder).
-Both model families (GPT-2 LayerNorm/GELU, Llama RMSNorm/RoPE/GQA/
-SwiGLU); greedy / temperature / top-k / top-p sampling with optional
+Model families: GPT-2 (LayerNorm/GELU), Llama (RMSNorm/RoPE/GQA/SwiGLU)
+and mixer stacks (Lasezen), which keep a paged cache with state slots
+(scaffold.cache) and run every call as one ragged batch (step); greedy / temperature / top-k / top-p sampling with optional
 EOS; hipGraph-replayed static decode (generate_graphed); per-row
 variable-position decode for continuous batching (decode_step_varpos);
 speculative decoding (generate_speculative); TP-sharded models reduce
@@ -23,8 +24,10 @@ import torch
 import torch.nn.functional as F
 
 from . import ops
+from .cache import PagedStateCache
 from .models.gpt2 import GPT2
 from .models.llama import Llama
+from .models.stack import MixerStack
 
 
 def _sdpa(q, k, v, causal):
@@ -98,8 +101,66 @@ class Generator:
     def __init__(self, model: torch.nn.Module):
         self.m = model
         self.is_llama = isinstance(model, Llama)
-        if not (self.is_llama or isinstance(model, GPT2)):
+        self.is_stack = isinstance(model, MixerStack)
+        if not (self.is_llama or self.is_stack or isinstance(model, GPT2)):
             raise TypeError(f"Generator: unsupported model {type(model).__name__}")
+
+    # ---- caches ---------------------------------------------------------
+    @property
+    def max_len(self) -> int:
+        """Longest sequence (prompt + new tokens) the model serves."""
+        if self.is_stack:
+            return self.m.max_seq_len
+        return (self.m.rope_cos.shape[0] if self.is_llama
+                else self.m.wpe.num_embeddings)
+
+    @property
+    def tp_sharded(self) -> bool:
+        attn = getattr(self.m.blocks[0], "attn", None)
+        return getattr(attn, "_tp_world", 1) > 1
+
+    def new_cache(self, B: int, max_len: int):
+        """Cache of B rows, max_len tokens each, ready for
+        _forward_tokens / decode_step_varpos."""
+        if self.is_stack:
+            cache = self.m.new_cache(B, B * -(-max_len // 64) * 64, max_len)
+            for b in range(B):
+                cache.reserve(cache.open(b), max_len)
+            return cache
+        attn0 = self.m.blocks[0].attn
+        p = next(self.m.parameters())
+        return KVCache(len(self.m.blocks), B,
+                       attn0.n_kv if self.is_llama else attn0.n_heads,
+                       max_len, attn0.head_dim, p.device, p.dtype)
+
+    # ---- ragged batches (mixer stacks) ----------------------------------
+    @torch.no_grad()
+    def step(self, cache: PagedStateCache, entries, on_layer=None
+             ) -> torch.Tensor:
+        """One ragged batch: entries of (slot, tokens, wanted places) run
+        together, prompt portions beside single tokens.  Returns the
+        wanted logits (rows, V) in entry order and advances the slots."""
+        plan, _ = cache.plan(entries)
+        logits = self.m.forward_step(plan, cache, on_layer=on_layer)
+        cache.commit(entries)
+        return logits
+
+    @staticmethod
+    def _mark(cache):
+        """Remember where the cache (B=1) stands, for _rewind."""
+        return (cache.snapshot(0, kv=False)
+                if isinstance(cache, PagedStateCache) else None)
+
+    def _rewind(self, cache, mark, out, n: int) -> None:
+        """Step the cache back to the first n tokens of `out`.  Keys and
+        values are simply overwritten later; recurrent states return to
+        the mark and take the tokens since then once more."""
+        if mark is None:
+            cache.len = min(cache.len, n)
+        elif cache.lens[0] > n:
+            cache.restore(0, mark)
+            if n > mark["len"]:
+                self.step(cache, [(0, out[mark["len"]:n], ())])
 
     # ---- per-family block math with external KV ------------------------
     def _gpt2_block(self, blk, x, cache: KVCache, i: int, pos0: int):
@@ -162,6 +223,16 @@ class Generator:
         or (B, S, V) for every position when all_logits (the speculative
         verify pass needs the target's prediction AFTER each draft)."""
         m = self.m
+        if self.is_stack:
+            B, S = tokens.shape
+            if S == 1:          # every row's next token, ids stay on device
+                pos = torch.full((B,), cache.seq_len, device=tokens.device)
+                lg = self.decode_step_varpos(tokens, cache, pos)
+                cache.advance(range(B))
+                return lg.unsqueeze(1) if all_logits else lg
+            want = range(S) if all_logits else (S - 1,)
+            lg = self.step(cache, [(b, tokens[b], want) for b in range(B)])
+            return lg.view(B, S, -1) if all_logits else lg
         if self.is_llama:
             x = m.embed(tokens)
             for i, blk in enumerate(m.blocks):
@@ -216,13 +287,8 @@ class Generator:
         """prompt (B, S0) int64 -> (B, S0 + max_new_tokens).  With
         eos_token_id, rows freeze at EOS (subsequent positions repeat
         it) and decoding stops early once every row has finished."""
-        n_layers = len(self.m.blocks)
         B, S0 = prompt.shape
-        attn0 = self.m.blocks[0].attn
-        n_kv = attn0.n_kv if self.is_llama else attn0.n_heads
-        dtype = next(self.m.parameters()).dtype
-        cache = KVCache(n_layers, B, n_kv, S0 + max_new_tokens,
-                        attn0.head_dim, prompt.device, dtype)
+        cache = self.new_cache(B, S0 + max_new_tokens)
         out = torch.empty(B, S0 + max_new_tokens, dtype=prompt.dtype,
                           device=prompt.device)
         out[:, :S0] = prompt
@@ -330,15 +396,20 @@ class Generator:
         argmaxes, writes the token at pos_dev+1 of out_dev, advances
         cur_tok and pos_dev IN PLACE (graph-replayable)."""
         m = self.m
-        if self.is_llama:
-            x = m.embed(cur_tok)
+        if self.is_stack:
+            logits = self.decode_step_varpos(
+                cur_tok, cache, pos_dev.expand(cur_tok.shape[0]))
         else:
-            x = m.wte(cur_tok) + m.wpe(pos_dev).unsqueeze(0)
-        for i, blk in enumerate(m.blocks):
-            x = self._block_static(blk, x, cache, i, pos_dev)
-        x = (ops.rms_norm(x, m.norm_f.weight, m.norm_f.eps) if self.is_llama
-             else ops.layer_norm(x, m.ln_f.weight, m.ln_f.bias, m.ln_f.eps))
-        logits = self._lin1(x, m.lm_head.weight)[:, 0]
+            if self.is_llama:
+                x = m.embed(cur_tok)
+            else:
+                x = m.wte(cur_tok) + m.wpe(pos_dev).unsqueeze(0)
+            for i, blk in enumerate(m.blocks):
+                x = self._block_static(blk, x, cache, i, pos_dev)
+            x = (ops.rms_norm(x, m.norm_f.weight, m.norm_f.eps)
+                 if self.is_llama else
+                 ops.layer_norm(x, m.ln_f.weight, m.ln_f.bias, m.ln_f.eps))
+            logits = self._lin1(x, m.lm_head.weight)[:, 0]
         nxt = logits.argmax(dim=-1, keepdim=True)
         out_dev.scatter_(1, (pos_dev + 1).expand(nxt.shape), nxt)
         cur_tok.copy_(nxt)
@@ -363,25 +434,16 @@ class Generator:
         if prompt.shape[0] != 1:
             raise ValueError("speculative decode is B=1 (per-row "
                              "acceptance lengths diverge in a batch)")
-        if getattr(self.m.blocks[0].attn, "_tp_world", 1) > 1:
+        if self.tp_sharded:
             # a lone rank issuing the TP all_reduces would deadlock the
             # group; speculative x TP needs the command-replay protocol
             raise NotImplementedError(
                 "speculative decode over a TP-sharded target is not "
                 "supported")
-        n_layers = len(self.m.blocks)
-        attn0 = self.m.blocks[0].attn
-        n_kv = attn0.n_kv if self.is_llama else attn0.n_heads
-        dtype = next(self.m.parameters()).dtype
         S0 = prompt.shape[1]
         L = S0 + max_new_tokens + k + 1   # headroom for a rolled-back tail
-        cache = KVCache(n_layers, 1, n_kv, L, attn0.head_dim,
-                        prompt.device, dtype)
-        d_attn = draft.m.blocks[0].attn
-        d_kv = d_attn.n_kv if draft.is_llama else d_attn.n_heads
-        d_dtype = next(draft.m.parameters()).dtype
-        dcache = KVCache(len(draft.m.blocks), 1, d_kv, L, d_attn.head_dim,
-                         prompt.device, d_dtype)
+        cache = self.new_cache(1, L)
+        dcache = draft.new_cache(1, L)
 
         out = [int(t) for t in prompt[0]]
         # prefill both; the target's prefill logits give token S0
@@ -394,6 +456,7 @@ class Generator:
         while produced < max_new_tokens and not done:
             kk = min(k, max_new_tokens - produced)
             base = len(out) - 1          # index of the newest token
+            mark, dmark = self._mark(cache), draft._mark(dcache)
             # --- draft proposes kk tokens from its own cache
             dtoks = []
             cur = torch.tensor([[out[base]]], device=prompt.device)
@@ -433,8 +496,8 @@ class Generator:
             # roll back the caches past what is actually accepted: the
             # target consumed the whole window; keep entries only for
             # tokens that are now part of `out` minus the newest
-            cache.len = len(out) - 1
-            dcache.len = min(dcache.len, len(out) - 1)
+            self._rewind(cache, mark, out, len(out) - 1)
+            draft._rewind(dcache, dmark, out, len(out) - 1)
         if stats is not None:
             stats["rounds"] = rounds
             stats["accepted"] = accepted_total
@@ -523,11 +586,18 @@ class Generator:
 
     @torch.no_grad()
     def decode_step_varpos(self, cur_tok: torch.Tensor, cache: KVCache,
-                           pos: torch.Tensor) -> torch.Tensor:
+                           pos: torch.Tensor,
+                           active: Optional[torch.Tensor] = None
+                           ) -> torch.Tensor:
         """cur_tok (B, 1) int64, pos (B,) int64 (per-row position of
         cur_tok) -> next-token logits (B, V).  Writes cur_tok's kv at
-        pos[b]; caller owns sampling and position advance."""
+        pos[b]; caller owns sampling and position advance.  Rows with
+        active[b] == 0 give undefined logits; a mixer stack leaves their
+        pages and states untouched."""
         m = self.m
+        if self.is_stack:
+            return m.forward_step(cache.decode_plan(cur_tok, pos, active),
+                                  cache)
         if self.is_llama:
             x = m.embed(cur_tok)
         else:
@@ -547,20 +617,15 @@ class Generator:
         masking, argmax and position advance all run device-side
         against a device position scalar.  use_graph=False runs the
         same static-shape step eagerly (the CPU-testable path)."""
-        n_layers = len(self.m.blocks)
         B, S0 = prompt.shape
-        attn0 = self.m.blocks[0].attn
-        if getattr(attn0, "_tp_world", 1) > 1:
+        if self.tp_sharded:
             # the static step has no TP reductions — failing loudly
             # beats silently wrong tokens; TP decode runs through
             # generate() / ContinuousBatcher (both reduce)
             raise NotImplementedError(
                 "generate_graphed does not support TP-sharded models")
-        n_kv = attn0.n_kv if self.is_llama else attn0.n_heads
-        dtype = next(self.m.parameters()).dtype
         L = S0 + max_new_tokens
-        cache = KVCache(n_layers, B, n_kv, L, attn0.head_dim,
-                        prompt.device, dtype)
+        cache = self.new_cache(B, L)
         out = torch.zeros(B, L, dtype=prompt.dtype, device=prompt.device)
         out[:, :S0] = prompt
         logits = self._forward_tokens(prompt, cache, 0)   # prefill

@@ -1,4 +1,5 @@
-"""Model zoo (contract C9): MLP, ResNet-50, GPT-2-small, Llama-3-8B."""
+"""Model zoo (contract C9): MLP, ResNet-50, GPT-2-small, Llama-3-8B, and
+mixer-stack models (Lasezen)."""
 
 from __future__ import annotations
 
@@ -8,8 +9,10 @@ from .mlp import MLP
 from .resnet import ResNet50
 from .gpt2 import GPT2
 from .llama import Llama
+from .stack import MixerStack
 
-__all__ = ["MLP", "ResNet50", "GPT2", "Llama", "build_model"]
+__all__ = ["MLP", "ResNet50", "GPT2", "Llama", "MixerStack",
+           "build_model"]
 
 
 def build_model(cfg) -> torch.nn.Module:
@@ -22,4 +25,6 @@ def build_model(cfg) -> torch.nn.Module:
         return GPT2(cfg)
     if name in ("llama", "llama3_8b"):
         return Llama(cfg)
+    if name == "lasezen":
+        return MixerStack(cfg)
     raise ValueError(f"unknown model {name!r}")

@@ -17,7 +17,9 @@ import torch
 import torch.nn.functional as F
 
 from . import backend
-from .backend import require_ext, has_ext, ext  # re-export
+from .backend import require_ext, require_lm_ext, has_ext, ext  # re-export
+from .lm import (decay_tables, embed_norm, gelu_erf, paged_attention,
+                 residual_norm, retention, rope_tables_exact)
 
 __all__ = [
     "layer_norm",
@@ -33,7 +35,15 @@ __all__ = [
     "lm_head_ce",
     "fused_adamw_step",
     "batch_norm_act",
+    "embed_norm",
+    "residual_norm",
+    "gelu_erf",
+    "paged_attention",
+    "retention",
+    "decay_tables",
+    "rope_tables_exact",
     "require_ext",
+    "require_lm_ext",
     "has_ext",
 ]
 

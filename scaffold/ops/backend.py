@@ -10,16 +10,18 @@ dispatch on the GPU path; eager is the CPU test path only).
 
 from __future__ import annotations
 
+import importlib.util
 import os
 import sys
-from typing import Optional
-
-_EXT = None
-_EXT_ERROR: Optional[str] = None
+from typing import Dict, List, Optional
 
 _REPO_ROOT = os.path.dirname(os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 BUILD_DIR = os.path.join(_REPO_ROOT, "csrc", "build")
-EXT_NAME = "scaffold_hip"
+
+# one native module per workload, so a serving process never waits for
+# the training kernels to compile (and the other way round)
+EXT_NAME = "scaffold_hip"          # training ops, comm, checkpoint IO
+LM_EXT_NAME = "scaffold_lm_hip"    # mixer-stack serving kernels
 
 _SOURCES = [
     "ext.cpp",
@@ -43,71 +45,115 @@ _SOURCES = [
     "kernels/probe.hip",
 ]
 
+_LM_SOURCES = [
+    "lm/ext.cpp",
+    "lm/norm.hip",
+    "lm/attn.hip",
+    "lm/attn_decode.hip",
+    "lm/retention.hip",
+]
 
-def _source_paths():
-    return [os.path.join(_REPO_ROOT, "csrc", s) for s in _SOURCES]
+# packed-FP32 instruction selection stays off: some packed forms have
+# returned wrong results on this hardware
+_HIPCC_FLAGS = ["-O3", "-std=c++17", "--offload-arch=gfx950",
+                "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+_EXTS: Dict[str, dict] = {
+    EXT_NAME: {"dir": BUILD_DIR, "sources": _SOURCES,
+               "ldflags": ["-L/opt/rocm/lib", "-lrccl"]},
+    LM_EXT_NAME: {"dir": os.path.join(BUILD_DIR, "lm"),
+                  "sources": _LM_SOURCES, "ldflags": []},
+}
+_LOADED: Dict[str, object] = {}
+_ERRORS: Dict[str, str] = {}
 
 
-def build_extension(verbose: bool = True):
-    """Compile the HIP extension for gfx950 into csrc/build (in-tree).
+def _source_paths(sources: List[str]):
+    return [os.path.join(_REPO_ROOT, "csrc", s) for s in sources]
+
+
+def build_extension(verbose: bool = True, name: str = EXT_NAME):
+    """Compile one HIP extension for gfx950 into csrc/build (in-tree).
 
     Cross-compiles fine without a GPU (hipcc targets gfx950 regardless).
     Uses torch.utils.cpp_extension so the torch ABI/link flags are right.
     """
     os.environ.setdefault("PYTORCH_ROCM_ARCH", "gfx950")
-    os.makedirs(BUILD_DIR, exist_ok=True)
+    spec = _EXTS[name]
+    os.makedirs(spec["dir"], exist_ok=True)
     from torch.utils.cpp_extension import load
 
-    ext = load(
-        name=EXT_NAME,
-        sources=_source_paths(),
-        build_directory=BUILD_DIR,
+    return load(
+        name=name,
+        sources=_source_paths(spec["sources"]),
+        build_directory=spec["dir"],
         extra_cflags=["-O3", "-std=c++17"],
-        extra_cuda_cflags=["-O3", "-std=c++17", "--offload-arch=gfx950"],
-        extra_ldflags=["-L/opt/rocm/lib", "-lrccl"],
+        extra_cuda_cflags=list(_HIPCC_FLAGS),
+        extra_ldflags=spec["ldflags"],
         verbose=verbose,
     )
-    return ext
 
 
-def _try_load():
+def build_all(verbose: bool = True) -> None:
+    for name in _EXTS:
+        build_extension(verbose=verbose, name=name)
+
+
+def _try_load(name: str = EXT_NAME):
     """Load the prebuilt in-tree .so without invoking the compiler."""
-    global _EXT, _EXT_ERROR
-    if _EXT is not None:
-        return _EXT
-    so_path = os.path.join(BUILD_DIR, f"{EXT_NAME}.so")
+    if name in _LOADED:
+        return _LOADED[name]
+    so_path = os.path.join(_EXTS[name]["dir"], f"{name}.so")
     if not os.path.exists(so_path):
-        _EXT_ERROR = f"extension not built: {so_path} missing (run __graft_entry__.build())"
+        _ERRORS[name] = (f"extension not built: {so_path} missing "
+                         "(run __graft_entry__.build())")
         return None
     try:
-        import importlib.util
+        import torch  # noqa: F401  (the .so links against libtorch)
 
-        spec = importlib.util.spec_from_file_location(EXT_NAME, so_path)
+        spec = importlib.util.spec_from_file_location(name, so_path)
         mod = importlib.util.module_from_spec(spec)
         spec.loader.exec_module(mod)
-        sys.modules[EXT_NAME] = mod
-        _EXT = mod
-        return _EXT
+        sys.modules[name] = mod
+        _LOADED[name] = mod
+        return mod
     except Exception as e:  # noqa: BLE001
-        _EXT_ERROR = f"failed to load {so_path}: {e}"
+        _ERRORS[name] = f"failed to load {so_path}: {e}"
         return None
 
 
 def ext():
-    """The loaded extension module, or None (CPU-only environments)."""
+    """The loaded training extension, or None (CPU-only environments)."""
     return _try_load()
 
 
-def require_ext():
-    """The extension, raising loudly if unavailable — the GPU path."""
-    m = _try_load()
+def _require(name: str):
+    m = _try_load(name)
     if m is None:
         raise RuntimeError(
             "scaffold HIP extension required on GPU but not available: "
-            f"{_EXT_ERROR}. Build it with __graft_entry__.build() "
+            f"{_ERRORS.get(name)}. Build it with __graft_entry__.build() "
             "(hipcc --offload-arch=gfx950, in-tree at csrc/build)."
         )
     return m
+
+
+def require_ext():
+    """The training extension, raising loudly if unavailable — the GPU
+    path."""
+    return _require(EXT_NAME)
+
+
+def require_lm_ext():
+    """The mixer-stack serving extension, raising loudly if unavailable."""
+    return _require(LM_EXT_NAME)
+
+
+def ensure_lm_ext():
+    """require_lm_ext(), compiling it first if this checkout has none."""
+    if _try_load(LM_EXT_NAME) is None:
+        build_extension(verbose=False, name=LM_EXT_NAME)
+    return _require(LM_EXT_NAME)
 
 
 def has_ext() -> bool:

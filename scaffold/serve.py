@@ -22,7 +22,9 @@ optional SSE stream), POST /v1/completions (text, with --tokenizer),
 GET /healthz, GET /v1/stats, GET /metrics (Prometheus).
 
 Run: `python -m scaffold.serve model.name=llama3_8b [--continuous]
-[--graph] [--weights w.safetensors] [--lora a.safetensors --lora-r 8]`
+[--graph] [--weights w.safetensors] [--lora a.safetensors --lora-r 8]`,
+or `python -m scaffold.serve model.dir=FOLDER ...` for a folder with
+config.json and model.safetensors (mixer-stack designs)
 """
 
 from __future__ import annotations
@@ -133,8 +135,7 @@ class InferenceWorker:
         self.draft = Generator(draft_model.eval()) if draft_model is not None \
             else None
         self.draft_k = draft_k
-        self.max_len = (model.rope_cos.shape[0] if self.gen.is_llama
-                        else model.wpe.num_embeddings)
+        self.max_len = self.gen.max_len
         self.device = next(model.parameters()).device
         self.max_batch = max_batch
         self.window_s = window_s
@@ -270,20 +271,29 @@ class ContinuousBatcher:
     def __init__(self, model: torch.nn.Module, max_slots: int = 8,
                  max_len: int = 0, max_new_tokens_cap: int = 512,
                  seed: int = 0, use_graph: bool = False,
-                 prefix_cache_entries: int = 8, max_queue: int = 256):
+                 prefix_cache_entries: int = 8, max_queue: int = 256,
+                 cache_tokens: int = 0, prefill_chunk: int = 2048):
+        """cache_tokens / prefill_chunk apply to models with a paged
+        cache (mixer stacks): pool size in tokens (0: every slot at full
+        length; less makes admission wait for pages) and the most prompt
+        tokens one step takes, shared by the prompts being read."""
         self.max_queue = max_queue
         self.gen = Generator(model.eval())
         self.device = next(model.parameters()).device
         m = model
         self.is_llama = self.gen.is_llama
-        attn0 = m.blocks[0].attn
-        self.n_kv = attn0.n_kv if self.is_llama else attn0.n_heads
-        self.head_dim = attn0.head_dim
+        self.paged = self.gen.is_stack
         self.n_layers = len(m.blocks)
+        if not self.paged:
+            attn0 = m.blocks[0].attn
+            self.n_kv = attn0.n_kv if self.is_llama else attn0.n_heads
+            self.head_dim = attn0.head_dim
         if not max_len:
-            max_len = (m.rope_cos.shape[0] if self.is_llama
-                       else m.wpe.num_embeddings)
+            max_len = self.gen.max_len
         self.max_len = max_len
+        self.prefill_chunk = max(1, int(prefill_chunk))
+        self.cache_tokens = (int(cache_tokens)
+                             or max_slots * -(-max_len // 64) * 64)
         self.max_slots = max_slots
         self.max_new_tokens_cap = max_new_tokens_cap
         self.dtype = next(m.parameters()).dtype
@@ -343,6 +353,10 @@ class ContinuousBatcher:
             raise ValueError(
                 f"prompt+max_new_tokens {len(tokens) + n} exceeds "
                 f"max_len {self.max_len}")
+        if self.paged and len(tokens) + n > self.cache_tokens:
+            raise ValueError(
+                f"prompt+max_new_tokens {len(tokens) + n} exceeds the "
+                f"cache pool ({self.cache_tokens} tokens)")
         req = _Request(torch.tensor(tokens, dtype=torch.int64), n,
                        float(temperature), int(top_k), float(top_p),
                        eos_token_id, t_submit=time.time(),
@@ -365,7 +379,10 @@ class ContinuousBatcher:
 
     # worker side ------------------------------------------------------
     def _ensure_cache(self):
-        if self._cache is None:
+        if self._cache is None and self.paged:
+            self._cache = self.gen.m.new_cache(
+                self.max_slots, self.cache_tokens, self.max_len)
+        elif self._cache is None:
             from .generate import KVCache
             self._cache = KVCache(self.n_layers, self.max_slots, self.n_kv,
                                   self.max_len, self.head_dim, self.device,
@@ -393,6 +410,9 @@ class ContinuousBatcher:
     def _admit(self, slot: int, req: _Request):
         """Prefill the request and install it in `slot`; a cached
         prefix of the prompt skips its share of the prefill."""
+        if self.paged:
+            self._admit_paged(slot, req)
+            return
         from .generate import KVCache
 
         prompt = req.tokens.view(1, -1).to(self.device)
@@ -440,8 +460,104 @@ class ContinuousBatcher:
         self._toks[slot, 0].copy_(first[0, 0])
         self._slots[slot] = {"req": req, "count": 1, "pos": S0}
 
+    # paged models: admission takes the pages, the steps read the prompt
+    def _fits(self, req: _Request) -> bool:
+        """Whether the pool has pages for the whole request now.  (Every
+        admitted request holds all the pages it will ever need, so a
+        running one never stops for want of a page.)"""
+        if not self.paged:
+            return True
+        self._ensure_cache()
+        n = self._cache.pages_for(int(req.tokens.numel())
+                                  + req.max_new_tokens)
+        return n * 64 <= self._cache.free_tokens
+
+    def _admit_paged(self, slot: int, req: _Request):
+        c = self._cache
+        c.open(slot)
+        try:
+            c.reserve(slot, int(req.tokens.numel()) + req.max_new_tokens)
+        except Exception:
+            c.close(slot)
+            raise
+        toks = tuple(req.tokens.tolist())
+        st = {"req": req, "count": 0, "pos": 0, "toks": toks,
+              "todo": list(toks)}
+        hit = self._prefix_lookup(toks)
+        if hit is not None:
+            snap = self._prefix_cache[hit]
+            c.restore(slot, snap)
+            st["pos"] = len(hit)
+            st["todo"] = st["todo"][len(hit):]
+            self.stats["prefix_hits"] = self.stats.get("prefix_hits", 0) + 1
+            self.stats["prefix_tokens_reused"] = (
+                self.stats.get("prefix_tokens_reused", 0) + len(hit))
+        self._slots[slot] = st
+        if not st["todo"]:                 # the whole prompt was cached
+            self._first_token(slot, snap["logits"])
+
+    def _first_token(self, slot: int, logits: torch.Tensor):
+        """The prompt is read; logits (1, V) are its last position's."""
+        st = self._slots[slot]
+        r = st["req"]
+        if self._prefix_entries and st["toks"] not in self._prefix_cache:
+            snap = self._cache.snapshot(slot)
+            snap["logits"] = logits.clone()
+            self._prefix_store(st["toks"], snap)
+        first = Generator._sample(logits, r.temperature, r.top_k, r.top_p,
+                                  self._sample_gen)
+        self._cur[slot].copy_(first[0])
+        self._toks[slot, 0].copy_(first[0, 0])
+        st["count"] = 1
+
+    @torch.no_grad()
+    def _mixed_step(self):
+        """One ragged step: the next portion of every prompt that is
+        still being read, beside one token of every decoding slot."""
+        budget = self.prefill_chunk
+        entries, decoding, reading = [], [], []
+        for b, st in enumerate(self._slots):
+            if st is None:
+                continue
+            if not st["todo"]:
+                entries.append((b, self._cur[b], (0,)))
+                decoding.append(b)
+            elif budget > 0:
+                n = min(budget, len(st["todo"]))
+                done = n == len(st["todo"])
+                entries.append((b, st["todo"][:n], (n - 1,) if done else ()))
+                reading.append((b, n, done))
+                budget -= n
+        logits = self.gen.step(self._cache, entries)
+        self.stats["steps"] += 1
+        row = 0
+        at = {}
+        for b, _, want in entries:
+            if want:
+                at[b] = row
+                row += 1
+        for b in decoding:
+            st = self._slots[b]
+            r = st["req"]
+            nxt = Generator._sample(logits[at[b]:at[b] + 1], r.temperature,
+                                    r.top_k, r.top_p, self._sample_gen)
+            self._cur[b].copy_(nxt[0])
+            self._toks[b, st["count"]].copy_(nxt[0, 0])
+        self._advance_host(decoding)
+        for b, n, done in reading:
+            st = self._slots[b]
+            st["todo"] = st["todo"][n:]
+            st["pos"] += n
+            if done:
+                self._first_token(b, logits[at[b]:at[b] + 1])
+                if st["count"] >= st["req"].max_new_tokens:
+                    self._flush_stream(b, st, final=True)
+                    self._finish(b)
+
     def _finish(self, slot: int):
         st = self._slots[slot]
+        if self.paged:
+            self._cache.close(slot)
         # the one host sync of a request's lifetime; EOS is trimmed at
         # harvest (the slot runs to max_new_tokens — early slot freeing
         # would need a per-step device read, defeating the sync-free
@@ -464,11 +580,13 @@ class ContinuousBatcher:
         if hi is None:
             hi = self.max_slots
             cache = self._cache
+        elif self.paged:
+            cache = self._cache
         else:
             cache = self._SlicedCache(self._cache, hi)
         cur, pos = self._cur[:hi], self._pos[:hi]
         count, act1 = self._count[:hi], self._active[:hi]
-        logits = self.gen.decode_step_varpos(cur, cache, pos)
+        logits = self.gen.decode_step_varpos(cur, cache, pos, active=act1)
         nxt = logits.argmax(dim=-1, keepdim=True)
         new = torch.where(act1.unsqueeze(1).bool(), nxt, cur)
         cur.copy_(new)
@@ -518,9 +636,9 @@ class ContinuousBatcher:
             r.stream.put(None)
             st["stream_done"] = True
 
-    def _advance_host(self):
+    def _advance_host(self, slots=None):
         for b, st in enumerate(self._slots):
-            if st is None:
+            if st is None or (slots is not None and b not in slots):
                 continue
             st["pos"] += 1
             st["count"] += 1
@@ -549,8 +667,13 @@ class ContinuousBatcher:
         pool costs half a step, not a full one); the graphed step keeps
         the full static width so ONE capture serves every occupancy."""
         active = [b for b, st in enumerate(self._slots) if st is not None]
+        if self.paged and any(self._slots[b]["todo"] for b in active):
+            self._mixed_step()
+            return
         greedy = all(self._slots[b]["req"].temperature <= 0 for b in active)
         self._upload_state()
+        if self.paged:
+            self._cache.advance(active)
         if greedy and self.use_graph and self.device.type == "cuda":
             self._graphed_step()
             self.stats["steps"] += 1
@@ -564,8 +687,9 @@ class ContinuousBatcher:
             return
         # sampled path (per-request temperature/top_k/top_p): eager
         logits = self.gen.decode_step_varpos(
-            self._cur[:hi], self._SlicedCache(self._cache, hi),
-            self._pos[:hi])
+            self._cur[:hi],
+            self._cache if self.paged else self._SlicedCache(self._cache, hi),
+            self._pos[:hi], active=self._active[:hi])
         self.stats["steps"] += 1
         nxt = self._cur[:hi].clone()
         for b in active:
@@ -587,7 +711,7 @@ class ContinuousBatcher:
         buffers that _upload_state refreshes.  TP-sharded models fall
         back to the eager step: capturing the in-step all_reduces is
         unvalidated on RCCL."""
-        if getattr(self.gen.m.blocks[0].attn, "_tp_world", 1) > 1:
+        if self.gen.tp_sharded:
             self._step_static()
             return
         if self._graph is None:
@@ -638,6 +762,10 @@ class ContinuousBatcher:
                 pending = []
                 for b in range(self.max_slots):
                     if self._slots[b] is None and self._q:
+                        if pending and self.paged:
+                            break      # one at a time: each takes pages
+                        if not self._fits(self._q[0]):
+                            break      # wait for a request to end
                         pending.append((b, self._q.popleft()))
             try:
                 self._ensure_cache()
@@ -660,6 +788,8 @@ class ContinuousBatcher:
                         st["req"].error = e
                         if st["req"].stream is not None:
                             st["req"].stream.put(None)
+                        if self.paged:
+                            self._cache.close(b)
                         st["req"].event.set()
                         self._slots[b] = None
 
@@ -862,7 +992,7 @@ def main(argv=None):
     ap.add_argument("--weights", default="",
                     help="initial weights: safetensors file, int8 "
                          "quantized export, or HF-layout directory "
-                         "(default: random init)")
+                         "(default: those of model.dir, else random init)")
     ap.add_argument("--lora", default="",
                     help="LoRA adapter state to merge into the weights "
                          "(requires --lora-r to rebuild the adapters)")
@@ -882,10 +1012,11 @@ def main(argv=None):
     dev = "cuda" if torch.cuda.is_available() else "cpu"
     dt = torch.bfloat16 if dev == "cuda" else torch.float32
     model = build_model(cfg)
-    if args.weights:
+    weights = args.weights or cfg.model.dir
+    if weights:
         from .trainer import Trainer
 
-        Trainer._load_init_weights(model, args.weights)
+        Trainer._load_init_weights(model, weights)
     if args.lora:
         import safetensors.torch as _st
 

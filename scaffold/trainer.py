@@ -138,7 +138,15 @@ class Trainer:
         from . import convert
 
         if _os.path.isdir(path):
-            convert.load_hf_dir(model, path)
+            from .models import MixerStack
+
+            if isinstance(model, MixerStack):
+                import safetensors.torch as _st
+
+                convert.load_stack(model, _st.load_file(
+                    _os.path.join(path, "model.safetensors")))
+            else:
+                convert.load_hf_dir(model, path)
             return
         from safetensors import safe_open
 
