@@ -123,7 +123,12 @@ def main() -> int:
     ap.add_argument("--steps", type=int, default=100)
     ap.add_argument("--warmup", type=int, default=20)
     ap.add_argument("--model", type=str, default="resnet50",
-                    choices=["resnet50", "gpt2", "llama3_8b", "mlp"])
+                    choices=["resnet50", "gpt2", "llama3_8b", "mlp",
+                             "lasezen"],
+                    help="lasezen: serving throughput (prefill, decode) "
+                         "beside llama at equal size, one JSON line each")
+    ap.add_argument("--sizes", type=str, default="",
+                    help="lasezen: comma-separated sizes (default all)")
     ap.add_argument("--batch-size", type=int, default=0, help="per-rank; 0=config default")
     ap.add_argument("--bucket-mb", type=float, default=0.0, help="bucket override")
     ap.add_argument("--sweep-buckets", type=str, default="",
@@ -131,6 +136,13 @@ def main() -> int:
     ap.add_argument("--config", type=str, default="")
     ap.add_argument("overrides", nargs="*", help="section.key=value overrides")
     args = ap.parse_args()
+
+    if args.model == "lasezen":
+        from benchmarks import stack_bench
+
+        stack_bench.run(args.steps, args.warmup,
+                        sizes=[x for x in args.sizes.split(",") if x])
+        return 0
 
     cfg_file = args.config or {
         "resnet50": "configs/resnet50.json",

@@ -304,7 +304,14 @@ torch::Tensor rope_apply(torch::Tensor x, torch::Tensor cos_t, torch::Tensor sin
   const int H = (int)x.size(1);
   const int S = (int)x.size(2);
   const int D = (int)x.size(3);
-  TORCH_CHECK(cos_t.size(0) >= S && cos_t.size(1) == D / 2, "rope table shape");
+  for (const auto& t : {cos_t, sin_t}) {
+    // a table left on the host would be read through a bad device address
+    TORCH_CHECK(t.is_cuda() && t.is_contiguous() &&
+                    t.scalar_type() == torch::kFloat32,
+                "rope tables must be contiguous float32 on the GPU");
+    TORCH_CHECK(t.dim() == 2 && t.size(0) >= S && t.size(1) == D / 2,
+                "rope table shape");
+  }
   auto xc = x.stride(3) == 1 ? x : x.contiguous();
   // output in (B,S,H,D) physical layout: feeds the strided attention path
   // and the un-transpose view backward without copies
