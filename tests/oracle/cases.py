@@ -1,0 +1,140 @@
+"""Small random Lasezen models and plans for the tests."""
+
+import random
+
+import torch
+
+from scaffold.cache import PagedStateCache, StateSpec, KVSpec
+from scaffold.config import load_config, read_model_dir
+from scaffold.convert import load_stack
+from scaffold.models import build_model
+
+
+def attn(heads=4, kv=2, dim=16, vdim=16, size=24, scale=0.3, ff=40):
+    return {"type": "attention",
+            "mixer": {"heads": heads, "kv_heads": kv, "dim": dim,
+                      "vdim": vdim, "mask": {"size": size}, "scale": scale},
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def ret(heads=3, dim=16, vdim=24, rot=16, base=1000.0, decay=None, ff=40):
+    return {"type": "retention",
+            "mixer": {"heads": heads, "dim": dim, "vdim": vdim,
+                      "rot": {"dims": rot, "base": base},
+                      "decay": decay or [0.98, 0.9, 0.999, 0.7][:heads]},
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def config(layers, width=32, vocab=61, loop=None, mult=0.5, eps=1e-5):
+    return {"architecture": "Lasezen", "layers": layers, "width": width,
+            "vocab": vocab, "norm": {"eps": eps}, "residual_mult": mult,
+            "loop": loop or {"start": 0, "stop": len(layers), "times": 1}}
+
+
+# name -> configuration; each makes some part matter that others leave idle
+CONFIGS = {
+    "plain": config([ret(), attn()]),
+    "looped": config([attn(size=17, ff=None), ret(ff=None), attn(kv=1),
+                      ret(heads=1, dim=12, vdim=8, rot=6, decay=[0.95])],
+                     loop={"start": 1, "stop": 3, "times": 3}, mult=0.8),
+    "odd": config([ret(heads=2, dim=10, vdim=7, rot=4, base=50.0),
+                   attn(heads=3, kv=3, dim=9, vdim=5, size=5, ff=21)],
+                  width=27, vocab=33, eps=0.05),
+    "wide": config([attn(heads=6, kv=2, dim=72, vdim=136, size=100),
+                    ret(heads=2, dim=72, vdim=136, rot=64)],
+                   width=48, mult=1.0),
+    "ones": config([attn(heads=1, kv=1, dim=32, vdim=32, size=1, scale=1.0),
+                    ret(heads=1, dim=32, vdim=32, rot=2, decay=[1.0]),
+                    attn(heads=2, kv=1, size=4096, scale=0.2)], mult=1.0),
+}
+
+
+def weights(cfg, seed=0):
+    """Random checkpoint (bfloat16-representable float32 tensors), scaled
+    so that scores, sinks and norms are far from trivial."""
+    g = torch.Generator().manual_seed(seed)
+    W, V = cfg["width"], cfg["vocab"]
+    w = {}
+
+    def mat(name, out, inp, gain=1.0):
+        w[name] = torch.randn(out, inp, generator=g) * gain * inp ** -0.5
+
+    def vec(name, n, around=1.0, spread=0.4):
+        w[name] = around + spread * torch.randn(n, generator=g)
+
+    def norm(name):
+        vec(name, W)
+        vec(name + ".b", W, 0.0, 0.3)
+
+    w["embed"] = torch.randn(V, W, generator=g)
+    for i, L in enumerate(cfg["layers"]):
+        p, mx = f"l{i}.", L["mixer"]
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if L["mlp"] else ()):
+            norm(p + n)
+        H, d, e = mx["heads"], mx["dim"], mx["vdim"]
+        if L["type"] == "attention":
+            G = mx["kv_heads"]
+            mat(p + "mix.q", H * d, W)
+            mat(p + "mix.k", G * d, W)
+            mat(p + "mix.v", G * e, W)
+            vec(p + "mix.q.norm", d, 1.5)
+            vec(p + "mix.k.norm", d, 1.5)
+            vec(p + "mix.sink", H, 1.0, 1.0)
+        else:
+            mat(p + "mix.q", H * d, W)
+            mat(p + "mix.k", H * d, W)
+            mat(p + "mix.v", H * e, W)
+            mat(p + "mix.g", H * e, W, 2.0)
+        mat(p + "mix.o", W, H * e)
+        if L["mlp"]:
+            mat(p + "mlp.up", L["mlp"]["ff"], W, 1.5)
+            mat(p + "mlp.down", W, L["mlp"]["ff"])
+    norm("final.norm")
+    mat("head", V, W, 2.0)
+    return {k: v.bfloat16().float() for k, v in w.items()}
+
+
+def build(cfg, w, device="cpu", dtype=torch.float32, max_len=512):
+    from scaffold import config as C
+
+    tc = load_config(None, [f"model.max_seq_len={max_len}"])
+    for k, v in C.ARCHITECTURES[cfg["architecture"]](cfg).items():
+        setattr(tc.model, k, v)
+    m = build_model(tc)
+    load_stack(m, w)
+    return m.to(device, dtype).eval()
+
+
+def tokens(cfg, n, seed=1):
+    r = random.Random(seed)
+    return [r.randrange(cfg["vocab"]) for _ in range(n)]
+
+
+def poison(cache):
+    """Fill every page and state with NaN: whatever is read before it is
+    written shows in the result."""
+    for t in cache.k + cache.v + cache.state:
+        if t is not None:
+            t.fill_(float("nan"))
+    return cache
+
+
+def op_cache(spec, device, dtype, slots=3, n_tokens=1024, max_len=1024):
+    return poison(PagedStateCache([spec], slots, n_tokens, max_len, device,
+                                  dtype))
+
+
+def cuts(n, sizes):
+    """Portion lengths covering n tokens, cycling through `sizes`."""
+    out, i = [], 0
+    while n > 0:
+        c = min(n, sizes[i % len(sizes)])
+        out.append(c)
+        n -= c
+        i += 1
+    return out
+
+
+__all__ = ["attn", "ret", "config", "CONFIGS", "weights", "build", "tokens",
+           "poison", "op_cache", "cuts", "KVSpec", "StateSpec",
+           "read_model_dir"]

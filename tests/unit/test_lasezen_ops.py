@@ -1,0 +1,276 @@
+"""Each mechanism of the Lasezen design against the plain oracle: the
+float32 forms on the CPU, the HIP kernels (float32 and bfloat16) on the
+GPU.  Caches start full of NaN, and a sequence is fed in several cuts."""
+
+import pytest
+import torch
+
+from scaffold import ops
+from tests.oracle import lasezen as L
+from tests.oracle.cases import KVSpec, StateSpec, cuts, op_cache
+
+gpu = pytest.mark.gpu
+PLACES = [pytest.param("cpu", torch.float32, id="cpu"),
+          pytest.param("cuda", torch.float32, id="gpu-f32", marks=gpu),
+          pytest.param("cuda", torch.bfloat16, id="gpu-bf16", marks=gpu)]
+place = pytest.mark.parametrize("dev,dt", PLACES)
+TOL = {torch.float32: 2e-5, torch.bfloat16: 2e-2}
+
+
+def rnd(*shape, seed=0, scale=1.0):
+    g = torch.Generator().manual_seed(seed)
+    return (torch.randn(*shape, generator=g) * scale).bfloat16().double()
+
+
+def close(got, want, dt, extra=1.0):
+    got = got.double().cpu()
+    assert torch.isfinite(got).all()
+    scale = want.abs().max().clamp_min(1.0)
+    err = ((got - want).abs().max() / scale).item()
+    assert err < TOL[dt] * extra, err
+
+
+# ------------------------------------------------------------------ norms
+@place
+@pytest.mark.parametrize("W", [8, 37, 256, 300, 1030, 2048, 4100])
+def test_residual_norm(dev, dt, W):
+    T, eps, mult = 7, 0.03, 0.7
+    x, y = rnd(T, W, seed=1, scale=3), rnd(T, W, seed=2)
+    pw, pb, nw, nb = (rnd(W, seed=s) for s in (3, 4, 5, 6))
+    to = lambda t: t.to(dev, dt)
+    xs = x.float().to(dev)
+    h = ops.residual_norm(xs, to(y), (to(pw), to(pb)), mult,
+                          (to(nw), to(nb)), eps)
+    x2 = x + mult * L.layer_norm(y, pw, pb, eps)
+    assert xs.dtype == torch.float32
+    close(xs, x2, torch.float32)          # the stream itself stays float32
+    close(h, L.layer_norm(x2, nw, nb, eps), dt)
+    # a row subset leaves the stream as it is
+    rows = torch.tensor([6, 0, 3], dtype=torch.int32, device=dev)
+    xs = x.float().to(dev)
+    h = ops.residual_norm(xs, to(y), None, mult, (to(nw), to(nb)), eps,
+                          rows=rows, store_x=False)
+    close(xs, x, torch.float32)
+    close(h, L.layer_norm(x + mult * y, nw, nb, eps)[[6, 0, 3]], dt)
+
+
+@place
+def test_embed_norm_and_gelu(dev, dt):
+    e, w, b = rnd(11, 52), rnd(52, seed=1), rnd(52, seed=2)
+    tok = torch.tensor([3, 10, 0, 3], device=dev)
+    x, h = ops.embed_norm(tok, e.to(dev, dt), w.to(dev, dt), b.to(dev, dt),
+                          1e-5)
+    close(x, e[tok.cpu()], torch.float32)
+    close(h, L.layer_norm(e[tok.cpu()], w, b, 1e-5), dt)
+    for n in (1, 5, 64, 1003):
+        z = rnd(n, scale=2.5)
+        close(ops.gelu_erf(z.to(dev, dt)), L.gelu(z), dt)
+
+
+# -------------------------------------------------------------- attention
+def run_attention(dev, dt, q, k, v, *, scale, size, sink, parts, qw=None,
+                  kw=None, eps=1e-6, cache=None, slot=None):
+    T, H, d = q.shape
+    G, e = k.shape[1], v.shape[2]
+    cache = cache or op_cache(KVSpec(G, d, e), dev, dt)
+    slot = cache.open() if slot is None else slot
+    qkv = torch.cat([t.reshape(T, -1) for t in (q, k, v)], 1).to(dev, dt)
+    outs, at = [], 0
+    for n in parts:
+        ent = [(slot, [0] * n, ())]
+        plan, _ = cache.plan(ent)
+        outs.append(ops.paged_attention(
+            qkv[at:at + n].contiguous(), cache, 0, plan, heads=H,
+            q_norm=None if qw is None else qw.to(dev, dt),
+            k_norm=None if kw is None else kw.to(dev, dt),
+            sink=None if sink is None else sink.to(dev, dt),
+            size=size, scale=scale, eps=eps))
+        cache.commit(ent)
+        at += n
+    assert at == T
+    return torch.cat(outs).view(T, H, e)
+
+
+SHAPES = [  # heads, kv, dim, vdim, chunk
+    (4, 2, 16, 24, 10), (3, 3, 9, 5, 7), (8, 2, 128, 96, 100),
+    (2, 1, 256, 200, 33), (12, 2, 64, 64, 64), (5, 1, 40, 72, 65),
+    (4, 4, 32, 32, 1), (2, 2, 64, 128, 0), (7, 1, 128, 128, 48)]
+
+
+@place
+@pytest.mark.parametrize("shape", SHAPES, ids=str)
+@pytest.mark.parametrize("parts", ["whole", "tokens", "portions"])
+def test_attention(dev, dt, shape, parts):
+    H, G, d, e, size = shape
+    T = 131 if parts != "tokens" else 70
+    q, k, v = rnd(T, H, d, seed=1), rnd(T, G, d, seed=2), rnd(T, G, e, seed=3)
+    qw, kw = rnd(d, seed=4) + 1, rnd(d, seed=5) + 1
+    sink = rnd(H, seed=6, scale=2)
+    cut = {"whole": [T], "tokens": [1] * T,
+           "portions": cuts(T, [2, 3, 61, 1, 64, 17])}[parts]
+    got = run_attention(dev, dt, q, k, v, scale=0.2, size=size, sink=sink,
+                        parts=cut, qw=qw, kw=kw, eps=0.01)
+    qn, kn = L.rms(q, 0.01, qw), L.rms(k, 0.01, kw)
+    want = L.sink_attention(qn, kn, v, 0.2, size, sink)
+    close(got, want, dt, extra=2.0)
+
+
+@place
+@pytest.mark.parametrize("size", [50, 64, 129])
+def test_attention_standout_key_at_chunk_edges(dev, dt, size):
+    """One key matches the query far better than all others; it counts
+    exactly when it is in the query's chunk, decoded or in a prompt."""
+    T, H, d, e = 300, 2, 32, 16
+    start = (T - 1) // size * size
+    for where in (start - 1, start, start + 1, T - 2, 0):
+        q, k = rnd(T, H, d, seed=1, scale=0.1), rnd(T, 1, d, seed=2, scale=0.1)
+        v = rnd(T, 1, e, seed=3)
+        k[where, 0] = 0
+        k[where, 0, 3] = 8.0
+        q[-1, :, 3] = 8.0
+        want = L.sink_attention(q[-1:], k[-1:], v[-1:], 0.25, 0, None)  # shape
+        scores = torch.stack([(q[-1] * k[j, 0]).sum(-1) * 0.25
+                              for j in range(start, T)])
+        want = (torch.softmax(scores, 0).T @ v[start:, 0])[None]
+        if where >= start:
+            assert (want[0] - v[where, 0]).abs().max() < 1e-3
+        else:
+            assert (want[0] - v[where, 0]).abs().max() > 0.1
+        for parts in ([T], [T - 1, 1], [T - 2, 2]):
+            got = run_attention(dev, dt, q, k, v, scale=0.25, size=size,
+                                sink=None, parts=parts)[-1:]
+            close(got, want, dt)
+
+
+@place
+def test_sink_takes_its_share(dev, dt):
+    """A sink far above the scores drains the output, one far below
+    changes nothing, and it differs by head."""
+    T, d = 20, 16
+    q, k, v = rnd(T, 3, d, seed=1), rnd(T, 3, d, seed=2), rnd(T, 3, d, seed=3)
+    sink = torch.tensor([30.0, -30.0, 1.0], dtype=torch.float64)
+    for parts in ([T], [1] * T):
+        got = run_attention(dev, dt, q, k, v, scale=0.25, size=8, sink=sink,
+                            parts=parts)
+        assert got[:, 0].abs().max() < 1e-3
+        close(got, L.sink_attention(q, k, v, 0.25, 8, sink), dt)
+        none = L.sink_attention(q, k, v, 0.25, 8, None)
+        close(got[:, 1], none[:, 1], dt)
+        assert (got[:, 2].double().cpu() - none[:, 2]).abs().max() > 0.05
+
+
+@place
+def test_attention_many_keys_split(dev, dt):
+    """Long chunks: a decoded token's keys are split over blocks."""
+    T, H, d = 700, 4, 64
+    q, k, v = rnd(T, H, d, seed=1), rnd(T, 2, d, seed=2), rnd(T, 2, d, seed=3)
+    sink = rnd(H, seed=4)
+    got = run_attention(dev, dt, q, k, v, scale=0.3, size=690, sink=sink,
+                        parts=[600] + [1] * 100)
+    last = list(range(680, 700))
+    want = torch.zeros(len(last), H, d, dtype=torch.float64)
+    for n, i in enumerate(last):
+        lo = i // 690 * 690
+        for h in range(H):
+            s = torch.cat([k[lo:i + 1, h // 2] @ q[i, h] * 0.3, sink[h:h + 1]])
+            want[n, h] = torch.softmax(s, 0)[:-1] @ v[lo:i + 1, h // 2]
+    close(got[last], want, dt)
+
+
+# -------------------------------------------------------------- retention
+def run_retention(dev, dt, q, k, v, g, decay, rot, base, parts, eps=1e-5):
+    T, H, dk = q.shape
+    dv = v.shape[2]
+    cache = op_cache(StateSpec(H, dk, dv), dev, dt)
+    slot = cache.open()
+    pows, dec = ops.decay_tables(decay, 64, dev)
+    x = torch.cat([t.reshape(T, -1) for t in (q, k, v, g)], 1).to(dev, dt)
+    outs, at = [], 0
+    for n in parts:
+        ent = [(slot, [0] * n, ())]
+        plan, _ = cache.plan(ent)
+        outs.append(ops.retention(
+            x[at:at + n].contiguous(), cache, 0, plan, pows=pows, dec=dec,
+            rope=cache.rope(base, rot) if rot else None, kscale=dk ** -0.5,
+            eps=eps))
+        cache.commit(ent)
+        at += n
+    return torch.cat(outs).view(T, H, dv), cache.state[0][slot]
+
+
+RSHAPES = [  # heads, dim, vdim, rotated
+    (2, 32, 32, 32), (3, 16, 24, 8), (2, 20, 12, 6), (4, 64, 128, 64),
+    (1, 128, 64, 96), (2, 256, 192, 0), (3, 9, 7, 2), (2, 128, 256, 128)]
+
+
+@place
+@pytest.mark.parametrize("shape", RSHAPES, ids=str)
+@pytest.mark.parametrize("parts", ["whole", "tokens", "portions"])
+def test_retention(dev, dt, shape, parts):
+    H, dk, dv, rot = shape
+    T = 150 if parts != "tokens" else 66
+    q, k = rnd(T, H, dk, seed=1), rnd(T, H, dk, seed=2)
+    v, g = rnd(T, H, dv, seed=3), rnd(T, H, dv, seed=4)
+    decay = [0.999, 0.9, 1.0, 0.5][:H]
+    cut = {"whole": [T], "tokens": [1] * T,
+           "portions": cuts(T, [2, 1, 63, 64, 5, 1, 130])}[parts]
+    got, S = run_retention(dev, dt, q, k, v, g, decay, rot, 100.0, cut)
+    qr, kr = q.clone(), k.clone()
+    if rot:
+        for t in range(T):
+            for h in range(H):
+                qr[t, h] = L.rotate_half(q[t, h], t, 100.0, rot)
+                kr[t, h] = L.rotate_half(k[t, h], t, 100.0, rot)
+    o, want_S = L.retention_core(qr, kr * dk ** -0.5, v, decay)
+    want = L.rms(o, 1e-5) * (g / (1 + torch.exp(-g)))
+    close(got, want, dt, extra=4.0)
+    # the state is float32 whatever the activations are
+    close(S.transpose(1, 2), want_S, torch.float32, extra=2.0)
+
+
+@place
+def test_retention_remembers_a_far_token(dev, dt):
+    """With decay 1 and everything else silent, the last query reads the
+    value stored 200 tokens ago."""
+    T, d = 220, 32
+    z = torch.zeros(T, 1, d, dtype=torch.float64)
+    q, k, v = z.clone(), z.clone(), z.clone()
+    k[5, 0, 7] = 2.0
+    v[5, 0] = rnd(d, seed=3)
+    v[6:, 0] = 1.0
+    q[-1, 0, 7] = 2.0
+    g = torch.ones_like(z)
+    o = v[5, 0] * (4.0 * d ** -0.5)
+    want = o / torch.sqrt((o * o).mean() + 1e-5) * torch.sigmoid(g[0, 0])
+    for parts in ([T], [T - 1, 1], [100, 118, 2]):
+        got, _ = run_retention(dev, dt, q, k, v, g, [1.0], 0, 1.0, parts)
+        close(got[-1, 0], want, dt)
+
+
+def test_rope_table_is_exact_at_far_positions():
+    c, s = ops.rope_tables_exact(100_001, 8, 10000.0, "cpu")
+    import math
+    for p in (1, 99_999, 100_000):
+        for i in range(4):
+            a = p * 10000.0 ** (-2.0 * i / 8)
+            assert abs(c[p, i].item() - math.cos(a)) < 1e-6
+            assert abs(s[p, i].item() - math.sin(a)) < 1e-6
+
+
+@gpu
+def test_binding_rejects_bad_operands():
+    """What the kernels assume is checked on the host."""
+    m = ops.require_lm_ext()
+    x = torch.zeros(4, 32, device="cuda")
+    w = torch.ones(32, device="cuda")
+    with pytest.raises(RuntimeError):
+        m.residual_norm(x, None, None, None, 1.0, w[:31].contiguous(), None,
+                        None, 1e-5, True)
+    with pytest.raises(RuntimeError):
+        m.gelu_erf(torch.zeros(4))
+    cache = op_cache(KVSpec(2, 16, 16), "cuda", torch.float32)
+    plan, _ = cache.plan([(cache.open(), [0] * 4, ())])
+    with pytest.raises(RuntimeError):
+        ops.paged_attention(torch.zeros(4, 95, device="cuda"), cache, 0, plan,
+                            heads=2, q_norm=None, k_norm=None, sink=None,
+                            size=8, scale=1.0, eps=1e-5)
