@@ -20,56 +20,52 @@ namespace {
 
 constexpr float LOG2E = 1.4426950408889634f;
 
-// One wave per (row, head) vector: RMS norm over `dim` for q heads (in
-// place) and k heads (into the cache), plain copy for v heads.
-template <bool F32>
+// One lane group (LPV lanes, 8 elements each) per (row, head) vector: RMS
+// norm over `dim` for q heads (in place) and k heads (into the cache),
+// plain copy for v heads.
+template <bool F32, int LPV>
 __global__ void __launch_bounds__(256)
 attn_prep_kernel(AttnArgs a, const int* __restrict__ pos,
                  const int* __restrict__ slot, int row0, int n) {
   using N = Num<F32>;
   using E = typename N::E;
   const int heads = a.H + 2 * a.G;
-  const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const long unit = ((long)blockIdx.x * 256 + threadIdx.x) / LPV;
   if (unit >= (long)n * heads) return;
-  const int l = threadIdx.x & 63;
+  const int c = (threadIdx.x % LPV) * 8;
   const int row = row0 + (int)(unit / heads);
   const int hd = (int)(unit % heads);
   const int s = slot[row];
   if (s < 0) return;
   const int p = pos[row];
-  E* base = (E*)a.qkv + (long)row * a.ld;
-
-  if (hd >= a.H + a.G) {           // value head
-    const int g = hd - a.H - a.G;
-    const E* src = base + (long)(a.H + a.G) * a.dim + (long)g * a.vdim;
-    const long page = a.table[(long)s * a.max_pages + p / LM_PAGE];
-    E* dst = (E*)a.vc + ((page * a.G + g) * LM_PAGE + p % LM_PAGE) * a.vdim;
-    for (int c = l; c < a.vdim; c += 64) dst[c] = src[c];
-    return;
-  }
-  E* src = base + (long)hd * a.dim;
-  const void* w = hd < a.H ? a.qw : a.kw;
-  float v[4];
-  float q = 0.f;
-  #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int c = i * 64 + l;
-    v[i] = c < a.dim ? N::up(src[c]) : 0.f;
-    q += v[i] * v[i];
-  }
-  const float inv = w ? 1.0f / sqrtf(wave_reduce_sum(q) / (float)a.dim + a.eps) : 1.f;
+  const bool aligned = a.dim % 8 == 0 && a.vdim % 8 == 0;
+  const bool is_v = hd >= a.H + a.G;
+  const int len = is_v ? a.vdim : a.dim;
+  E* src = (E*)a.qkv + (long)row * a.ld +
+           (is_v ? (long)(a.H + a.G) * a.dim + (long)(hd - a.H - a.G) * a.vdim
+                 : (long)hd * a.dim);
   E* dst = src;
   if (hd >= a.H) {
-    const int g = hd - a.H;
+    const int g = is_v ? hd - a.H - a.G : hd - a.H;
     const long page = a.table[(long)s * a.max_pages + p / LM_PAGE];
-    dst = (E*)a.kc + ((page * a.G + g) * LM_PAGE + p % LM_PAGE) * a.dim;
+    dst = (E*)(is_v ? a.vc : a.kc) +
+          ((page * a.G + g) * LM_PAGE + p % LM_PAGE) * len;
   }
+  float v[8];
+  load8<F32>(src + c, len - c, aligned, v);
+  const E* w = (const E*)(is_v ? nullptr : hd < a.H ? a.qw : a.kw);
+  float q = 0.f;
   #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int c = i * 64 + l;
-    if (c < a.dim)
-      dst[c] = N::down(w ? v[i] * inv * N::up(((const E*)w)[c]) : v[i]);
+  for (int i = 0; i < 8; ++i) q += v[i] * v[i];
+  q = group_sum<LPV>(q);
+  if (w) {
+    const float inv = 1.0f / sqrtf(q / (float)a.dim + a.eps);
+    float wv[8];
+    load8<F32>(w + c, len - c, aligned, wv);
+    #pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= inv * wv[i];
   }
+  store8<F32>(dst + c, len - c, aligned, v);
 }
 
 // 4 waves, 16 query rows each; one query head per block.
@@ -244,20 +240,35 @@ void pick_dk(const AttnArgs& a, const int4* tiles, int n, hipStream_t st) {
 
 }  // namespace
 
+namespace {
+template <bool F32>
+void run_prep(const AttnArgs& a, const int* pos, const int* slot, int row0,
+              int n, hipStream_t st) {
+  const long units = (long)n * (a.H + 2 * a.G);
+  const int d = std::max(a.dim, a.vdim);
+  #define AP_GO(LPV)                                                           \
+    hipLaunchKernelGGL((attn_prep_kernel<F32, LPV>),                           \
+                       dim3((unsigned)((units * LPV + 255) / 256)), dim3(256), \
+                       0, st, a, pos, slot, row0, n)
+  if (d <= 32) AP_GO(4);
+  else if (d <= 64) AP_GO(8);
+  else if (d <= 128) AP_GO(16);
+  else AP_GO(32);
+  #undef AP_GO
+}
+}  // namespace
+
 void lm_attn_prep(const AttnArgs& a, const int* pos, const int* slot, int row0,
                   int n, bool f32, hipStream_t stream) {
   if (n <= 0) return;
-  const long units = (long)n * (a.H + 2 * a.G);
-  const dim3 grid((units + 3) / 4);
-  if (f32)
-    hipLaunchKernelGGL((attn_prep_kernel<true>), grid, dim3(256), 0, stream, a, pos, slot, row0, n);
-  else
-    hipLaunchKernelGGL((attn_prep_kernel<false>), grid, dim3(256), 0, stream, a, pos, slot, row0, n);
+  if (f32) run_prep<true>(a, pos, slot, row0, n, stream);
+  else run_prep<false>(a, pos, slot, row0, n, stream);
 }
 
 void lm_attn_prefill(const AttnArgs& a, const int4* tiles, int n_tiles,
                      bool f32, hipStream_t stream) {
   if (n_tiles <= 0) return;
   if (f32) pick_dk<true>(a, tiles, n_tiles, stream);
+  else if (lm_attn_mfma_ok(a)) lm_attn_prefill_mfma(a, tiles, n_tiles, stream);
   else pick_dk<false>(a, tiles, n_tiles, stream);
 }

@@ -16,13 +16,6 @@ namespace {
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr float NEG = -1e30f;
 
-template <int LPK>
-DEVINL float group_sum(float v) {
-  #pragma unroll
-  for (int o = 1; o < LPK; o <<= 1) v += __shfl_xor(v, o, 64);
-  return v;
-}
-
 // 8 elements, normed over the lane group and rounded to the cache's type
 template <bool F32, int LPK>
 DEVINL void head_norm(float* v, const void* w, int c, int dim, float eps) {

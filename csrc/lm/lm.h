@@ -48,6 +48,10 @@ void lm_attn_prep(const AttnArgs& a, const int* pos, const int* slot, int row0,
                   int n, bool f32, hipStream_t stream);
 void lm_attn_prefill(const AttnArgs& a, const int4* tiles, int n_tiles,
                      bool f32, hipStream_t stream);
+// bf16, head sizes that are multiples of 8 up to 128
+bool lm_attn_mfma_ok(const AttnArgs& a);
+void lm_attn_prefill_mfma(const AttnArgs& a, const int4* tiles, int n_tiles,
+                          hipStream_t stream);
 // rows [0, R), one token each; ws holds R*H*nsplit*(vdim+2) floats
 void lm_attn_decode(const AttnArgs& a, const int* pos, const int* slot, int R,
                     int nsplit, float* ws, bool f32, hipStream_t stream);

@@ -56,7 +56,7 @@ DEVINL void stv(void* base, long i, const Pack<VEC>& p) {
 
 template <int TPR>
 DEVINL float row_sum(float v, float* red) {
-  v = wave_reduce_sum(v);
+  v = group_sum<64>(v);
   if constexpr (TPR == 256) {
     const int w = threadIdx.x >> 6;
     __syncthreads();             // the previous use of red is over

@@ -76,6 +76,28 @@ DEVINL void load8(const typename Num<F32>::E* p, int valid, bool aligned,
   }
 }
 
+// counterpart of load8; elements at or past `valid` are left alone
+template <bool F32>
+DEVINL void store8(typename Num<F32>::E* p, int valid, bool aligned,
+                   const float* v) {
+  if (valid <= 0) return;
+  if (aligned) {
+    if constexpr (F32) {
+      *(f32x4*)p = *(const f32x4*)v;
+      *(f32x4*)(p + 4) = *(const f32x4*)(v + 4);
+    } else {
+      bf16x8 t;
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) t[i] = cvt_bf16(v[i]);
+      *(bf16x8*)p = t;
+    }
+  } else {
+    #pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (i < valid) p[i] = Num<F32>::down(v[i]);
+  }
+}
+
 // Operand kept at (nearly) float precision in LDS.  In bf16 mode a value
 // is the sum of two bf16 (16 significand bits) and a product is three
 // MFMAs; in float mode it is the value itself.
@@ -117,13 +139,32 @@ DEVINL f32x4 mma_sp(const typename Split<F32>::Frag& a,
   return Num<F32>::mma(a.hi, b, c);
 }
 
-DEVINL float sum16(float v) {  // over the 16 lanes that share l/16
-  #pragma unroll
-  for (int o = 1; o < 16; o <<= 1) v += __shfl_xor(v, o, 64);
+// DPP lane exchanges: VALU speed, no LDS pipe.  Applied in this order
+// (neighbour, pair, 4, 8) each step pairs lanes whose partial results
+// already agree within the smaller group, so mirrors serve as xor 4 and 8.
+template <int CTRL>
+DEVINL float dpp(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+      0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
+}
+constexpr int DPP_XOR1 = 0xB1, DPP_XOR2 = 0x4E;           // quad_perm
+constexpr int DPP_HALF_MIRROR = 0x141, DPP_MIRROR = 0x140;  // of 8, of 16
+
+// over aligned groups of N lanes (N = 2..64), result in every lane
+template <int N>
+DEVINL float group_sum(float v) {
+  if constexpr (N >= 2) v += dpp<DPP_XOR1>(v);
+  if constexpr (N >= 4) v += dpp<DPP_XOR2>(v);
+  if constexpr (N >= 8) v += dpp<DPP_HALF_MIRROR>(v);
+  if constexpr (N >= 16) v += dpp<DPP_MIRROR>(v);
+  if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
+  if constexpr (N >= 64) v += __shfl_xor(v, 32, 64);
   return v;
 }
+DEVINL float sum16(float v) { return group_sum<16>(v); }
 DEVINL float max16(float v) {
-  #pragma unroll
-  for (int o = 1; o < 16; o <<= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
-  return v;
+  v = fmaxf(v, dpp<DPP_XOR1>(v));
+  v = fmaxf(v, dpp<DPP_XOR2>(v));
+  v = fmaxf(v, dpp<DPP_HALF_MIRROR>(v));
+  return fmaxf(v, dpp<DPP_MIRROR>(v));
 }

@@ -49,6 +49,7 @@ _LM_SOURCES = [
     "lm/ext.cpp",
     "lm/norm.hip",
     "lm/attn.hip",
+    "lm/attn_mfma.hip",
     "lm/attn_decode.hip",
     "lm/retention.hip",
 ]
