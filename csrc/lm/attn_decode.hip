@@ -7,6 +7,9 @@
 // LPK lanes share one key (8 elements each), 64/LPK keys go through a wave
 // at a time and each lane group keeps its own running softmax; groups,
 // waves and splits merge at the end.  The sink joins the last merge.
+// The next pass's keys and values are loaded before the current ones are
+// used, and the split's page ids wait in LDS, so a pass costs no
+// dependent memory round trip.
 
 #include "lm.h"
 #include "tile.h"
@@ -40,9 +43,12 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
   using N = Num<F32>;
   using E = typename N::E;
   constexpr int KPW = 64 / LPK;      // keys per wave and pass
-  constexpr int KB = 4;              // passes in flight
-  __shared__ float acc_s[4][HGC][LPK * 8];
-  __shared__ float m_s[4][HGC], l_s[4][HGC];
+  constexpr int KB = F32 ? 2 : 4;    // keys per lane group and pass
+  constexpr int TABS = 512;          // page ids kept in LDS
+  __shared__ int tab_s[TABS];
+  constexpr int NP = 4 * KPW;        // partial results of a block
+  __shared__ __attribute__((aligned(16))) float acc_s[HGC][NP][LPK * 8];
+  __shared__ float m_s[HGC][NP], l_s[HGC][NP];
 
   const int split = blockIdx.x, row = blockIdx.z;
   const int hg = a.H / a.G, nhc = (hg + HGC - 1) / HGC;
@@ -87,8 +93,7 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
     for (int j = 0; j < 8; ++j) acc[i][j] = 0.f;
   }
 
-  auto fold = [&](const float (&k)[KB][8], const float (&v)[KB][8],
-                  const bool (&ok)[KB]) {
+  auto fold = [&](const auto& k, const auto& v, const bool (&ok)[KB]) {
     #pragma unroll
     for (int i = 0; i < HGC; ++i) {
       float sc[KB], mx = m[i];
@@ -120,72 +125,78 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
     }
   };
 
-  const int jc = min(je, p);                  // cached keys end here
-  for (int j0 = jb; j0 < jc; j0 += 4 * KPW * KB) {
-    float k[KB][8], v[KB][8];
-    bool ok[KB];
+  const int jc = min(je, p + 1);              // p itself is not cached yet
+  const int pg0 = jb / LM_PAGE;
+  const int npg = jc > jb ? (jc - 1) / LM_PAGE - pg0 + 1 : 0;
+  const bool in_lds = npg <= TABS;
+  if (in_lds) {
+    for (int i = tid; i < npg; i += 256) tab_s[i] = tab[pg0 + i];
+    __syncthreads();
+  }
+  // the new token's key and value, in every lane group of the split that
+  // has it; the group whose turn it is takes them from here
+  Raw8<F32> knew, vnew;
+  if (has_new) {
+    float k0[8];
+    load8<F32>(qkv + (long)(a.H + g) * a.dim + c, a.dim - c, aligned, k0);
+    vnew.load(qkv + (long)(a.H + a.G) * a.dim + (long)g * a.vdim + c,
+              a.vdim - c, aligned);
+    head_norm<F32, LPK>(k0, a.kw, c, a.dim, a.eps);
+    #pragma unroll
+    for (int j = 0; j < 8; ++j) knew.e[j] = N::down(k0[j]);
+    if (w == 0 && grp == 0 && hc == 0) {
+      const long cell = ((long)tab[p / LM_PAGE] * a.G + g) * LM_PAGE + p % LM_PAGE;
+      float v0[8];
+      #pragma unroll
+      for (int j = 0; j < 8; ++j) v0[j] = vnew[j];
+      store8<F32>((E*)a.kc + cell * a.dim + c, a.dim - c, aligned, k0);
+      store8<F32>((E*)a.vc + cell * a.vdim + c, a.vdim - c, aligned, v0);
+    }
+  }
+  Raw8<F32> kn[KB], vn[KB];
+  bool okn[KB];
+  auto fetch = [&](int j0) {
     #pragma unroll
     for (int u = 0; u < KB; ++u) {
       const int j = j0 + (u * 4 + w) * KPW + grp;
-      ok[u] = j < jc;
-      long kb = 0, vb = 0;
-      if (ok[u]) {
-        const long cell = ((long)tab[j / LM_PAGE] * a.G + g) * LM_PAGE + j % LM_PAGE;
-        kb = cell * a.dim + c;
-        vb = cell * a.vdim + c;
+      okn[u] = j < jc;
+      const bool cached = j < min(jc, p);
+      long cell = 0;
+      if (cached) {
+        const int page = in_lds ? tab_s[j / LM_PAGE - pg0] : tab[j / LM_PAGE];
+        cell = ((long)page * a.G + g) * LM_PAGE + j % LM_PAGE;
       }
-      load8<F32>((const E*)a.kc + kb, ok[u] ? a.dim - c : 0, aligned, k[u]);
-      load8<F32>((const E*)a.vc + vb, ok[u] ? a.vdim - c : 0, aligned, v[u]);
+      kn[u].load((const E*)a.kc + cell * a.dim + c, cached ? a.dim - c : 0, aligned);
+      vn[u].load((const E*)a.vc + cell * a.vdim + c, cached ? a.vdim - c : 0, aligned);
+      if (j == p && okn[u]) {
+        kn[u] = knew;
+        vn[u] = vnew;
+      }
     }
-    fold(k, v, ok);
-  }
-  if (has_new && w == 0) {
-    float k[KB][8], v[KB][8];
+  };
+  constexpr int STEP = 4 * KPW * KB;
+  if (jb < jc) fetch(jb);
+  for (int j0 = jb; j0 < jc; j0 += STEP) {
+    Raw8<F32> k[KB], v[KB];
     bool ok[KB];
     #pragma unroll
     for (int u = 0; u < KB; ++u) {
-      ok[u] = u == 0 && grp == 0;
-      #pragma unroll
-      for (int j = 0; j < 8; ++j) k[u][j] = v[u][j] = 0.f;
+      k[u] = kn[u];
+      v[u] = vn[u];
+      ok[u] = okn[u];
     }
-    load8<F32>(qkv + (long)(a.H + g) * a.dim + c, a.dim - c, aligned, k[0]);
-    load8<F32>(qkv + (long)(a.H + a.G) * a.dim + (long)g * a.vdim + c,
-               a.vdim - c, aligned, v[0]);
-    head_norm<F32, LPK>(k[0], a.kw, c, a.dim, a.eps);
-    if (grp == 0 && hc == 0) {
-      const long cell = ((long)tab[p / LM_PAGE] * a.G + g) * LM_PAGE + p % LM_PAGE;
-      E* kd = (E*)a.kc + cell * a.dim + c;
-      E* vd = (E*)a.vc + cell * a.vdim + c;
-      #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        if (c + j < a.dim) kd[j] = N::down(k[0][j]);
-        if (c + j < a.vdim) vd[j] = N::down(v[0][j]);
-      }
-    }
+    if (j0 + STEP < jc) fetch(j0 + STEP);
     fold(k, v, ok);
   }
-
-  // lane groups of a wave, then the four waves
+  // every lane group's partial meets in LDS
   #pragma unroll
   for (int i = 0; i < HGC; ++i) {
-    #pragma unroll
-    for (int o = LPK; o < 64; o <<= 1) {
-      const float mo = __shfl_xor(m[i], o, 64), lo = __shfl_xor(ls[i], o, 64);
-      const float mn = fmaxf(m[i], mo);
-      const float x = exp2f(m[i] - mn), y = exp2f(mo - mn);
-      ls[i] = ls[i] * x + lo * y;
-      #pragma unroll
-      for (int j = 0; j < 8; ++j)
-        acc[i][j] = acc[i][j] * x + __shfl_xor(acc[i][j], o, 64) * y;
-      m[i] = mn;
-    }
-    if (grp == 0) {
-      #pragma unroll
-      for (int j = 0; j < 8; ++j) acc_s[w][i][c + j] = acc[i][j];
-      if (l == 0) {
-        m_s[w][i] = m[i];
-        l_s[w][i] = ls[i];
-      }
+    float* d = acc_s[i][w * KPW + grp] + c;
+    *(f32x4*)d = *(const f32x4*)acc[i];
+    *(f32x4*)(d + 4) = *(const f32x4*)(acc[i] + 4);
+    if (c == 0) {
+      m_s[i][w * KPW + grp] = m[i];
+      l_s[i][w * KPW + grp] = ls[i];
     }
   }
   __syncthreads();
@@ -193,13 +204,13 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
     const int i = t / a.vdim, d = t % a.vdim;
     float mn = NEG;
     #pragma unroll
-    for (int x = 0; x < 4; ++x) mn = fmaxf(mn, m_s[x][i]);
+    for (int x = 0; x < NP; ++x) mn = fmaxf(mn, m_s[i][x]);
     float lt = 0.f, av = 0.f;
     #pragma unroll
-    for (int x = 0; x < 4; ++x) {
-      const float f = exp2f(m_s[x][i] - mn);
-      lt += l_s[x][i] * f;
-      av += acc_s[x][i][d] * f;
+    for (int x = 0; x < NP; ++x) {
+      const float f = exp2f(m_s[i][x] - mn);
+      lt += l_s[i][x] * f;
+      av += acc_s[i][x][d] * f;
     }
     if (nsplit == 1) {
       if (a.sink) {
@@ -221,6 +232,7 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
   }
 }
 
+// One wave-pair or more per (row, head); lane i weighs split i (at most 64).
 template <bool F32>
 __global__ void __launch_bounds__(256)
 attn_combine_kernel(AttnArgs a, const int* __restrict__ slot, int nsplit,
@@ -228,20 +240,25 @@ attn_combine_kernel(AttnArgs a, const int* __restrict__ slot, int nsplit,
   using N = Num<F32>;
   using E = typename N::E;
   const int h = blockIdx.x, row = blockIdx.y;
-  if (slot[row] < 0) return;
-  const float* p = ws + ((long)row * a.H + h) * nsplit * (a.vdim + 2);
+  const int l = threadIdx.x & 63;
   const int st = a.vdim + 2;
-  float mn = a.sink ? N::up(((const E*)a.sink)[h]) * LOG2E : NEG;
-  float lt = 0.f;
-  const float m0 = mn;
-  for (int i = 0; i < nsplit; ++i) mn = fmaxf(mn, p[i * st]);
-  if (a.sink) lt = exp2f(m0 - mn);
-  for (int i = 0; i < nsplit; ++i) lt += p[i * st + 1] * exp2f(p[i * st] - mn);
-  for (int d = threadIdx.x; d < a.vdim; d += 256) {
+  const float* p = ws + ((long)row * a.H + h) * nsplit * st;
+  const bool on = l < nsplit;
+  const float mi = on ? p[l * st] : NEG, li = on ? p[l * st + 1] : 0.f;
+  const float sk = a.sink ? N::up(((const E*)a.sink)[h]) * LOG2E : NEG;
+  const bool idle = slot[row] < 0;            // its output is already set
+  const float mn = wave_reduce_max(fmaxf(mi, sk));
+  const float f = on ? exp2f(mi - mn) : 0.f;
+  const float lt = group_sum<64>(li * f) + (a.sink ? exp2f(sk - mn) : 0.f);
+  const float inv = 1.0f / lt;
+  for (int d = threadIdx.x; d < (a.vdim + 63) / 64 * 64; d += blockDim.x) {
+    const int dc = min(d, a.vdim - 1);
     float av = 0.f;
+    #pragma unroll 8
     for (int i = 0; i < nsplit; ++i)
-      av += p[i * st + 2 + d] * exp2f(p[i * st] - mn);
-    ((E*)a.out)[((long)row * a.H + h) * a.vdim + d] = N::down(av / lt);
+      av = fmaf(p[i * st + 2 + dc], __shfl(f, i, 64), av);
+    if (d < a.vdim && !idle)
+      ((E*)a.out)[((long)row * a.H + h) * a.vdim + d] = N::down(av * inv);
   }
 }
 

@@ -160,7 +160,8 @@ Tensor paged_attention(Tensor qkv, Tensor kc, Tensor vc, Tensor table,
   auto st = cur_stream();
   if (n_dec > 0) {
     TORCH_CHECK(n_dec <= 65535, "too many decode rows");
-    // enough blocks to fill the chip, none with fewer than ~128 keys
+    // enough blocks to fill the chip, none with fewer than ~128 keys;
+    // the merge takes at most 64 splits
     const long hg = a.H / a.G, hc = hg <= 2 ? hg : 4;
     const long blocks = n_dec * a.G * ((hg + hc - 1) / hc);
     const long keys = size > 0 ? std::min<long>(size, max_len) : max_len;
@@ -223,7 +224,7 @@ Tensor retention(Tensor qkvg, Tensor state, Tensor pos, Tensor slot,
   auto st = cur_stream();
   if (n_dec > 0) lm_ret_decode(a, pp, sp, (int)n_dec, f32, st);
   if (nt > 0) {
-    TORCH_CHECK(ns >= 1 && ns <= 65535, "prompt portions");
+    TORCH_CHECK(ns >= 1 && ns <= 65535 && nt <= 65535, "prompt portions");
     auto cs = torch::empty({nt, a.H, a.dv, a.dk}, state.options());
     lm_ret_prefill(a, tp, (int)nt, qp, (int)ns, cs.data_ptr<float>(), f32, st);
   }

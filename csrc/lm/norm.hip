@@ -35,6 +35,23 @@ DEVINL Pack<VEC> ldv(const void* base, long i) {
   return p;
 }
 
+// VEC elements as stored (half the registers of their float form in bf16)
+template <bool F32, int VEC> struct Held {
+  typename Num<F32>::E e[VEC];
+  DEVINL void load(const void* base, long i) {
+    const auto* s = (const typename Num<F32>::E*)base + i;
+    if constexpr (VEC == 4 && F32) *(f32x4*)e = *(const f32x4*)s;
+    else if constexpr (VEC == 4) *(bf16x4*)e = *(const bf16x4*)s;
+    else e[0] = s[0];
+  }
+  DEVINL Pack<VEC> up() const {
+    Pack<VEC> p;
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) p.v[j] = Num<F32>::up(e[j]);
+    return p;
+  }
+};
+
 template <bool F32, int VEC>
 DEVINL void stv(void* base, long i, const Pack<VEC>& p) {
   if constexpr (F32) {
@@ -123,6 +140,25 @@ residual_norm_kernel(NormArgs a) {
   const long row = a.rows ? a.rows[out_row] : out_row;
   const int W = a.W;
 
+  // the weights of a narrow share are fetched with the row, so that the
+  // reductions wait for one memory round trip and not for three
+  constexpr bool EARLY = NV <= 4;
+  Held<F32, VEC> wp[EARLY ? NV : 1], bp[EARLY ? NV : 1], wn[EARLY ? NV : 1],
+      bn[EARLY ? NV : 1];
+  if constexpr (EARLY) {
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      wp[i] = bp[i] = wn[i] = bn[i] = Held<F32, VEC>{};
+      if (c < W) {
+        if (a.pw) wp[i].load(a.pw, c);
+        if (a.pb) bp[i].load(a.pb, c);
+        if (a.nw) wn[i].load(a.nw, c);
+        if (a.nb) bn[i].load(a.nb, c);
+      }
+    }
+  }
+
   Pack<VEC> x[NV];
   if (a.tokens) {
     const long tok = a.tokens[row];
@@ -156,9 +192,14 @@ residual_norm_kernel(NormArgs a) {
       const int c = (i * TPR + tid) * VEC;
       if (c < W) {
         if (a.pw) {
-          const Pack<VEC> w = ldv<F32, VEC>(a.pw, c);
-          Pack<VEC> b{};
-          if (a.pb) b = ldv<F32, VEC>(a.pb, c);
+          Pack<VEC> w, b{};
+          if constexpr (EARLY) {
+            w = wp[i].up();
+            b = bp[i].up();
+          } else {
+            w = ldv<F32, VEC>(a.pw, c);
+            if (a.pb) b = ldv<F32, VEC>(a.pb, c);
+          }
           #pragma unroll
           for (int j = 0; j < VEC; ++j)
             y[i].v[j] = y[i].v[j] * w.v[j] + b.v[j];
@@ -175,9 +216,14 @@ residual_norm_kernel(NormArgs a) {
     for (int i = 0; i < NV; ++i) {
       const int c = (i * TPR + tid) * VEC;
       if (c < W) {
-        const Pack<VEC> w = ldv<F32, VEC>(a.nw, c);
-        Pack<VEC> b{};
-        if (a.nb) b = ldv<F32, VEC>(a.nb, c);
+        Pack<VEC> w, b{};
+        if constexpr (EARLY) {
+          w = wn[i].up();
+          b = bn[i].up();
+        } else {
+          w = ldv<F32, VEC>(a.nw, c);
+          if (a.nb) b = ldv<F32, VEC>(a.nb, c);
+        }
         #pragma unroll
         for (int j = 0; j < VEC; ++j)
           x[i].v[j] = x[i].v[j] * w.v[j] + b.v[j];

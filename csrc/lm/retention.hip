@@ -59,8 +59,89 @@ DEVINL void load_rot8(const typename Num<F32>::E* head, int c, const RetArgs& a,
   for (int j = 0; j < 8; ++j) out[j] *= mul;
 }
 
+// Visit a tile's 64 x D elements of one head's q or k, rotated and scaled by
+// mul(j), 8 at a time: put(j, c, v).  Rows past `rows` are zeros.  The usual
+// shapes take a branch-free path whose loads are all in flight together.
+template <bool F32, int D, typename Mul, typename Put>
+DEVINL void stage_rot(const typename Num<F32>::E* head0, const RetArgs& a,
+                      int pos0, int rows, bool aligned, Mul mul, Put put) {
+  constexpr int N = 64 * (D / 8) / 256;
+  const int half = a.rd >> 1;
+  if (aligned && half % 8 == 0) {
+    Raw8<F32> own[N], oth[N];
+    float cv[N][8], sv[N][8];
+    #pragma unroll
+    for (int it = 0; it < N; ++it) {
+      const int u = it * 256 + threadIdx.x;
+      const int j = min(u / (D / 8), rows - 1);
+      int c = (u % (D / 8)) * 8;
+      c = c < a.dk ? c : 0;
+      const bool in = c < a.rd, low = c < half;
+      const int oc = in ? (low ? c + half : c - half) : c;
+      const typename Num<F32>::E* p = head0 + (long)j * a.ld;
+      own[it].load(p + c, 8, true);
+      oth[it].load(p + oc, 8, true);
+      if (half) {                              // uniform
+        const long ti = (long)(pos0 + j) * half + (in ? (low ? c : c - half) : 0);
+        load8<true>(a.cos_t + ti, 8, true, cv[it]);
+        load8<true>(a.sin_t + ti, 8, true, sv[it]);
+      }
+    }
+    #pragma unroll
+    for (int it = 0; it < N; ++it) {
+      const int u = it * 256 + threadIdx.x;
+      const int j = u / (D / 8), c = (u % (D / 8)) * 8;
+      const bool in = c < a.rd, low = c < half;
+      const float f = j < rows && c < a.dk ? mul(min(j, rows - 1)) : 0.f;
+      float v[8];
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float x = own[it][i], y = oth[it][i];
+        float r = x;
+        if (half) {
+          const float w = low ? -y : y;
+          r = in ? x * cv[it][i] + w * sv[it][i] : x;
+        }
+        v[i] = r * f;
+      }
+      put(j, c, v);
+    }
+  } else {
+    for (int u = threadIdx.x; u < 64 * (D / 8); u += 256) {
+      const int j = u / (D / 8), c = (u % (D / 8)) * 8;
+      float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (j < rows)
+        load_rot8<F32>(head0 + (long)j * a.ld, c, a, pos0 + j, mul(j), aligned, v);
+      put(j, c, v);
+    }
+  }
+}
+
 DEVINL bool ret_aligned(const RetArgs& a) {
   return a.dk % 8 == 0 && a.dv % 8 == 0;
+}
+
+// value rows of a tile, zeros past its end
+template <bool F32, int DV>
+DEVINL void stage_v(const ColTile<F32, DV>& V, const typename Num<F32>::E* v0,
+                    const RetArgs& a, int rows, bool aligned) {
+  constexpr int N = LM_TILE * (DV / 8) / 256;
+  Raw8<F32> r[N];
+  #pragma unroll
+  for (int it = 0; it < N; ++it) {
+    const int u = it * 256 + threadIdx.x, c = (u % (DV / 8)) * 8;
+    const typename Num<F32>::E* p = v0 + (long)min(u / (DV / 8), rows - 1) * a.ld;
+    if (aligned) r[it].load(p + (c < a.dv ? c : 0), 8, true);
+    else r[it].load(p + c, a.dv - c, false);
+  }
+  #pragma unroll
+  for (int it = 0; it < N; ++it) {
+    const int u = it * 256 + threadIdx.x;
+    const int j = u / (DV / 8), c = (u % (DV / 8)) * 8;
+    if (j >= rows || c >= a.dv) r[it] = Raw8<F32>{};
+    if constexpr (F32) V.put8(j, c, r[it].e);
+    else V.put_raw(j, c, *(const bf16x8*)r[it].e);
+  }
 }
 
 // state contribution of one tile and head: sum_j d^(n-1-j) v_j k_j^T
@@ -70,64 +151,76 @@ ret_chunk_state_kernel(RetArgs a, const int4* __restrict__ tiles,
                        float* __restrict__ cs) {
   using N = Num<F32>;
   using E = typename N::E;
-  constexpr int LDJ = LM_TILE + N::PAD;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  E* Vt = (E*)smem;                         // [DV][LDJ]
-  E* Kb = Vt + DV * LDJ;                    // [PARTS][DK][LDJ]
-  const Split<F32> K{Kb, Kb + DK * LDJ};
+  const ColTile<F32, DV> V{(E*)smem};
+  const ColTile<F32, DK> Kh{V.p + V.SIZE}, Kl{Kh.p + Kh.SIZE};
 
-  const int4 t = tiles[blockIdx.x];
-  const int h = blockIdx.y;
+  const int4 t = tiles[blockIdx.y];
+  const int h = blockIdx.x;   // heads of a row run together: whole rows stream
   const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
   const int lr = l & 15, lg = l >> 4;
   const bool aligned = ret_aligned(a);
   const float* pw = a.pows + (long)h * (LM_TILE + 1);
   const E* base = (const E*)a.qkvg + (long)t.x * a.ld;
 
-  for (int u = tid; u < LM_TILE * (DK / 8); u += 256) {
-    const int j = u % LM_TILE, c = (u / LM_TILE) * 8;
-    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (j < t.y)
-      load_rot8<F32>(base + (long)j * a.ld + (long)(a.H + h) * a.dk, c, a,
-                     t.z + j, a.kscale * pw[t.y - 1 - j], aligned, v);
-    #pragma unroll
-    for (int i = 0; i < 8; ++i) K.put((c + i) * LDJ + j, v[i]);
-  }
-  for (int u = tid; u < LM_TILE * (DV / 8); u += 256) {
-    const int j = u % LM_TILE, c = (u / LM_TILE) * 8;
-    float v[8];
-    load8<F32>(base + (long)min(j, t.y - 1) * a.ld + (long)2 * a.H * a.dk +
-                   (long)h * a.dv + c,
-               j < t.y ? a.dv - c : 0, aligned, v);
-    #pragma unroll
-    for (int i = 0; i < 8; ++i) Vt[(c + i) * LDJ + j] = N::down(v[i]);
-  }
+  stage_rot<F32, DK>(
+      base + (long)(a.H + h) * a.dk, a, t.z, t.y, aligned,
+      [&](int j) { return a.kscale * pw[t.y - 1 - j]; },
+      [&](int j, int c, float* v) {
+        Kh.put8(j, c, v);
+        if constexpr (!F32) {
+          #pragma unroll
+          for (int i = 0; i < 8; ++i) v[i] -= bf2f(cvt_bf16(v[i]));
+          Kl.put8(j, c, v);
+        }
+      });
+  stage_v<F32, DV>(V, base + (long)2 * a.H * a.dk + (long)h * a.dv, a, t.y,
+                   aligned);
   __syncthreads();
 
-  float* dst = cs + ((long)blockIdx.x * a.H + h) * a.dv * a.dk;
-  constexpr int RT = DV / 64;               // 16-row tiles of a wave
-  for (int ct = 0; ct < DK / 16; ++ct) {
-    if (ct * 16 >= a.dk) break;
-    f32x4 acc[RT];
+  // wave w owns DV/4 state rows, in groups of 16; 64 columns at a time
+  float* dst = cs + ((long)blockIdx.y * a.H + h) * a.dv * a.dk;
+  constexpr int RT = DV / 64;
+  for (int c4 = 0; c4 < DK / 16; c4 += 4) {
+    if (c4 * 16 >= a.dk) break;
+    f32x4 acc[RT][4];
     #pragma unroll
-    for (int i = 0; i < RT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < RT; ++i)
+      #pragma unroll
+      for (int x = 0; x < 4; ++x) acc[i][x] = f32x4{0.f, 0.f, 0.f, 0.f};
     #pragma unroll
     for (int kb = 0; kb < LM_TILE / 32; ++kb) {
-      const auto kf = K.load((ct * 16 + lr) * LDJ, kb * 32 + lg * 8);
+      typename N::Frag vf[4], kh[4], kl[4];
+      // the wave's row tiles are among these four (RT divides 4)
+      V.frags4((w * RT) / 4 * 4, kb, l, vf);
+      Kh.frags4(c4, kb, l, kh);
+      if constexpr (!F32) Kl.frags4(c4, kb, l, kl);
       #pragma unroll
       for (int i = 0; i < RT; ++i) {
-        const auto vf = N::load(Vt + ((w * RT + i) * 16 + lr) * LDJ, kb * 32 + lg * 8);
-        if constexpr (!F32) acc[i] = N::mma(vf, kf.lo, acc[i]);
-        acc[i] = N::mma(vf, kf.hi, acc[i]);
+        typename N::Frag r = vf[i];
+        if constexpr (RT < 4) {
+          // select tile w*RT + i without indexing registers by a variable
+          #pragma unroll
+          for (int y = 0; y < 4; ++y)
+            if ((w * RT) % 4 + i == y) r = vf[y];
+        }
+        #pragma unroll
+        for (int x = 0; x < 4; ++x) {
+          if constexpr (!F32) acc[i][x] = N::mma(r, kl[x], acc[i][x]);
+          acc[i][x] = N::mma(r, kh[x], acc[i][x]);
+        }
       }
     }
     #pragma unroll
     for (int i = 0; i < RT; ++i)
       #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int row = (w * RT + i) * 16 + 4 * lg + r, col = ct * 16 + lr;
-        if (row < a.dv && col < a.dk) dst[(long)row * a.dk + col] = acc[i][r];
-      }
+      for (int x = 0; x < 4; ++x)
+        #pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int row = (w * RT + i) * 16 + 4 * lg + r;
+          const int col = (c4 + x) * 16 + lr;
+          if (row < a.dv && col < a.dk) dst[(long)row * a.dk + col] = acc[i][x][r];
+        }
   }
 }
 
@@ -166,14 +259,14 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
   constexpr int LDK = DK + N::PAD;
   constexpr int LDJ = LM_TILE + N::PAD;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  E* Vt = (E*)smem;                         // [DV][LDJ]
-  E* Pb = Vt + DV * LDJ;                    // [PARTS][64][LDJ]
+  const ColTile<F32, DV> V{(E*)smem};
+  E* Pb = V.p + V.SIZE;                     // [PARTS][64][LDJ]
   E* Xb = Pb + Split<F32>::PARTS * LM_TILE * LDJ;   // [PARTS][64][LDK]
   const Split<F32> P{Pb, Pb + LM_TILE * LDJ};
   const Split<F32> X{Xb, Xb + LM_TILE * LDK};       // q, then k, then S
 
-  const int4 t = tiles[blockIdx.x];
-  const int h = blockIdx.y;
+  const int4 t = tiles[blockIdx.y];
+  const int h = blockIdx.x;   // heads of a row run together: whole rows stream
   const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
   const int lr = l & 15, lg = l >> 4;
   const bool aligned = ret_aligned(a);
@@ -181,25 +274,13 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
   const E* base = (const E*)a.qkvg + (long)t.x * a.ld;
 
   auto stage_qk = [&](long off, float mul) {
-    for (int u = tid; u < LM_TILE * (DK / 8); u += 256) {
-      const int j = u / (DK / 8), c = (u % (DK / 8)) * 8;
-      float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (j < t.y)
-        load_rot8<F32>(base + (long)j * a.ld + off, c, a, t.z + j, mul, aligned, v);
-      #pragma unroll
-      for (int i = 0; i < 8; ++i) X.put(j * LDK + c + i, v[i]);
-    }
+    stage_rot<F32, DK>(base + off, a, t.z, t.y, aligned,
+                       [&](int) { return mul; },
+                       [&](int j, int c, float* v) { X.put8(j * LDK + c, v); });
   };
   stage_qk((long)h * a.dk, 1.f);
-  for (int u = tid; u < LM_TILE * (DV / 8); u += 256) {
-    const int j = u % LM_TILE, c = (u / LM_TILE) * 8;
-    float v[8];
-    load8<F32>(base + (long)min(j, t.y - 1) * a.ld + (long)2 * a.H * a.dk +
-                   (long)h * a.dv + c,
-               j < t.y ? a.dv - c : 0, aligned, v);
-    #pragma unroll
-    for (int i = 0; i < 8; ++i) Vt[(c + i) * LDJ + j] = N::down(v[i]);
-  }
+  stage_v<F32, DV>(V, base + (long)2 * a.H * a.dk + (long)h * a.dv, a, t.y,
+                   aligned);
   __syncthreads();
   typename Split<F32>::Frag qf[DK / 32];
   #pragma unroll
@@ -227,19 +308,29 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
 
   // incoming state, 64 value rows at a time through X
   f32x4 o[DV / 16];
-  const float* S = cs + ((long)blockIdx.x * a.H + h) * a.dv * a.dk;
+  const float* S = cs + ((long)blockIdx.y * a.H + h) * a.dv * a.dk;
   const bool s_al = a.dk % 8 == 0;
   #pragma unroll
   for (int vb = 0; vb < DV / 64; ++vb) {
     __syncthreads();
-    for (int u = tid; u < 64 * (DK / 8); u += 256) {
-      const int j = u / (DK / 8), c = (u % (DK / 8)) * 8;
-      float v[8];
-      const int row = vb * 64 + j;
-      load8<true>(S + (long)min(row, a.dv - 1) * a.dk + c,
-                  row < a.dv ? a.dk - c : 0, s_al, v);
+    constexpr int NS = 64 * (DK / 8) / 256;
+    float v[NS][8];
+    #pragma unroll
+    for (int it = 0; it < NS; ++it) {
+      const int u = it * 256 + tid, c = (u % (DK / 8)) * 8;
+      const long row = min(vb * 64 + u / (DK / 8), a.dv - 1);
+      if (s_al)                                // uniform
+        load8<true>(S + row * a.dk + (c < a.dk ? c : 0), 8, true, v[it]);
+      else
+        load8<true>(S + row * a.dk + c, a.dk - c, false, v[it]);
+    }
+    #pragma unroll
+    for (int it = 0; it < NS; ++it) {
+      const int u = it * 256 + tid, j = u / (DK / 8), c = (u % (DK / 8)) * 8;
+      const float on = vb * 64 + j < a.dv && c < a.dk ? 1.f : 0.f;
       #pragma unroll
-      for (int i = 0; i < 8; ++i) X.put(j * LDK + c + i, v[i]);
+      for (int i = 0; i < 8; ++i) v[it][i] *= on;
+      X.put8(j * LDK + c, v[it]);
     }
     __syncthreads();
     #pragma unroll
@@ -250,6 +341,16 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
         acc = mma_ss<F32>(qf[kb], X.load((i * 16 + lr) * LDK, kb * 32 + lg * 8), acc);
       o[vb * 4 + i] = acc;
     }
+  }
+  // gates: all in flight here, used in the epilogue
+  E gz[4][DV / 16];
+  #pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const E* gate = base + (long)min(16 * w + 4 * lg + r, t.y - 1) * a.ld +
+                    (long)2 * a.H * a.dk + (long)(a.H + h) * a.dv;
+    #pragma unroll
+    for (int i = 0; i < DV / 16; ++i)
+      gz[r][i] = gate[min(i * 16 + lr, a.dv - 1)];
   }
   float ss[4] = {0.f, 0.f, 0.f, 0.f};
   #pragma unroll
@@ -263,8 +364,12 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
     if (kb * 2 > w) continue;               // keys after all of these rows
     const auto pf = P.load((16 * w + lr) * LDJ, kb * 32 + lg * 8);
     #pragma unroll
-    for (int i = 0; i < DV / 16; ++i)
-      o[i] = mma_sp<F32>(pf, N::load(Vt + (i * 16 + lr) * LDJ, kb * 32 + lg * 8), o[i]);
+    for (int i = 0; i < DV / 16; i += 4) {
+      typename N::Frag vf[4];
+      V.frags4(i, kb, l, vf);
+      #pragma unroll
+      for (int x = 0; x < 4; ++x) o[i + x] = mma_sp<F32>(pf, vf[x], o[i + x]);
+    }
   }
   #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -276,14 +381,12 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
   for (int r = 0; r < 4; ++r) {
     const int row = 16 * w + 4 * lg + r;
     if (row >= t.y) continue;
-    const E* gate = base + (long)row * a.ld + (long)2 * a.H * a.dk +
-                    (long)(a.H + h) * a.dv;
     E* dst = (E*)a.out + ((long)(t.x + row) * a.H + h) * a.dv;
     #pragma unroll
     for (int i = 0; i < DV / 16; ++i) {
       const int c = i * 16 + lr;
       if (c < a.dv) {
-        const float z = N::up(gate[c]);
+        const float z = N::up(gz[r][i]);
         dst[c] = N::down(o[i][r] * ss[r] * (z / (1.0f + expf(-z))));
       }
     }
@@ -406,8 +509,9 @@ void launch_prefill(const RetArgs& a, const int4* tiles, int n_tiles,
   using S = Split<F32>;
   constexpr size_t es = sizeof(typename N::E);
   constexpr int LDJ = LM_TILE + N::PAD;
-  constexpr size_t lds1 = es * (DV * LDJ + S::PARTS * DK * LDJ);
-  constexpr size_t lds2 = es * (DV * LDJ + S::PARTS * LM_TILE * LDJ +
+  using V = ColTile<F32, DV>;
+  constexpr size_t lds1 = es * (V::SIZE + S::PARTS * ColTile<F32, DK>::SIZE);
+  constexpr size_t lds2 = es * (V::SIZE + S::PARTS * LM_TILE * LDJ +
                                 S::PARTS * LM_TILE * (DK + N::PAD));
   static_assert(lds1 <= 160 * 1024 && lds2 <= 160 * 1024, "exceeds the CU's LDS");
   static const hipError_t attr1 = hipFuncSetAttribute(
@@ -418,12 +522,12 @@ void launch_prefill(const RetArgs& a, const int4* tiles, int n_tiles,
       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds2);
   (void)attr1;
   (void)attr2;
-  hipLaunchKernelGGL((ret_chunk_state_kernel<F32, DK, DV>), dim3(n_tiles, a.H),
+  hipLaunchKernelGGL((ret_chunk_state_kernel<F32, DK, DV>), dim3(a.H, n_tiles),
                      dim3(256), lds1, st, a, tiles, cs);
   hipLaunchKernelGGL(ret_scan_kernel,
                      dim3((unsigned)(((long)a.dv * a.dk + 255) / 256), a.H, n_seqs),
                      dim3(256), 0, st, a, tiles, seqs, cs);
-  hipLaunchKernelGGL((ret_chunk_out_kernel<F32, DK, DV>), dim3(n_tiles, a.H),
+  hipLaunchKernelGGL((ret_chunk_out_kernel<F32, DK, DV>), dim3(a.H, n_tiles),
                      dim3(256), lds2, st, a, tiles, (const float*)cs);
 }
 

@@ -76,6 +76,29 @@ DEVINL void load8(const typename Num<F32>::E* p, int valid, bool aligned,
   }
 }
 
+// The same 8 elements, still in storage form (for loads kept in flight).
+template <bool F32> struct Raw8 {
+  using E = typename Num<F32>::E;
+  E e[8];
+  DEVINL void load(const E* p, int valid, bool aligned) {
+    if (valid <= 0) {
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) e[i] = 0;
+    } else if (aligned) {
+      if constexpr (F32) {
+        *(f32x4*)e = *(const f32x4*)p;
+        *(f32x4*)(e + 4) = *(const f32x4*)(p + 4);
+      } else {
+        *(bf16x8*)e = *(const bf16x8*)p;
+      }
+    } else {
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) e[i] = i < valid ? p[i] : E(0);
+    }
+  }
+  DEVINL float operator[](int i) const { return Num<F32>::up(e[i]); }
+};
+
 // counterpart of load8; elements at or past `valid` are left alone
 template <bool F32>
 DEVINL void store8(typename Num<F32>::E* p, int valid, bool aligned,
@@ -113,11 +136,70 @@ template <bool F32> struct Split {
     hi[i] = h;
     if constexpr (!F32) lo[i] = N::down(v - N::up(h));
   }
+  DEVINL void put8(int i, const float* v) const {   // 16-byte aligned i
+    if constexpr (F32) {
+      *(f32x4*)(hi + i) = *(const f32x4*)v;
+      *(f32x4*)(hi + i + 4) = *(const f32x4*)(v + 4);
+    } else {
+      bf16x8 h, r;
+      #pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        h[j] = cvt_bf16(v[j]);
+        r[j] = cvt_bf16(v[j] - bf2f(h[j]));
+      }
+      *(bf16x8*)(hi + i) = h;
+      *(bf16x8*)(lo + i) = r;
+    }
+  }
   DEVINL Frag load(int row_off, int k) const {
     Frag f;
     f.hi = N::load(hi + row_off, k);
     if constexpr (!F32) f.lo = N::load(lo + row_off, k);
     return f;
+  }
+};
+
+// LDS tile of 64 tokens x D columns used as an operand whose k-index is
+// the token.  bf16: packed 4x16 subtiles, written 16 bytes at a time and
+// read transposed by ds_read_b64_tr_b16.  float: kept transposed.
+template <bool F32, int D> struct ColTile {
+  using N = Num<F32>;
+  using E = typename N::E;
+  static constexpr int LDJ = 64 + N::PAD;
+  static constexpr int SIZE = F32 ? D * LDJ : 64 * D;
+  E* p;
+  DEVINL void put8(int j, int c, const float* v) const {
+    if constexpr (F32) {
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) p[(c + i) * LDJ + j] = v[i];
+    } else {
+      bf16x8 t;
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) t[i] = cvt_bf16(v[i]);
+      put_raw(j, c, t);
+    }
+  }
+  DEVINL void put_raw(int j, int c, bf16x8 t) const {
+    *(bf16x8*)(p + ((j >> 2) * (D / 16) + (c >> 4)) * 64 + (j & 3) * 16 +
+               (c & 15)) = t;
+  }
+  // fragments of column tiles ct..ct+3 for tokens 32*kb..+31
+  DEVINL void frags4(int ct, int kb, int l, typename N::Frag (&f)[4]) const {
+    const int lr = l & 15, lg = l >> 4;
+    if constexpr (F32) {
+      #pragma unroll
+      for (int i = 0; i < 4; ++i)
+        f[i] = N::load(p + ((ct + i) * 16 + lr) * LDJ, kb * 32 + lg * 8);
+    } else {
+      constexpr unsigned Q = (D / 16) * 128;      // bytes of a 4-token band
+      const unsigned a = lds_byte_off(p) + (unsigned)(kb * 8 + 2 * lg) * Q +
+                         (unsigned)ct * 128 + (lr >> 2) * 32 + (lr & 3) * 8;
+      const bf16x8_quad q = tr_read_quad(a, a + Q, a + 128, a + Q + 128,
+                                         a + 256, a + Q + 256, a + 384,
+                                         a + Q + 384);
+      #pragma unroll
+      for (int i = 0; i < 4; ++i) f[i] = q.f[i];
+    }
   }
 };
 
