@@ -153,7 +153,8 @@ def require_lm_ext():
 def ensure_lm_ext():
     """require_lm_ext(), compiling it first if this checkout has none."""
     if _try_load(LM_EXT_NAME) is None:
-        build_extension(verbose=False, name=LM_EXT_NAME)
+        _LOADED[LM_EXT_NAME] = build_extension(verbose=False,
+                                               name=LM_EXT_NAME)
     return _require(LM_EXT_NAME)
 
 
