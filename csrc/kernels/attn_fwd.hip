@@ -148,6 +148,7 @@ void launch_fwd(const torch::Tensor& q, const torch::Tensor& k,
   if (D == 64) LAUNCH_D(64);
   else if (D == 128) LAUNCH_D(128);
   else if (D == 32) LAUNCH_D(32);
+  else if (D == 16) LAUNCH_D(16);
   else TORCH_CHECK(false, "attn_fwd: unsupported head dim ", D);
   #undef LAUNCH_D
 }
