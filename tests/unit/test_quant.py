@@ -69,6 +69,6 @@ def test_quantized_load_gpu(tmp_path):
     load_quantized(mg, p)
     tok = torch.randint(0, 128, (2, 16), device="cuda")
     la = mg(tok, tok).float().cpu()
-    lb = m(tok, tok).float()
+    lb = m(tok.cpu(), tok.cpu()).float()
     torch.cuda.synchronize()
     assert torch.allclose(la, lb, rtol=0.1, atol=0.1), (la, lb)
