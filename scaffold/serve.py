@@ -797,12 +797,14 @@ class ContinuousBatcher:
 def create_app(model: torch.nn.Module, max_batch: int = 8,
                window_s: float = DEFAULT_WINDOW_S, use_graph: bool = False,
                tokenizer=None, continuous: bool = False,
-               draft_model=None, draft_k: int = 4, worker=None):
+               draft_model=None, draft_k: int = 4, worker=None,
+               batcher_options: Optional[dict] = None):
     """FastAPI app around an inference worker.  `model` is an eval-mode
     LM from scaffold.models (tests inject a tiny CPU one).  Passing a
     `tokenizers.Tokenizer` adds the text endpoint /v1/completions.
     continuous=True serves from the ContinuousBatcher (slot-level
-    admission/retirement) instead of the same-shape batch worker."""
+    admission/retirement) instead of the same-shape batch worker;
+    batcher_options are further keyword arguments of that batcher."""
     from contextlib import asynccontextmanager
 
     from fastapi import FastAPI, HTTPException
@@ -810,7 +812,8 @@ def create_app(model: torch.nn.Module, max_batch: int = 8,
     if worker is None:
         if continuous:
             worker = ContinuousBatcher(model.eval(), max_slots=max_batch,
-                                       use_graph=use_graph)
+                                       use_graph=use_graph,
+                                       **(batcher_options or {}))
         else:
             worker = InferenceWorker(model.eval(), max_batch=max_batch,
                                      window_s=window_s, use_graph=use_graph,
@@ -1005,6 +1008,12 @@ def main(argv=None):
                          "'model.name=llama,model.n_layers=4')")
     ap.add_argument("--draft-config", default="")
     ap.add_argument("--draft-k", type=int, default=4)
+    ap.add_argument("--prefill-chunk", type=int, default=2048,
+                    help="paged models, --continuous: most prompt tokens "
+                         "per step")
+    ap.add_argument("--cache-tokens", type=int, default=0,
+                    help="paged models, --continuous: cache pool size in "
+                         "tokens (0: every slot at full length)")
     args = ap.parse_args(argv)
 
     import uvicorn
@@ -1043,7 +1052,9 @@ def main(argv=None):
         draft = draft.to(dev, dt).eval()
     app = create_app(model, max_batch=args.max_batch, use_graph=args.graph,
                      tokenizer=tok, continuous=args.continuous,
-                     draft_model=draft, draft_k=args.draft_k)
+                     draft_model=draft, draft_k=args.draft_k,
+                     batcher_options={"prefill_chunk": args.prefill_chunk,
+                                      "cache_tokens": args.cache_tokens})
     uvicorn.run(app, host=args.host, port=args.port, log_level="warning")
 
 

@@ -7,6 +7,7 @@ import os
 import queue
 import random
 import subprocess
+import sys
 
 import pytest
 import torch
@@ -394,11 +395,58 @@ def test_inference_worker_and_http():
             assert r.result == expected("looped", t[:9], 12)
     finally:
         w.close()
-    with TestClient(create_app(m, continuous=True, max_batch=2)) as client:
+    app = create_app(m, continuous=True, max_batch=2,
+                     batcher_options={"prefill_chunk": 4,
+                                      "cache_tokens": 128})
+    with TestClient(app) as client:
         r = client.post("/v1/generate", json={"tokens": [t[:9], t[:3]],
                                               "max_new_tokens": 12})
         assert r.json()["tokens"] == [expected("looped", t[:9], 12),
                                       expected("looped", t[:3], 12)]
+
+
+@dev_
+def test_serve_command_line(dev, tmp_path):
+    """The server program on a model folder, one request over HTTP."""
+    import socket
+    import time
+    import urllib.request
+
+    d = model_dir(tmp_path, "looped")
+    m = load_model_dir(d, torch.bfloat16 if dev == "cuda" else torch.float32,
+                       dev)
+    _, t, _ = make("looped", "cpu")
+    want = Generator(m).generate(torch.tensor([t[:9]], device=dev),
+                                 6)[0, 9:].tolist()
+    with socket.socket() as s:
+        s.bind(("127.0.0.1", 0))
+        port = s.getsockname()[1]
+    env = dict(os.environ)
+    if dev == "cpu":
+        env["HIP_VISIBLE_DEVICES"] = env["CUDA_VISIBLE_DEVICES"] = "-1"
+    p = subprocess.Popen(
+        [sys.executable, "-m", "scaffold.serve", f"model.dir={d}",
+         "model.max_seq_len=128", "--continuous", "--prefill-chunk", "4",
+         "--port", str(port)], cwd=REPO, env=env)
+    try:
+        req = urllib.request.Request(
+            f"http://127.0.0.1:{port}/v1/generate", method="POST",
+            data=json.dumps({"tokens": t[:9], "max_new_tokens": 6}).encode(),
+            headers={"Content-Type": "application/json"})
+        for _ in range(90):
+            assert p.poll() is None
+            try:
+                with urllib.request.urlopen(req, timeout=30) as r:
+                    got = json.load(r)["tokens"][0]
+                break
+            except OSError:
+                time.sleep(0.5)
+        assert len(got) == 6
+        if dev == "cpu":          # float32 there: the same greedy rollout
+            assert got == want == expected("looped", t[:9], 12)[:6]
+    finally:
+        p.terminate()
+        p.wait(20)
 
 
 @pytest.mark.gpu

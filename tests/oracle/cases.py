@@ -5,7 +5,7 @@ import random
 import torch
 
 from scaffold.cache import PagedStateCache, StateSpec, KVSpec
-from scaffold.config import load_config, read_model_dir
+from scaffold.config import load_config
 from scaffold.convert import load_stack
 from scaffold.models import build_model
 
@@ -136,5 +136,4 @@ def cuts(n, sizes):
 
 
 __all__ = ["attn", "ret", "config", "CONFIGS", "weights", "build", "tokens",
-           "poison", "op_cache", "cuts", "KVSpec", "StateSpec",
-           "read_model_dir"]
+           "poison", "op_cache", "cuts", "KVSpec", "StateSpec"]
