@@ -10,6 +10,7 @@ dispatch on the GPU path; eager is the CPU test path only).
 
 from __future__ import annotations
 
+import glob
 import importlib.util
 import os
 import sys
@@ -95,8 +96,12 @@ def build_extension(verbose: bool = True, name: str = EXT_NAME):
     )
 
 
-def build_all(verbose: bool = True) -> None:
-    for name in _EXTS:
+def build_all(verbose: bool = True, force: bool = False) -> None:
+    """Build every extension; force recompiles what is already built."""
+    for name, spec in _EXTS.items():
+        if force:
+            for o in glob.glob(os.path.join(spec["dir"], "*.o")):
+                os.unlink(o)
         build_extension(verbose=verbose, name=name)
 
 
