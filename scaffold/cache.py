@@ -7,7 +7,9 @@ shared by all attention layer runs (each has its own key/value or latent
 tensors of the same page count); a recurrent layer run keeps one state per
 slot, which may consist of several tensors.
 Layers that run several times in a forward pass are separate runs here,
-so every pass has its own keys, values and state.
+so every pass has its own keys, values and state.  A layer may have both
+pages and a state; what a model keeps of a sequence beside its mixers (the
+previous token, the inputs that a shift looks back at) are runs of their own.
 
 A freed page or slot is handed out again as it is: nothing is cleared.
 Kernels never read a key that the sequence did not write, and a sequence
@@ -58,9 +60,10 @@ class LatentSpec:
 
 @dataclass(frozen=True)
 class StateSpec:
-    """What one run of a recurrent layer keeps per sequence: float32
-    tensors of these shapes."""
+    """What one run of a recurrent layer keeps per sequence: tensors of
+    these shapes, float32 unless said otherwise."""
     shapes: Tuple[Tuple[int, ...], ...]
+    dtype: torch.dtype = torch.float32
 
 
 def _pad8(n: int) -> int:
@@ -129,8 +132,10 @@ Entry = Tuple[int, object, Sequence[int]]
 class PagedStateCache:
     def __init__(self, specs: Sequence[object], n_slots: int, n_tokens: int,
                  max_len: int, device, dtype):
-        """n_tokens: pool size in tokens (rounded up to whole pages);
-        max_len: the longest sequence a slot can hold."""
+        """specs: one per run, or a tuple of them (one of what tokens leave
+        in pages, any of what a sequence keeps); n_tokens: pool size in tokens
+        (rounded up to whole pages); max_len: the longest sequence a slot can
+        hold."""
         self.device = torch.device(device)
         self.specs = list(specs)
         self.n_slots = n_slots
@@ -140,30 +145,31 @@ class PagedStateCache:
         self.k: List[Optional[torch.Tensor]] = []
         self.v: List[Optional[torch.Tensor]] = []
         self.state: List[Optional[Tuple[torch.Tensor, ...]]] = []
-        for s in self.specs:
-            if isinstance(s, KVSpec):
-                self.k.append(torch.zeros(self.n_pages, s.kv_heads, PAGE, s.dim,
-                                          device=device, dtype=dtype))
-                self.v.append(torch.zeros(self.n_pages, s.kv_heads, PAGE, s.vdim,
-                                          device=device, dtype=dtype))
-                self.state.append(None)
-            elif isinstance(s, TiedSpec):
-                self.k.append(torch.zeros(self.n_pages, s.kv_heads, PAGE, s.dim,
-                                          device=device, dtype=dtype))
-                self.v.append(torch.zeros(self.n_pages, PAGE, device=device,
-                                          dtype=torch.float32))
-                self.state.append(None)
-            elif isinstance(s, LatentSpec):
-                self.k.append(torch.zeros(self.n_pages, PAGE, s.row,
-                                          device=device, dtype=dtype))
-                self.v.append(None)
-                self.state.append(None)
-            else:
-                self.state.append(tuple(
-                    torch.zeros(n_slots, *shape, device=device,
-                                dtype=torch.float32) for shape in s.shapes))
-                self.k.append(None)
-                self.v.append(None)
+        for spec in self.specs:
+            k = v = state = None
+            for s in spec if isinstance(spec, tuple) else (spec,):
+                if isinstance(s, StateSpec):
+                    state = (state or ()) + tuple(
+                        torch.zeros(n_slots, *shape, device=device,
+                                    dtype=s.dtype) for shape in s.shapes)
+                    continue
+                if k is not None:
+                    raise ValueError("a run has one cache of tokens")
+                if isinstance(s, LatentSpec):
+                    k = torch.zeros(self.n_pages, PAGE, s.row, device=device,
+                                    dtype=dtype)
+                    continue
+                k = torch.zeros(self.n_pages, s.kv_heads, PAGE, s.dim,
+                                device=device, dtype=dtype)
+                if isinstance(s, KVSpec):
+                    v = torch.zeros(self.n_pages, s.kv_heads, PAGE, s.vdim,
+                                    device=device, dtype=dtype)
+                else:
+                    v = torch.zeros(self.n_pages, PAGE, device=device,
+                                    dtype=torch.float32)
+            self.k.append(k)
+            self.v.append(v)
+            self.state.append(state)
         self.table = torch.zeros(n_slots, self.max_pages, dtype=torch.int32,
                                  device=device)
         self._pages: List[List[int]] = [[] for _ in range(n_slots)]

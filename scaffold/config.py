@@ -18,7 +18,7 @@ import hashlib
 import json
 import os
 from dataclasses import dataclass, field
-from typing import Any, Dict, List, Optional
+from typing import Any, Dict, List, Optional, Tuple
 
 SCHEMA_VERSION = 1
 
@@ -26,7 +26,7 @@ SCHEMA_VERSION = 1
 @dataclass
 class ModelConfig:
     # mlp | resnet50 | gpt2 | llama3_8b | llama (custom dims) | lasezen |
-    # nekozen | babodra
+    # nekozen | babodra | tilivik
     name: str = "mlp"
     # a model folder: config.json (its "architecture" picks the name and
     # fills the fields below) beside model.safetensors
@@ -77,17 +77,27 @@ class ModelConfig:
     layers: List[Any] = field(default_factory=list)
     loop: Optional[Dict[str, int]] = None
     residual_mult: float = 1.0
-    # the stack's norms (layer_norm | rms_norm | dynamic_tanh), whether
-    # sublayers have one before and one after them, the number of learned
-    # position vectors (0: none), whether each pass of the loop starts from a
-    # projection of the stream and the embeddings, and the soft cap of the
-    # logits (0: none)
+    # the stack's norms (layer_norm | rms_norm | scalar_rms_norm |
+    # dynamic_tanh), whether sublayers have one before and one after them,
+    # the number of learned position vectors (0: none), whether each pass of
+    # the loop starts from a projection of the stream and the embeddings, and
+    # the soft cap of the logits (0: none)
     norm: str = "layer_norm"
     pre_norm: bool = True
     post_norm: bool = True
     positions: int = 0
     loop_input: bool = False
     logit_softcap: float = 0.0
+    # whether the embeddings are added to the stream before each pass of the
+    # loop but the first, and a vector of its own before each pass
+    loop_add: bool = False
+    # base of the sinusoidal position vectors that embeddings take (0: none),
+    # the table that adds a vector per pair of neighbouring tokens
+    # ({"buckets", "mul_prev", "mul_cur"}), and whether a mixer's input is
+    # blended with the previous token's
+    sinusoid_base: float = 0.0
+    bigram: Optional[Dict[str, int]] = None
+    token_shift: bool = False
 
 
 @dataclass
@@ -283,7 +293,11 @@ def load_config(path: Optional[str] = None, overrides: Optional[List[str]] = Non
     return cfg
 
 
-def _lasezen_fields(d: Dict[str, Any]) -> Dict[str, Any]:
+# shapes of a checkpoint's tensors by name: some sizes stand only there
+Shapes = Dict[str, Tuple[int, ...]]
+
+
+def _lasezen_fields(d: Dict[str, Any], shapes: Shapes) -> Dict[str, Any]:
     return {"name": "lasezen", "vocab_size": d["vocab"],
             "d_model": d["width"], "n_layers": len(d["layers"]),
             "norm_eps": d["norm"]["eps"],
@@ -297,7 +311,7 @@ def _lasezen_fields(d: Dict[str, Any]) -> Dict[str, Any]:
 _NEKOZEN = {"norm": "dynamic_tanh", "post_norm": False, "loop_input": True}
 
 
-def _nekozen_fields(d: Dict[str, Any]) -> Dict[str, Any]:
+def _nekozen_fields(d: Dict[str, Any], shapes: Shapes) -> Dict[str, Any]:
     same = ("latent_attention", "mamba2", "mlstm")
     layers = _renamed(d["layers"], {n: n for n in same},
                       {"dense": "gated"})  # its dense layer has a gate
@@ -312,13 +326,44 @@ def _nekozen_fields(d: Dict[str, Any]) -> Dict[str, Any]:
 _BABODRA = {"norm": "rms_norm", "pre_norm": False, "post_norm": True}
 
 
-def _babodra_fields(d: Dict[str, Any]) -> Dict[str, Any]:
+def _babodra_fields(d: Dict[str, Any], shapes: Shapes) -> Dict[str, Any]:
     return {"name": "babodra", "vocab_size": d["vocab"],
             "d_model": d["width"], "n_layers": len(d["layers"]),
             "norm_eps": d["norm"]["eps"],
             "layers": _renamed(d["layers"], {"attention": "tied_attention"},
                                {"dense": "clamped", "moe": "moe"}),
             "positions": d["max_positions"], **_BABODRA}
+
+
+# what the Tilivik design fixes for every model of it
+_TILIVIK = {"norm": "scalar_rms_norm", "post_norm": False, "loop_add": True,
+            "sinusoid_base": 10000.0, "token_shift": True}
+
+
+def _tilivik_fields(d: Dict[str, Any], shapes: Shapes) -> Dict[str, Any]:
+    layers = _renamed(d["layers"], {"lightning": "lightning",
+                                    "parallel": "parallel"},
+                      {"moe": "table_moe"})
+
+    def size(name: str, axis: int) -> int:
+        if name not in shapes:
+            raise ValueError(f"the shape of {name!r} is needed: no such "
+                             "tensor in the checkpoint")
+        return shapes[name][axis]
+
+    for i, s in enumerate(layers):
+        if s["type"] == "parallel":
+            mx, p = s["mixer"], f"l{i}.mix."
+            s["mixer"] = dict(
+                mx, left=dict(mx["left"], type="window_attention",
+                              buckets=size(p + "left.rel", 0)),
+                right=dict(mx["right"], type="gla",
+                           rank=size(p + "right.a1", 0)))
+    return {"name": "tilivik", "vocab_size": d["vocab"],
+            "d_model": d["width"], "n_layers": len(layers),
+            "norm_eps": d["norm"]["eps"], "layers": layers,
+            "loop": d.get("loop"), "bigram": d["embedding"]["bigram"],
+            **_TILIVIK}
 
 
 def _renamed(layers: List[Any], mixers: Dict[str, str], ffs: Dict[str, str]
@@ -342,7 +387,18 @@ def _renamed(layers: List[Any], mixers: Dict[str, str], ffs: Dict[str, str]
 
 # config.json "architecture" -> reader of that file's keys
 ARCHITECTURES = {"Lasezen": _lasezen_fields, "Nekozen": _nekozen_fields,
-                 "Babodra": _babodra_fields}
+                 "Babodra": _babodra_fields, "Tilivik": _tilivik_fields}
+
+
+def tensor_shapes(path: str) -> Shapes:
+    """Shapes of a safetensors file's tensors, from its header; of a file
+    that is not there, none."""
+    if not os.path.exists(path):
+        return {}
+    with open(path, "rb") as fh:
+        head = json.loads(fh.read(int.from_bytes(fh.read(8), "little")))
+    return {n: tuple(t["shape"]) for n, t in head.items()
+            if n != "__metadata__"}
 
 
 def read_model_dir(path: str) -> Dict[str, Any]:
@@ -353,7 +409,8 @@ def read_model_dir(path: str) -> Dict[str, Any]:
     if arch not in ARCHITECTURES:
         raise ValueError(f"{path}: unknown architecture {arch!r} (known: "
                          f"{', '.join(sorted(ARCHITECTURES))})")
-    return ARCHITECTURES[arch](d)
+    return ARCHITECTURES[arch](
+        d, tensor_shapes(os.path.join(path, "model.safetensors")))
 
 
 def _apply_model_preset(cfg: TrainConfig) -> None:
@@ -362,7 +419,7 @@ def _apply_model_preset(cfg: TrainConfig) -> None:
     if m.dir:
         for k, v in read_model_dir(m.dir).items():
             setattr(m, k, v)
-    fixed = {"nekozen": _NEKOZEN, "babodra": _BABODRA}
+    fixed = {"nekozen": _NEKOZEN, "babodra": _BABODRA, "tilivik": _TILIVIK}
     for k, v in fixed.get(m.name, {}).items():
         setattr(m, k, v)
     if m.positions:

@@ -349,7 +349,12 @@ def load_stack(model: MixerStack, sd: Dict[str, torch.Tensor]) -> None:
         for p in model.parameters():
             p.zero_()
         for n, dst in want:
+            if dst.is_floating_point() != sd[n].is_floating_point():
+                raise ValueError(f"{n}: {sd[n].dtype}, expected {dst.dtype}")
             dst.copy_(sd[n])
+        for mod in model.modules():
+            if hasattr(mod, "check"):
+                mod.check()
 
 
 def to_stack(model: MixerStack) -> Dict[str, torch.Tensor]:

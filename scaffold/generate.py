@@ -7,8 +7,8 @@ single new query against the cache.  The decode GEMVs take the library
 path — the hand decode_gemv kernel measured below hipBLASLt in-graph
 and is parked behind SCAFFOLD_DECODE_GEMV=1 (NOTES r2 serving ladder).
 Model families: GPT-2 (LayerNorm/GELU), Llama (RMSNorm/RoPE/GQA/SwiGLU)
-and mixer stacks (Lasezen, Nekozen, Babodra), which keep a paged cache with
-state slots (scaffold.cache) and run every call as one ragged batch (step);
+and mixer stacks (Lasezen, Nekozen, Babodra, Tilivik), which keep a paged
+cache with state slots (scaffold.cache) and run every call as one ragged batch (step);
 greedy / temperature / top-k / top-p sampling with optional EOS; hipGraph-replayed static decode (generate_graphed); per-row
 variable-position decode for continuous batching (decode_step_varpos);
 speculative decoding (generate_speculative); TP-sharded models reduce

@@ -1,5 +1,5 @@
 """Model zoo (contract C9): MLP, ResNet-50, GPT-2-small, Llama-3-8B, and
-mixer-stack models (Lasezen, Nekozen, Babodra)."""
+mixer-stack models (Lasezen, Nekozen, Babodra, Tilivik)."""
 
 from __future__ import annotations
 
@@ -25,6 +25,6 @@ def build_model(cfg) -> torch.nn.Module:
         return GPT2(cfg)
     if name in ("llama", "llama3_8b"):
         return Llama(cfg)
-    if name in ("lasezen", "nekozen", "babodra"):
+    if name in ("lasezen", "nekozen", "babodra", "tilivik"):
         return MixerStack(cfg)
     raise ValueError(f"unknown model {name!r}")

@@ -9,10 +9,12 @@ come from scaffold.models.mixers.  The residual stream is float32
 throughout.
 
 What a configuration can choose besides the layers: the kind of norm,
-whether sublayers have one before them, after them or both, learned
-position vectors, a factor of every sublayer, a projection of the stream
-and the embeddings before each pass of the repeated span, and a soft cap
-on the logits.
+whether sublayers have one before them, after them or both, learned or
+sinusoidal position vectors, a vector per pair of neighbouring tokens, a
+blend of every mixer's input with the previous token's, a factor of every
+sublayer, what happens before each pass of the repeated span (a projection of
+the stream and the embeddings, or the embeddings and a vector of the pass
+added to the stream), and a soft cap on the logits.
 """
 
 from __future__ import annotations
@@ -23,7 +25,7 @@ import torch
 import torch.nn as nn
 
 from .. import ops
-from ..cache import PagedStateCache, StepPlan
+from ..cache import PagedStateCache, StateSpec, StepPlan
 from .gpt2 import LayerNorm
 from .mixers import FEED_FORWARDS, MIXERS
 
@@ -46,8 +48,16 @@ class RMSNorm(nn.Module):
         self.weight = nn.Parameter(torch.ones(width))
 
 
+class ScalarRMSNorm(nn.Module):
+    """x over its root mean square, times one number."""
+
+    def __init__(self, width: int, eps: float):
+        super().__init__()
+        self.weight = nn.Parameter(torch.ones(()))
+
+
 NORMS = {"layer_norm": LayerNorm, "rms_norm": RMSNorm,
-         "dynamic_tanh": DynamicTanh}
+         "scalar_rms_norm": ScalarRMSNorm, "dynamic_tanh": DynamicTanh}
 
 
 def _lookup(table: dict, name: str, what: str):
@@ -58,8 +68,8 @@ def _lookup(table: dict, name: str, what: str):
 
 
 class StackLayer(nn.Module):
-    """One layer: (norm1 ->) mixer (-> norm1b), then (if it has one)
-    (norm2 ->) feed-forward (-> norm2b)."""
+    """One layer: (norm1 ->) (blend with the previous token's ->) mixer
+    (-> norm1b), then (if it has one) (norm2 ->) feed-forward (-> norm2b)."""
 
     def __init__(self, m, spec: dict):
         super().__init__()
@@ -69,12 +79,14 @@ class StackLayer(nn.Module):
         for n in ("norm1", "norm2")[:1 if ff is None else 2]:
             setattr(self, n, norm(width, eps) if m.pre_norm else None)
             setattr(self, n + "b", norm(width, eps) if m.post_norm else None)
+        self.shift = (nn.Parameter(torch.full((width,), 0.5))
+                      if m.token_shift else None)
         self.mixer = _lookup(MIXERS, spec["type"], "mixer")(
             width, spec["mixer"], eps)
         self.ff = None
         if ff is not None:
             self.ff = _lookup(FEED_FORWARDS, ff["kind"], "feed-forward")(
-                width, ff)
+                width, ff, m.vocab_size)
 
 
 def _params(norm) -> Optional[tuple]:
@@ -107,6 +119,21 @@ class MixerStack(nn.Module):
         if m.positions:
             self.pos = nn.Embedding(m.positions, m.d_model)
             self.max_seq_len = min(m.max_seq_len, m.positions)
+        # a vector per pair of neighbouring tokens, the last row for a
+        # sequence's first token; turns per position of sinusoidal vectors
+        self.bigram = None
+        if m.bigram:
+            self.pair_mul = m.bigram["mul_prev"], m.bigram["mul_cur"]
+            self.bigram = nn.Embedding(m.bigram["buckets"] + 1, m.d_model)
+        self.sinusoid_base = float(m.sinusoid_base)
+        self._rates: Dict[str, torch.Tensor] = {}
+        if m.positions and (self.bigram is not None or self.sinusoid_base):
+            raise ValueError("learned positions beside sinusoids or pairs")
+        # streams that make a mixer's input in shift_norm
+        self.shifted = m.token_shift
+        if (m.token_shift or m.loop_add) and (m.post_norm or not m.pre_norm
+                                              or m.loop_input):
+            raise ValueError("token_shift and loop_add go with pre_norm alone")
         self.blocks = nn.ModuleList(StackLayer(m, s) for s in m.layers)
         self.norm_f = _lookup(NORMS, m.norm, "norm")(m.d_model, m.norm_eps)
         self.lm_head = nn.Linear(m.d_model, m.vocab_size, bias=False)
@@ -118,14 +145,16 @@ class MixerStack(nn.Module):
         # the layers in running order; position in this list = cache run
         self.runs: List[int] = [*range(lo), *([*range(lo, hi)] * times),
                                 *range(hi, n)]
-        # runs that begin a pass whose input is a projection of the stream
-        # and the embeddings -> the number of the pass
+        # runs that begin a pass with something of their own (loop_input,
+        # loop_add) -> the number of the pass
         self.entries: Dict[int, int] = {}
-        if m.loop and m.loop_input:
+        self.loop_in = None
+        if m.loop and (m.loop_input or m.loop_add):
             if lo == hi:
                 raise ValueError(f"loop {loop} repeats no layer")
             self.entries = {lo + t * (hi - lo): t for t in range(times)}
-            self.loop_in = nn.Linear(2 * m.d_model, m.d_model, bias=False)
+            if m.loop_input:
+                self.loop_in = nn.Linear(2 * m.d_model, m.d_model, bias=False)
             self.loop_step = nn.Parameter(torch.zeros(times, m.d_model))
         for p in self.parameters():
             if p.dim() > 1:
@@ -144,9 +173,12 @@ class MixerStack(nn.Module):
         out = [("embed", self.embed.weight)]
         if self.pos is not None:
             out.append(("pos", self.pos.weight))
+        if self.bigram is not None:
+            out.append(("bigram", self.bigram.weight))
+        if self.loop_in is not None:
+            out.append(("loop.in", self.loop_in.weight))
         if self.entries:
-            out += [("loop.in", self.loop_in.weight),
-                    ("loop.step", self.loop_step)]
+            out.append(("loop.step", self.loop_step))
         for i, blk in enumerate(self.blocks):
             for n in ("norm1", "norm1b", "norm2", "norm2b"):
                 if getattr(blk, n, None) is not None:
@@ -156,6 +188,8 @@ class MixerStack(nn.Module):
             out += [(f"l{i}.mix.{n}", t) for n, t in blk.mixer.packed()]
             if blk.ff is not None:
                 out += [(f"l{i}.mlp.{n}", t) for n, t in blk.ff.packed()]
+            if blk.shift is not None:
+                out.append((f"l{i}.shift", blk.shift))
         return out + norm("final.norm", self.norm_f) + [
             ("head", self.lm_head.weight)]
 
@@ -165,9 +199,29 @@ class MixerStack(nn.Module):
         w = self.embed.weight
         if self.pos is not None:
             max_len = min(max_len, self.pos.num_embeddings)
-        return PagedStateCache([self.blocks[i].mixer.cache_spec()
-                                for i in self.runs], n_slots, n_tokens,
-                               max_len, w.device, w.dtype)
+        specs = [self.blocks[i].mixer.cache_spec() for i in self.runs]
+        # behind the layer runs: what their inputs look back at, then the
+        # token before
+        if self.shifted:
+            specs += [StateSpec(((w.shape[1],),))] * len(self.runs)
+        if self.bigram is not None:
+            specs.append(StateSpec(((),), torch.int64))
+        return PagedStateCache(specs, n_slots, n_tokens, max_len, w.device,
+                               w.dtype)
+
+    def _embed(self, plan: StepPlan, cache: PagedStateCache) -> torch.Tensor:
+        """The stream as the embeddings leave it (sinusoids, pairs)."""
+        w, rates = self.embed.weight, None
+        if self.sinusoid_base:
+            key = str(w.device)
+            if key not in self._rates:
+                self._rates[key] = ops.turn_rates(w.shape[1],
+                                                  self.sinusoid_base, w.device)
+            rates = self._rates[key]
+        if self.bigram is None:
+            return ops.stream_embed(plan, w, rates=rates)
+        return ops.stream_embed(plan, w, rates=rates, pairs=self.bigram.weight,
+                                mul=self.pair_mul, last=cache.state[-1][0])
 
     def _logits(self, h: torch.Tensor) -> torch.Tensor:
         if not self.softcap:
@@ -182,6 +236,10 @@ class MixerStack(nn.Module):
         (rows, vocab).  Keys, values and states go into the cache.
         on_layer(run, x) sees the residual stream after every layer run."""
         blocks, eps, embed = self.blocks, self.eps, self.embed.weight
+        last = len(self.runs) - 1
+        rows = plan.rows
+        own_start = bool(self.sinusoid_base) or self.bigram is not None
+        added = bool(self.entries) and self.loop_in is None
 
         def first(run):
             return _params(blocks[self.runs[run]].norm1)
@@ -192,16 +250,36 @@ class MixerStack(nn.Module):
                                        plan.tokens, embed)
             if on_layer is not None and run:
                 on_layer(run - 1, x)
-            return ops.replace_norm(
+            return x, ops.replace_norm(
                 x, ops.linear_f32(both, self.loop_in.weight),
                 self.loop_step[self.entries[run]], first(run), eps)
 
-        x, h = ops.embed_norm(plan.tokens, embed, first(0), eps, plan.pos,
-                              None if self.pos is None else self.pos.weight)
-        if 0 in self.entries:
-            h = begin_pass(0, x, None, None)
-        last = len(self.runs) - 1
-        rows = plan.rows
+        def mixer_input(run, x, y):
+            """The stream with y added, what begins a pass included, and
+            run's input."""
+            blk, n = blocks[self.runs[run]], self.entries.get(run)
+            if on_layer is not None and run:
+                x, _ = ops.shift_norm(x, y, self.mult, first(run), eps, plan)
+                on_layer(run - 1, x)
+                y = None
+            state = cache.state[last + 1 + run][0] if self.shifted else None
+            return ops.shift_norm(
+                x, y, self.mult, first(run), eps, plan, shift=blk.shift,
+                state=state, add=start if n else None,
+                step=None if n is None else self.loop_step[n])
+
+        if own_start:
+            start = x = self._embed(plan, cache)
+            if not (self.shifted or added):
+                h = ops.residual_norm(x, None, None, 1.0, first(0), eps)
+        else:
+            x, h = ops.embed_norm(plan.tokens, embed, first(0), eps, plan.pos,
+                                  None if self.pos is None else self.pos.weight)
+            start = x
+        if self.shifted or added:
+            x, h = mixer_input(0, x, None)
+        elif 0 in self.entries:
+            x, h = begin_pass(0, x, None, None)
         for run, i in enumerate(self.runs):
             blk = blocks[i]
             end = run == last
@@ -213,9 +291,12 @@ class MixerStack(nn.Module):
             if blk.ff is not None:
                 h = ops.residual_norm(x, y, _params(post), self.mult,
                                       _params(blk.norm2), eps)
-                y, post = blk.ff.step(h), blk.norm2b
+                y, post = blk.ff.step(h, plan), blk.norm2b
+            if not end and (self.shifted or added):
+                x, h = mixer_input(run + 1, x, y)
+                continue
             if run + 1 in self.entries:
-                h = begin_pass(run + 1, x, y, _params(post))
+                x, h = begin_pass(run + 1, x, y, _params(post))
                 continue
             # only wanted rows pass the last norm, unless someone watches x
             few = end and rows is not None and on_layer is None

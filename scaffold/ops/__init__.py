@@ -18,10 +18,12 @@ import torch.nn.functional as F
 
 from . import backend
 from .backend import require_ext, require_lm_ext, has_ext, ext  # re-export
-from .lm import (Parts, clamped_glu, decay_tables, embed_norm, geglu_tanh,
-                 gelu_erf, latent_attention, linear_f32, mamba2, mlstm, moe,
-                 paged_attention, replace_norm, residual_concat, residual_norm,
-                 retention, rope_tables_exact, softcap, tied_attention)
+from .lm import (Parts, clamped_glu, decay_tables, distance_bias, embed_norm,
+                 geglu_tanh, gelu_erf, gla, latent_attention, lightning,
+                 linear_f32, mamba2, mlstm, moe, paged_attention, replace_norm,
+                 residual_concat, residual_norm, retention, rope_tables_exact,
+                 shift_norm, softcap, stream_embed, table_moe, tied_attention,
+                 turn_rates, window_attention)
 
 __all__ = [
     "layer_norm",
@@ -38,6 +40,14 @@ __all__ = [
     "fused_adamw_step",
     "batch_norm_act",
     "embed_norm",
+    "stream_embed",
+    "turn_rates",
+    "shift_norm",
+    "lightning",
+    "gla",
+    "window_attention",
+    "distance_bias",
+    "table_moe",
     "residual_norm",
     "residual_concat",
     "replace_norm",

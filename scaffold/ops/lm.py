@@ -1,7 +1,7 @@
-"""Ops of the mixer-stack models (paged, tied and latent attention,
-retention, state-space and matrix-memory recurrences, routed experts,
-residual norms).  GPU tensors
-run the HIP kernels of csrc/lm, required; CPU tensors run the plain float32
+"""Ops of the mixer-stack models (paged, tied, window and latent attention,
+retention, gated linear attention, state-space and matrix-memory
+recurrences, routed experts, embeddings, residual norms).  GPU tensors run
+the HIP kernels of csrc/lm, required; CPU tensors run the plain float32
 forms below, which the CPU tests use.
 """
 
@@ -66,8 +66,8 @@ class Parts(NamedTuple):
         return (self.y.float() * self.weights.unsqueeze(2)).sum(1)
 
 
-# A norm is given as its parameters: (weight,) is an RMS norm, (weight,
-# bias or None) a layer norm, (weight, bias, alpha) a dynamic tanh, None
+# A norm is given as its parameters: (weight,) is an RMS norm (its weight may
+# be a single number), (weight, bias or None) a layer norm, (weight, bias, alpha) a dynamic tanh, None
 # leaves its input as it is.
 def _norm(x, p, eps):
     if p is None:
@@ -110,6 +110,74 @@ def embed_norm(tokens, embed, norm, eps, pos=None, positions=None):
     if positions is not None:
         x = x + positions[pos.long()].float()
     return x, _norm(x, norm, eps).to(embed.dtype)
+
+
+def turn_rates(width: int, base: float, device) -> torch.Tensor:
+    """(width/2, rounded up) float64: what entries 2i and 2i+1 of a
+    sinusoidal position vector turn by per position, base^(-2i/width), in
+    whole turns."""
+    i = torch.arange(-(-width // 2), dtype=torch.float64)
+    return (float(base) ** (-2.0 * i / width) / (2 * math.pi)).to(device)
+
+
+def _before(t, plan, state):
+    """Rows t (T, ...) of a ragged batch moved down by one token: each gets
+    its predecessor's, a sequence's first one zeros, a portion's first one
+    what `state` kept; then state keeps the portions' last rows."""
+    out = torch.zeros_like(t)
+    for r0, n, p0, s in _portions(plan):
+        out[r0 + 1:r0 + n] = t[r0:r0 + n - 1]
+        if p0:
+            out[r0] = state[s]
+        state[s] = t[r0 + n - 1]
+    return out
+
+
+def stream_embed(plan, embed, *, rates=None, pairs=None, mul=(0, 0),
+                 last=None):
+    """Residual stream x (float32) of a ragged batch's tokens: their
+    embeddings, plus (rates: turn_rates) sinusoidal position vectors, plus
+    (pairs: a table) row (previous * mul[0] + token * mul[1]) mod (rows - 1),
+    for a sequence's first token the last row.  last (slots,) int64: the
+    token before, kept per slot."""
+    if embed.is_cuda:
+        return require_lm_ext().stream_embed(
+            plan.tokens, embed, plan.pos, plan.slot, plan.tiles, plan.seqs,
+            plan.n_dec, rates, pairs, *mul, last)
+    x = embed[plan.tokens].float()
+    if pairs is not None:
+        n = pairs.shape[0] - 1
+        row = (_before(plan.tokens, plan, last) * mul[0]
+               + plan.tokens * mul[1]) % n
+        x = x + pairs[row.masked_fill(plan.pos == 0, n)].float()
+    if rates is not None:
+        turns = plan.pos.double().unsqueeze(1) * rates
+        ang = 2 * math.pi * (turns - turns.floor())
+        x = x + torch.stack([ang.sin(), ang.cos()], 2).flatten(1)[
+            :, :x.shape[1]].float()
+    return x
+
+
+def shift_norm(x, y, mult, nxt, eps, plan, *, shift=None, state=None, add=None,
+               step=None):
+    """A new stream x + mult * y + add + step (y: (T, W), Parts or None; add:
+    a float32 stream or None; step: a vector or None) and its norm, which
+    (shift: a vector) is blended with the previous token's, h + (h' - h) *
+    shift.  state (slots, W) keeps a sequence's last h, unblended; None:
+    nobody looks back at these."""
+    if x.is_cuda:
+        return require_lm_ext().shift_norm(
+            x, *_yw(y), mult, *_wba(nxt), eps, plan.pos, plan.slot, plan.tiles,
+            plan.seqs, plan.n_dec, shift, state, add, step)
+    z = x.clone() if y is None else _advance(x, y, None, mult, eps)
+    if add is not None:
+        z = z + add
+    if step is not None:
+        z = z + step.float()
+    h = _norm(z, nxt, eps)
+    if shift is not None:
+        h = h + (_before(h, plan, state) - h) * shift.float()
+    return z, h.to(nxt[0].dtype)
 
 
 def residual_norm(x, y, post, mult, nxt, eps, rows=None, store_x=True):
@@ -205,10 +273,14 @@ def _rms(x, eps, w=None):
     return y if w is None else y * w.float()
 
 
-def _attend(q, k, v, pos, j, *, size, scale, sink, slopes):
+def _attend(q, k, v, pos, j, *, size, scale, sink=None, slopes=None,
+            keep=None, softcap=0.0, bias=None):
     """q (n, H, d) at positions pos over keys k, values v (m, G, .) at
     positions j -> (n, H, e), float32.  sink: (H,) scores without a value,
-    or None; slopes: (H,) off the scores per step of distance, or None."""
+    or None; slopes: (H,) off the scores per step of distance, or None; size:
+    chunk length or (keep is a number) window length beside which the first
+    `keep` tokens stay visible; bias: (H, n) added per distance, the last
+    column from there on."""
     n, H, _ = q.shape
     rep = H // k.shape[1]
     kk = k.float().repeat_interleave(rep, 1)
@@ -217,8 +289,15 @@ def _attend(q, k, v, pos, j, *, size, scale, sink, slopes):
     if slopes is not None:
         dist = (pos[:, None] - j[None]).float()
         sc = sc - slopes.float().view(-1, 1, 1) * dist
+    if softcap:
+        sc = softcap * torch.tanh(sc / softcap)
+    if bias is not None:
+        dist = (pos[:, None] - j[None]).clamp(0, bias.shape[1] - 1)
+        sc = sc + bias[:, dist]
     see = j[None] <= pos[:, None]
-    if size:
+    if size and keep is not None:
+        see &= (pos[:, None] - j[None] < size) | (j[None] < keep)
+    elif size:
         see &= j[None] // size == pos[:, None] // size
     sc = sc.masked_fill(~see, float("-inf"))
     if sink is not None:
@@ -261,6 +340,61 @@ def paged_attention(qkv, cache, run, plan, *, heads, q_norm, k_norm, sink,
             q[r0:r0 + n], kc[cell, :, j % page], vc[cell, :, j % page], i, j,
             size=size, scale=scale, sink=sink, slopes=slopes).to(qkv.dtype)
     return out.reshape(qkv.shape[0], heads * vdim)
+
+
+def distance_bias(rel: torch.Tensor, far: int) -> torch.Tensor:
+    """(heads, far + 1) float32: a learned table rel (rows, heads) laid out
+    by distance.  The first half of the rows belongs to the distances below
+    rows/2 one by one, the others share what follows up to `far` by its
+    logarithm (Raffel et al., "Exploring the Limits of Transfer Learning with
+    a Unified Text-to-Text Transformer"); the last one also has all beyond."""
+    rows = rel.shape[0]
+    half = rows // 2
+
+    def row(n):
+        if n < half:
+            return n
+        t = math.log(n / half) / math.log(far / half)
+        return min(rows - 1, half + math.floor(t * (rows - half)))
+
+    pick = torch.tensor([row(n) for n in range(far + 1)], device=rel.device)
+    return rel.detach()[pick].float().t().contiguous()
+
+
+def window_attention(x, col, out, out_col, cache, run, plan, *, heads, bias,
+                     softcap, size, keep, scale, out_scale, eps):
+    """Attention of a ragged batch over the last `size` tokens (0: all) and
+    the first `keep`; appends its keys and values to run `run` of the cache.
+    x's columns from `col` on are [q | k | v | gate]; each head's value is
+    divided by its root mean square.  Scores are capped (softcap, 0: not),
+    then take bias (heads, n) by distance.  The result, times the gate's
+    sigmoid and out_scale, goes to out's columns from out_col on."""
+    kc, vc = cache.k[run], cache.v[run]
+    if x.is_cuda:
+        return require_lm_ext().window_attention(
+            x, col, out, out_col, kc, vc, cache.table, plan.pos, plan.slot,
+            plan.tiles, plan.n_dec, bias, softcap, heads, size, keep, scale,
+            out_scale, eps, cache.max_len)
+    G, page, dim, vdim = kc.shape[1], kc.shape[2], kc.shape[3], vc.shape[3]
+    q, k, v, g = torch.split(
+        x[:, col:col + heads * (dim + vdim) + G * (dim + vdim)],
+        [heads * dim, G * dim, G * vdim, heads * vdim], dim=1)
+    q, k = q.reshape(-1, heads, dim), k.reshape(-1, G, dim)
+    v = _rms(v.reshape(-1, G, vdim), eps).to(x.dtype)
+    for r0, n, p0, s in _portions(plan):
+        i = torch.arange(p0, p0 + n)
+        cell = cache.table[s].long()[i // page]
+        kc[cell, :, i % page] = k[r0:r0 + n]
+        vc[cell, :, i % page] = v[r0:r0 + n]
+        j = torch.arange(p0 + n)
+        if size:
+            j = j[(j < keep) | (j > p0 - size)]
+        cell = cache.table[s].long()[j // page]
+        o = _attend(q[r0:r0 + n], kc[cell, :, j % page], vc[cell, :, j % page],
+                    i, j, size=size, keep=keep, scale=scale, softcap=softcap,
+                    bias=bias).reshape(n, heads * vdim)
+        o = o * torch.sigmoid(g[r0:r0 + n].float()) * out_scale
+        out[r0:r0 + n, out_col:out_col + heads * vdim] = o.to(x.dtype)
 
 
 def tied_attention(x, cache, run, plan, *, heads, q_norm, k_norm, temp, slopes,
@@ -349,6 +483,66 @@ def retention(qkvg, cache, run, plan, *, pows, dec, rope, kscale, eps):
         st[sl] = S
     y = _rms(o, eps) * F.silu(g)
     return y.reshape(qkvg.shape[0], H * dv).to(qkvg.dtype)
+
+
+def lightning(p, cache, run, plan, *, pows, dec, norm, eps):
+    """Linear attention with a fixed decay per head over run `run` of the
+    cache's states; rows of p are [q | k | v | gate], the first three through
+    silu.  Returns (rows, H * dv): all heads together through an RMS norm with
+    weights `norm`, times the gate's sigmoid."""
+    st, = cache.state[run]
+    if p.is_cuda:
+        m = require_lm_ext()
+        o = m.retention(p, st, plan.pos, plan.slot, plan.tiles, plan.seqs,
+                        plan.n_dec, pows, dec, None, None, 1.0, eps, True)
+        H, dv, dk = st.shape[1:]
+        return m.gated_rms(o, norm, p, H * (2 * dk + dv), eps)
+    H, dv, dk = st.shape[1:]
+    q, k, v, g = torch.split(p.float(), [H * dk, H * dk, H * dv, H * dv], dim=1)
+    q, k, v = (F.silu(t).view(p.shape[0], H, -1) for t in (q, k, v))
+    d = dec.sum(1).view(H, 1, 1)
+    o = torch.zeros(p.shape[0], H, dv)
+    for r0, n, p0, sl in _portions(plan):
+        S = torch.zeros_like(st[sl]) if p0 == 0 else st[sl]
+        for r in range(r0, r0 + n):
+            S = d * S + v[r].unsqueeze(2) * k[r].unsqueeze(1)
+            o[r] = (S @ q[r].unsqueeze(2)).squeeze(2)
+        st[sl] = S
+    o = o.reshape(p.shape[0], H * dv).to(p.dtype)
+    return (_rms(o, eps, norm) * torch.sigmoid(g)).to(p.dtype)
+
+
+def gla(x, col, out, out_col, cache, run, plan, *, rank, a2, a2_b, tau, norm,
+        out_scale, eps):
+    """Gated linear attention (Yang et al., "Gated Linear Attention
+    Transformers with Hardware-Efficient Training") of a ragged batch over run
+    `run` of the cache's states: S <- diag(alpha) S + k v^T, o = S^T q /
+    sqrt(dim), with alpha = sigmoid(a2 u + a2_b)^(1/tau) per key channel.  x's
+    columns from `col` on are [q | k | v | gate | u], u `rank` wide.  Each
+    head's result, RMS-normed (weights `norm`), times silu of its gate and
+    out_scale, goes to out's columns from out_col on."""
+    st = cache.state[run][0]
+    if x.is_cuda:
+        return require_lm_ext().gla(
+            x, col, out, out_col, st, plan.pos, plan.slot, plan.tiles,
+            plan.seqs, plan.n_dec, a2, a2_b, tau, norm, out_scale, eps)
+    H, dv, dk = st.shape[1:]
+    T = x.shape[0]
+    q, k, v, g, u = torch.split(
+        x[:, col:col + 2 * H * (dk + dv) + rank].float(),
+        [H * dk, H * dk, H * dv, H * dv, rank], dim=1)
+    alpha = torch.exp(F.logsigmoid(F.linear(u, a2.float(), a2_b.float())) / tau)
+    q, k, v = (t.reshape(T, H, -1) for t in (q * dk ** -0.5, k, v))
+    alpha = alpha.view(T, H, 1, dk)
+    o = torch.zeros(T, H, dv)
+    for r0, n, p0, s in _portions(plan):
+        S = torch.zeros_like(st[s]) if p0 == 0 else st[s]
+        for r in range(r0, r0 + n):
+            S = alpha[r] * S + v[r].unsqueeze(2) * k[r].unsqueeze(1)
+            o[r] = (S @ q[r].unsqueeze(2)).squeeze(2)
+        st[s] = S
+    y = _rms(o, eps, norm).reshape(T, H * dv) * F.silu(g) * out_scale
+    out[:, out_col:out_col + H * dv] = y.to(x.dtype)
 
 
 def latent_attention(a, cache, run, plan, *, heads, dim, vdim, rot, q_norm,
@@ -529,19 +723,36 @@ def moe(h, router, gate_up, down, shared, *, top, groups, keep, scale) -> Parts:
     off.scatter_(1, merit.topk(keep, dim=1).indices, False)
     ids = z[:, :E].masked_fill(off.repeat_interleave(E // groups, 1),
                                float("-inf")).topk(top, dim=1).indices
-
-    def expert(x, gu, dn):
-        g, u = F.linear(x.float(), gu.float()).to(h.dtype).float().chunk(2, -1)
-        return F.linear((F.silu(g) * u).to(h.dtype).float(),
-                        dn.float()).to(h.dtype)
-
     weights = s.gather(1, ids) * scale
-    y = h.new_empty(T, top, h.shape[1])
-    for e in range(E):
-        t, k = (ids == e).nonzero(as_tuple=True)
-        if t.numel():
-            y[t, k] = expert(h[t], gate_up[e], down[e])
+    y = _experts(h, ids, gate_up, down)
     if shared is not None:
-        y = torch.cat([y, expert(h, *shared).unsqueeze(1)], 1)
+        y = torch.cat([y, _expert(h, *shared).unsqueeze(1)], 1)
         weights = torch.cat([weights, torch.sigmoid(z[:, E:E + 1])], 1)
     return Parts(y, weights)
+
+
+def table_moe(h, tokens, table, gate_up, down) -> Parts:
+    """Gated experts of rows h (T, W), chosen by token id: table (vocab, top)
+    int32 names each token's experts, which have equal weights; gate_up
+    (E, 2 ff, W), down (E, W, ff)."""
+    if h.is_cuda:
+        return Parts(*require_lm_ext().table_moe(h, tokens, table, gate_up,
+                                                 down))
+    ids = table[tokens].long()
+    return Parts(_experts(h, ids, gate_up, down),
+                 torch.full(ids.shape, 1.0 / ids.shape[1]))
+
+
+def _expert(x, gu, dn):
+    g, u = F.linear(x.float(), gu.float()).to(x.dtype).float().chunk(2, -1)
+    return F.linear((F.silu(g) * u).to(x.dtype).float(), dn.float()).to(x.dtype)
+
+
+def _experts(h, ids, gate_up, down):
+    """(T, top, W): every row by each of its experts ids (T, top)."""
+    y = h.new_empty(*ids.shape, h.shape[1])
+    for e in range(gate_up.shape[0]):
+        t, k = (ids == e).nonzero(as_tuple=True)
+        if t.numel():
+            y[t, k] = _expert(h[t], gate_up[e], down[e])
+    return y

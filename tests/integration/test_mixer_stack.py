@@ -1,5 +1,5 @@
-"""Mixer-stack models (Lasezen, Nekozen, Babodra) through the framework (cache,
-batches, scheduler, sampling, command line) against the plain oracles.  float32 throughout;
+"""Mixer-stack models (Lasezen, Nekozen, Babodra, Tilivik) through the framework
+(cache, batches, scheduler, sampling, command line) against the plain oracles.  float32 throughout;
 the GPU form of each test runs the HIP kernels."""
 
 import json
@@ -26,7 +26,7 @@ DEVS = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
 dev_ = pytest.mark.parametrize("dev", DEVS)
 each = pytest.mark.parametrize("name", sorted(C.CONFIGS))
 looped = pytest.mark.parametrize("name", ["looped", "neko-looped",
-                                          "bab-plain"])
+                                          "bab-plain", "tili-looped"])
 
 _made = {}
 
@@ -80,7 +80,8 @@ def _feed(m, t, parts):
 @dev_
 @pytest.mark.parametrize("name,runs", [("looped", 1 + 3 * 2 + 1),
                                        ("neko-looped", 1 + 3 * 3 + 1),
-                                       ("bab-plain", 3)])
+                                       ("bab-plain", 3),
+                                       ("tili-looped", 1 + 3 * 2 + 1)])
 def test_residual_stream_after_every_layer_run(dev, name, runs):
     m, t, _ = make(name, dev)
     cfg = C.CONFIGS[name]
@@ -184,7 +185,8 @@ def test_bfloat16_stays_near(name):
 # ------------------------------------------------------- registry, weights
 @pytest.mark.parametrize("name,missing", [("plain", "l0.mix.g"),
                                           ("neko-plain", "l0.mix.dkv.norm"),
-                                          ("bab-plain", "l1.mlp.shared.sg")])
+                                          ("bab-plain", "l1.mlp.shared.sg"),
+                                          ("tili-looped", "l1.shift")])
 def test_checkpoint_round_trip_and_strictness(name, missing):
     cfg = C.CONFIGS[name]
     w = C.weights(cfg)
@@ -217,6 +219,15 @@ def test_config_errors_are_loud():
                 dict(C.attn(), type="latent_attention")):
         with pytest.raises(ValueError):
             C.build(C.babodra_config([bad]), {})
+    for bad in (C.light(decay=[0.9]), C.par(C.window(heads=3, kv=2)),
+                C.par(C.window(far=7)), C.light(mlp=C.table_ff(3, 4)),
+                C.light(mlp={"kind": "dense", "ff": 8}),
+                dict(C.light(), type="gla")):
+        cfg = C.tilivik_config([bad])
+        with pytest.raises(ValueError):
+            C.build(cfg, C.weights(dict(cfg, layers=[C.par()])))
+    with pytest.raises(ValueError, match="left.rel"):
+        C.build(C.tilivik_config([C.par()]), {})
     for bad in (dict(C.attn(), type="spiral"),
                 C.ret(decay=[0.9]),
                 dict(C.attn(), mlp={"kind": "moe", "ff": 8})):
@@ -233,8 +244,10 @@ def model_dir(tmp_path, name):
     cfg = C.CONFIGS[name]
     d = tmp_path / name
     d.mkdir()
-    (d / "config.json").write_text(json.dumps(cfg))
-    st.save_file({k: v.bfloat16() for k, v in C.weights(cfg).items()},
+    (d / "config.json").write_text(json.dumps(
+        {k: v for k, v in cfg.items() if not k.startswith("_")}))
+    st.save_file({k: v.bfloat16() if v.is_floating_point() else v
+                  for k, v in C.weights(cfg).items()},
                  str(d / "model.safetensors"))
     return str(d)
 
@@ -254,7 +267,8 @@ def test_model_dir_loads_by_architecture(tmp_path, name):
         load_config(None, [f"model.dir={tmp_path / 'x'}"])
 
 
-@pytest.mark.parametrize("name", ["plain", "neko-plain", "bab-plain"])
+@pytest.mark.parametrize("name", ["plain", "neko-plain", "bab-plain",
+                                  "tili-plain"])
 def test_scoring_matches_and_training_is_refused(name):
     m, t, ref = make(name, "cpu")
     x = torch.tensor([t[:-1], t[:-1]])
@@ -266,6 +280,18 @@ def test_scoring_matches_and_training_is_refused(name):
     with pytest.raises(NotImplementedError):
         m.train()(x, y)
     m.eval()
+
+
+@pytest.mark.parametrize("entry", [-1, 5, "twice"])
+def test_expert_tables_are_checked(entry):
+    cfg = C.CONFIGS["tili-plain"]
+    w = C.weights(cfg)
+    t = w["l1.mlp.table"].clone()                    # 5 experts, 3 a token
+    t[7, 1] = t[7, 0] if entry == "twice" else entry
+    with pytest.raises(ValueError, match="table"):
+        C.build(cfg, dict(w, **{"l1.mlp.table": t}))
+    with pytest.raises(ValueError, match="int32"):
+        C.build(cfg, dict(w, **{"l1.mlp.table": t.float()}))
 
 
 def test_learned_positions_end_a_sequence():
@@ -352,7 +378,8 @@ def expected(name, prompt, n):
 
 @dev_
 @pytest.mark.parametrize("name", ["looped", "odd", "neko-looped", "neko-odd",
-                                  "bab-plain", "bab-odd"])
+                                  "bab-plain", "bab-odd", "tili-looped",
+                                  "tili-odd"])
 def test_greedy_generation(dev, name):
     m, t, _ = make(name, dev)
     gen = Generator(m)
@@ -543,7 +570,8 @@ def test_graph_replays_equal_eager(name):
 
 # ----------------------------------------------------------- trace replay
 @dev_
-@pytest.mark.parametrize("name", ["plain", "neko-plain", "bab-even"])
+@pytest.mark.parametrize("name", ["plain", "neko-plain", "bab-even",
+                                  "tili-even"])
 def test_trace_run_program(dev, tmp_path, name):
     d = model_dir(tmp_path, name)
     _, t, ref = make(name, "cpu")

@@ -8,9 +8,10 @@ from scaffold.cache import KVSpec, PagedStateCache, StateSpec, TiedSpec
 from scaffold.config import load_config
 from scaffold.convert import load_stack
 from scaffold.models import build_model
-from tests.oracle import babodra, lasezen, nekozen
+from tests.oracle import babodra, lasezen, nekozen, tilivik
 
-ORACLES = {"Lasezen": lasezen, "Nekozen": nekozen, "Babodra": babodra}
+ORACLES = {"Lasezen": lasezen, "Nekozen": nekozen, "Babodra": babodra,
+           "Tilivik": tilivik}
 
 
 def attn(heads=4, kv=2, dim=16, vdim=16, size=24, scale=0.3, ff=40):
@@ -166,6 +167,88 @@ BABODRA = {
 CONFIGS.update(BABODRA)
 
 
+def table_ff(experts=6, top=2, ff=24):
+    return {"kind": "moe", "expert": {"ff": ff},
+            "router": {"experts": experts, "top": top}}
+
+
+def light(heads=3, dim=16, vdim=24, decay=None, mlp=None):
+    return {"type": "lightning", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": dim, "vdim": vdim,
+        "decay": decay or [0.97, 0.6, 0.999, 0.85][:heads]}}
+
+
+def window(heads=4, kv=2, dim=16, vdim=24, size=21, keep=3, far=50, scale=0.3,
+           cap=6.0):
+    return {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim,
+            "bias_max": far, "mask": {"size": size, "keep_first": keep},
+            "scale": scale, "softcap": cap}
+
+
+def chan(heads=3, dim=24, vdim=16, tau=4.0):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "tau": tau}
+
+
+def par(left=None, right=None, ls=0.7, rs=1.3, mlp=None):
+    return {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": left or window(), "right": right or chan(), "left_scale": ls,
+        "right_scale": rs}}
+
+
+def tilivik_config(layers, width=32, vocab=61, loop=None, eps=1e-5,
+                   buckets=97, muls=(31, 11), rel=14, rank=8):
+    """rel, rank: sizes that only the tensors' shapes tell."""
+    return {"architecture": "Tilivik", "layers": layers, "width": width,
+            "vocab": vocab, "norm": {"eps": eps}, "loop": loop,
+            "embedding": {"bigram": {"buckets": buckets, "mul_prev": muls[0],
+                                     "mul_cur": muls[1]}},
+            "_rel": rel, "_rank": rank}
+
+
+TILIVIK = {
+    "tili-plain": tilivik_config([light(mlp=table_ff()),
+                                  par(mlp=table_ff(5, 3))]),
+    "tili-looped": tilivik_config(
+        [light(heads=2), par(window(kv=1, size=33, keep=0), mlp=table_ff()),
+         light(heads=4, dim=12, vdim=8, mlp=table_ff(4, 1)),
+         par(window(heads=2, kv=2, size=70, keep=66), chan(tau=1.0))],
+        loop={"start": 1, "stop": 3, "times": 3}),
+    "tili-odd": tilivik_config(
+        [par(window(heads=3, kv=3, dim=9, vdim=5, size=5, keep=1, far=9),
+             chan(heads=2, dim=10, vdim=7, tau=0.7), mlp=table_ff(5, 3, 13)),
+         light(heads=3, dim=5, vdim=7, mlp=table_ff(3, 3, 9)),
+         par(window(heads=5, kv=1, dim=7, vdim=9, size=64, keep=64),
+             chan(heads=5, dim=9, vdim=3))],
+        width=27, vocab=33, eps=0.05, buckets=13, muls=(5, 3), rel=7, rank=5,
+        loop={"start": 0, "stop": 2, "times": 2}),
+    "tili-wide": tilivik_config(
+        [par(window(heads=6, kv=2, dim=72, vdim=136, size=100, keep=70,
+                    scale=0.1, far=128),
+             chan(heads=2, dim=136, vdim=72), mlp=table_ff(70, 9, 16)),
+         light(heads=2, dim=72, vdim=136)],
+        width=48, rel=32, rank=16, loop={"start": 1, "stop": 2, "times": 2}),
+    "tili-even": tilivik_config(
+        [par(window(heads=4, kv=2, dim=64, vdim=64, size=48, keep=5,
+                    scale=0.125, far=128, cap=30.0),
+             chan(heads=2, dim=64, vdim=128, tau=16.0),
+             mlp=table_ff(8, 2, 64)),
+         light(heads=2, dim=64, vdim=64, mlp=table_ff(4, 2, 128)),
+         par(window(heads=4, kv=1, dim=128, vdim=64, size=130, keep=8,
+                    scale=0.1), chan(heads=1, dim=128, vdim=64, tau=8.0))],
+        width=64, rel=32, rank=16),
+    "tili-ones": tilivik_config(
+        [light(heads=1, dim=1, vdim=1, decay=[1.0], mlp=table_ff(1, 1, 1)),
+         par(window(heads=1, kv=1, dim=1, vdim=1, size=1, keep=0, far=2,
+                    scale=1.0, cap=1.0),
+             chan(heads=1, dim=1, vdim=1, tau=1.0), ls=1.0, rs=1.0),
+         par(window(heads=2, kv=1, size=4096, keep=1, far=4096),
+             chan(heads=1, dim=32, vdim=32))],
+        buckets=1, muls=(0, 1), rel=2, rank=1,
+        loop={"start": 1, "stop": 3, "times": 1}),
+}
+CONFIGS.update(TILIVIK)
+
+
 def oracle(cfg):
     return ORACLES[cfg["architecture"]]
 
@@ -284,6 +367,69 @@ def babodra_weights(cfg, seed=0):
     return {k: v.bfloat16().float() for k, v in w.items()}
 
 
+def tilivik_weights(cfg, seed=0):
+    """As weights(): no shift, gate, bias, cap or decay is near what would
+    leave it out."""
+    g = torch.Generator().manual_seed(seed)
+    W, V = cfg["width"], cfg["vocab"]
+    w = {}
+
+    def mat(name, out, inp, gain=1.0):
+        w[name] = torch.randn(out, inp, generator=g) * gain * inp ** -0.5
+
+    def vec(name, n, around=1.0, spread=0.4):
+        w[name] = around + spread * torch.randn(n, generator=g)
+
+    def num(name):
+        w[name] = 0.8 + 0.4 * torch.rand((), generator=g)
+
+    mat("embed", V, W, W ** 0.5)
+    mat("bigram", cfg["embedding"]["bigram"]["buckets"] + 1, W, W ** 0.5)
+    if cfg["loop"]:
+        mat("loop.step", cfg["loop"]["times"], W, W ** 0.5)
+    for i, L in enumerate(cfg["layers"]):
+        p, mx = f"l{i}.", L["mixer"]
+        for n in ("norm1", "norm2") if L["mlp"] else ("norm1",):
+            num(p + n)
+        vec(p + "shift", W, 0.4, 0.3)
+        if L["type"] == "lightning":
+            a, b = mx["heads"] * mx["dim"], mx["heads"] * mx["vdim"]
+            for n, rows in (("q", a), ("k", a), ("v", b), ("g", b)):
+                mat(f"{p}mix.{n}", rows, W, 1.5)
+            mat(p + "mix.o", W, b)
+            vec(p + "mix.norm", b)
+        else:
+            m, q = mx["left"], p + "mix.left."
+            mat(q + "q", m["heads"] * m["dim"], W, 2.0)
+            mat(q + "k", m["kv_heads"] * m["dim"], W, 2.0)
+            mat(q + "v", m["kv_heads"] * m["vdim"], W)
+            mat(q + "g", m["heads"] * m["vdim"], W, 2.0)
+            mat(q + "o", W, m["heads"] * m["vdim"])
+            w[q + "rel"] = torch.randn(cfg["_rel"], m["heads"], generator=g)
+            m, q = mx["right"], p + "mix.right."
+            a, b = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            for n, rows in (("q", a), ("k", a), ("v", b), ("g", b)):
+                mat(q + n, rows, W, 1.5)
+            mat(q + "a1", cfg["_rank"], W)
+            mat(q + "a2", a, cfg["_rank"], 2.0)
+            vec(q + "a2.b", a, 2.0, 1.5)
+            mat(q + "o", W, b)
+            vec(q + "norm", m["vdim"])
+        if L["mlp"]:
+            E, top = (L["mlp"]["router"][n] for n in ("experts", "top"))
+            ff = L["mlp"]["expert"]["ff"]
+            for e in range(E):
+                mat(f"{p}mlp.e{e}.gate", ff, W, 1.5)
+                mat(f"{p}mlp.e{e}.up", ff, W, 1.5)
+                mat(f"{p}mlp.e{e}.down", W, ff, 1.5)
+            w[p + "mlp.table"] = torch.rand(V, E, generator=g).argsort(
+                1)[:, :top].to(torch.int32).contiguous()
+    num("final.norm")
+    mat("head", V, W, 3.0)
+    return {k: v.bfloat16().float() if v.is_floating_point() else v
+            for k, v in w.items()}
+
+
 def weights(cfg, seed=0):
     """Random checkpoint (bfloat16-representable float32 tensors), scaled
     so that scores, sinks and norms are far from trivial."""
@@ -291,6 +437,8 @@ def weights(cfg, seed=0):
         return babodra_weights(cfg, seed)
     if cfg["architecture"] == "Nekozen":
         return nekozen_weights(cfg, seed)
+    if cfg["architecture"] == "Tilivik":
+        return tilivik_weights(cfg, seed)
     g = torch.Generator().manual_seed(seed)
     W, V = cfg["width"], cfg["vocab"]
     w = {}
@@ -337,7 +485,8 @@ def build(cfg, w, device="cpu", dtype=torch.float32, max_len=512):
     from scaffold import config as C
 
     tc = load_config(None, [f"model.max_seq_len={max_len}"])
-    for k, v in C.ARCHITECTURES[cfg["architecture"]](cfg).items():
+    shapes = {k: tuple(v.shape) for k, v in w.items()}
+    for k, v in C.ARCHITECTURES[cfg["architecture"]](cfg, shapes).items():
         setattr(tc.model, k, v)
     m = build_model(tc)
     load_stack(m, w)
@@ -354,7 +503,7 @@ def poison(cache):
     written shows in the result."""
     for t in cache.k + cache.v + [t for s in cache.state for t in s or ()]:
         if t is not None:
-            t.fill_(float("nan"))
+            t.fill_(float("nan") if t.is_floating_point() else -10**15)
     return cache
 
 
@@ -376,6 +525,7 @@ def cuts(n, sizes):
 
 __all__ = ["attn", "ret", "latent", "mamba", "mem", "config",
            "nekozen_config", "tied", "clamped", "routed", "babodra_config",
-           "CONFIGS", "NEKOZEN", "BABODRA", "oracle", "weights", "build",
+           "light", "window", "chan", "par", "table_ff", "tilivik_config",
+           "CONFIGS", "NEKOZEN", "BABODRA", "TILIVIK", "oracle", "weights", "build",
            "tokens", "poison", "op_cache", "cuts", "KVSpec", "StateSpec",
            "TiedSpec"]
