@@ -1,6 +1,8 @@
 // Prompt attention over a paged cache: grouped heads, chunked causal mask,
 // optional sink in the softmax denominator, separate key and value widths,
-// or values that are the keys (tied form), a bias by distance, an output gate.
+// or values that are the keys (tied form), a bias by distance, an output gate;
+// or a sliding window beside which the first tokens stay visible, soft-capped
+// scores and a learned bias by distance (window form).
 //
 // The kv loop walks cache pages (64 keys), so a tile of keys is one
 // contiguous block per kv head whatever the prompt's cut.  Row i of a tile
@@ -23,20 +25,20 @@ namespace {
 constexpr float LOG2E = 1.4426950408889634f;
 
 // One lane group (LPV lanes, 8 elements each) per (row, head) vector: RMS
-// norm over `dim` for q heads (in place) and k heads (into the cache),
-// plain copy for v heads.
+// norm over `dim` for q heads (in place; left out if q has none) and k heads
+// (into the cache), plain copy for v heads or (v_norm) a norm without weights.
 template <bool F32, int LPV>
 __global__ void __launch_bounds__(256)
 attn_prep_kernel(AttnArgs a, const int* __restrict__ pos,
                  const int* __restrict__ slot, int row0, int n) {
   using N = Num<F32>;
   using E = typename N::E;
-  const int heads = a.H + 2 * a.G;
+  const int h0 = a.qw ? 0 : a.H, heads = a.H + 2 * a.G - h0;
   const long unit = ((long)blockIdx.x * 256 + threadIdx.x) / LPV;
   if (unit >= (long)n * heads) return;
   const int c = (threadIdx.x % LPV) * 8;
   const int row = row0 + (int)(unit / heads);
-  const int hd = (int)(unit % heads);
+  const int hd = h0 + (int)(unit % heads);
   const int s = slot[row];
   if (s < 0) return;
   const int p = pos[row];
@@ -66,6 +68,10 @@ attn_prep_kernel(AttnArgs a, const int* __restrict__ pos,
     load8<F32>(w + c, len - c, aligned, wv);
     #pragma unroll
     for (int i = 0; i < 8; ++i) v[i] *= inv * wv[i];
+  } else if (is_v && a.v_norm) {
+    const float inv = 1.0f / sqrtf(q / (float)a.vdim + a.eps);
+    #pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= inv;
   }
   store8<F32>(dst + c, len - c, aligned, v);
 }
@@ -183,15 +189,17 @@ attn_prefill_kernel(AttnArgs a, const int4* __restrict__ tiles) {
   for (int r = 0; r < 4; ++r) {
     const int row = 16 * w + 4 * lg + r;
     ip[r] = t.z + min(row, t.y - 1);
-    cs[r] = a.size ? ip[r] - ip[r] % a.size : 0;
+    cs[r] = first_seen(a, ip[r]);
     m[r] = a.has_sink ? sink_score<F32>(a, h) * LOG2E : -1e30f;
     lsum[r] = a.has_sink ? 1.f : 0.f;
   }
 
   const int p_last = t.z + t.y - 1;
-  const int j_first = a.size ? t.z - t.z % a.size : 0;
+  const PageList pages(a, t.z, p_last);
   const int* tab = a.table + (long)t.w * a.max_pages;
-  for (int pg = j_first / LM_PAGE; pg <= p_last / LM_PAGE; ++pg) {
+  const float* bias = a.bias ? a.bias + (long)h * a.n_bias : nullptr;
+  for (int it = 0; it < pages.n; ++it) {
+    const int pg = pages[it];
     const long page = tab[pg];
     const E* kp = (const E*)a.kc + (page * a.G + g) * LM_PAGE * a.dim;
     const E* vp = (const E*)a.vc + (page * a.G + g) * LM_PAGE * a.vdim;
@@ -202,7 +210,7 @@ attn_prefill_kernel(AttnArgs a, const int4* __restrict__ tiles) {
     for (int u = tid; u < LM_PAGE * (DK / 8); u += 256) {
       const int j = u / (DK / 8), c = (u % (DK / 8)) * 8;
       float v[8];
-      const bool ok = j0 + j >= j_first && j0 + j <= p_last;
+      const bool ok = j0 + j <= p_last;
       load8<F32>(kp + (long)j * a.dim + c, ok ? a.dim - c : 0, aligned, v);
       #pragma unroll
       for (int i = 0; i < 8; ++i) Ks[j * LDK + c + i] = N::down(v[i]);
@@ -210,7 +218,7 @@ attn_prefill_kernel(AttnArgs a, const int4* __restrict__ tiles) {
     for (int u = tid; u < LM_PAGE * (DV / 8); u += 256) {
       const int j = u % LM_PAGE, c = (u / LM_PAGE) * 8;
       float v[8];
-      const bool ok = j0 + j >= j_first && j0 + j <= p_last;
+      const bool ok = j0 + j <= p_last;
       load8<F32>(vp + (long)j * a.vdim + c, ok ? a.vdim - c : 0, aligned, v);
       #pragma unroll
       for (int i = 0; i < 8; ++i) Vt[(c + i) * LDJ + j] = N::down(v[i]);
@@ -231,10 +239,16 @@ attn_prefill_kernel(AttnArgs a, const int4* __restrict__ tiles) {
       #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int j = j0 + ct * 16 + lr;
-        const bool see = j <= ip[r] && j >= cs[r];
-        s[ct][r] = see ? s[ct][r] * (scale2 * Kf[ct * 16 + lr]) -
-                             slope2 * (float)(ip[r] - j)
-                       : -1e30f;
+        const bool see = j <= ip[r] && (j >= cs[r] || j < a.keep);
+        float x = s[ct][r];
+        if (bias) {
+          x *= a.scale;
+          if (a.softcap > 0.f) x = a.softcap * tanhf(x / a.softcap);
+          x = (x + bias[min(max(ip[r] - j, 0), a.n_bias - 1)]) * LOG2E;
+        } else {
+          x = x * (scale2 * Kf[ct * 16 + lr]) - slope2 * (float)(ip[r] - j);
+        }
+        s[ct][r] = see ? x : -1e30f;
         mx[r] = fmaxf(mx[r], s[ct][r]);
       }
     #pragma unroll
@@ -271,8 +285,8 @@ attn_prefill_kernel(AttnArgs a, const int4* __restrict__ tiles) {
   for (int r = 0; r < 4; ++r) {
     const int row = 16 * w + 4 * lg + r;
     if (row >= t.y) continue;
-    const float inv = lsum[r] > 0.f ? 1.0f / lsum[r] : 0.f;
-    E* dst = (E*)a.out + (long)(t.x + row) * a.H * a.vdim + (long)h * a.vdim;
+    const float inv = lsum[r] > 0.f ? a.out_scale / lsum[r] : 0.f;
+    E* dst = (E*)a.out + (long)(t.x + row) * a.ldo + (long)h * a.vdim;
     const E* gate = a.gate ? (const E*)a.gate + (long)(t.x + row) * a.ld +
                                  (long)h * a.vdim : nullptr;
     #pragma unroll
@@ -321,7 +335,7 @@ namespace {
 template <bool F32>
 void run_prep(const AttnArgs& a, const int* pos, const int* slot, int row0,
               int n, hipStream_t st) {
-  const long units = (long)n * (a.H + 2 * a.G);
+  const long units = (long)n * ((a.qw ? a.H : 0) + 2 * a.G);
   const int d = std::max(a.dim, a.vdim);
   #define AP_GO(LPV)                                                           \
     hipLaunchKernelGGL((attn_prep_kernel<F32, LPV>),                           \

@@ -11,6 +11,10 @@
 // used, and the split's page ids wait in LDS, so a pass costs no
 // dependent memory round trip.
 //
+// Window form: a split is a span of the visible keys in order, the kept first
+// ones before the window's; a new value is normed over its head; scores pass
+// the soft cap and take their distance's bias (from LDS if it fits).
+//
 // Tied form: one cached row is key and value, so only half the bytes are
 // read; every block takes the root mean squares over the whole of q and of
 // the new k itself, and the key weights go to the query's side.
@@ -38,6 +42,17 @@ DEVINL void head_norm(float* v, const void* w, int c, int dim, float eps) {
   for (int i = 0; i < 8; ++i)
     if (c + i < dim)
       v[i] = N::up(N::down(v[i] * inv * N::up(((const typename N::E*)w)[c + i])));
+}
+
+// over its root mean square, without weights
+template <bool F32, int LPK>
+DEVINL void unit_norm(float* v, int dim, float eps) {
+  float q = 0.f;
+  #pragma unroll
+  for (int i = 0; i < 8; ++i) q += v[i] * v[i];
+  const float inv = 1.0f / sqrtf(group_sum<LPK>(q) / (float)dim + eps);
+  #pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] *= inv;
 }
 
 // What norms the new token's q (its temperature included) and k: a block of
@@ -80,7 +95,9 @@ DEVINL void tied_factors(const AttnArgs& a, const typename Num<F32>::E* qkv,
   inv_k = 1.0f / sqrtf(sk / (float)nk + a.eps);
 }
 
-template <bool F32, int LPK, int HGC, bool TIED>
+enum Form { PLAIN, TIED_KV, WINDOW };
+
+template <bool F32, int LPK, int HGC, int FORM>
 __global__ void __launch_bounds__(256)
 attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
                    const int* __restrict__ slot, int nsplit,
@@ -90,7 +107,10 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
   constexpr int KPW = 64 / LPK;      // keys per wave and pass
   constexpr int KB = F32 ? 2 : 4;    // keys per lane group and pass
   constexpr int TABS = 512;          // page ids kept in LDS
+  constexpr int BIAS = 512;          // and entries of a head's bias
+  constexpr bool TIED = FORM == TIED_KV, WIN = FORM == WINDOW;
   __shared__ int tab_s[TABS];
+  __shared__ float bias_s[WIN ? HGC : 1][WIN ? BIAS : 1];
   constexpr int NP = 4 * KPW;        // partial results of a block
   __shared__ __attribute__((aligned(16))) float acc_s[HGC][NP][LPK * 8];
   __shared__ float m_s[HGC][NP], l_s[HGC][NP];
@@ -103,7 +123,7 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
   const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
   const int grp = l / LPK, c = (l % LPK) * 8;
   const bool aligned = a.dim % 8 == 0 && a.vdim % 8 == 0;
-  E* out = (E*)a.out + (long)row * a.H * a.vdim;
+  E* out = (E*)a.out + (long)row * a.ldo;
 
   const int s = slot[row];
   if (s < 0) {                        // idle row: a defined, unused output
@@ -117,12 +137,16 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
     return;
   }
   const int p = pos[row];
-  const int cs = a.size ? p - p % a.size : 0;
-  const int nkeys = p - cs + 1;
+  // visible keys in order: `nk` kept ones from 0 on, then those from cs on;
+  // u counts them from cs - nk, so that u is the position of the latter
+  const int cs = first_seen(a, p), nk = WIN ? min(a.keep, cs) : 0;
+  const int u0 = cs - nk;
+  const int nkeys = p - u0 + 1;
   const int per = (nkeys + nsplit - 1) / nsplit;
-  const int jb = cs + split * per;
+  const int jb = u0 + split * per;
   const int je = min(jb + per, p + 1);        // may be <= jb: empty split
   const bool has_new = jb <= p && je == p + 1;
+  auto place = [&](int u) { return WIN && u < cs ? u - u0 : u; };
   const int* tab = a.table + (long)s * a.max_pages;
   const E* qkv = (const E*)a.qkv + (long)row * a.ld;
 
@@ -154,6 +178,29 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
     for (int j = 0; j < 8; ++j) acc[i][j] = 0.f;
   }
 
+  const bool bias_lds = a.n_bias <= BIAS;
+  const float* bias_g[HGC];
+  if constexpr (WIN) {
+    #pragma unroll
+    for (int i = 0; i < HGC; ++i)
+      bias_g[i] = a.bias + (long)(h0 + min(i, nh - 1)) * a.n_bias;
+    if (bias_lds) {
+      #pragma unroll
+      for (int i = 0; i < HGC; ++i)
+        for (int d = tid; d < a.n_bias; d += 256) bias_s[i][d] = bias_g[i][d];
+    }
+  }
+  const SoftCap cap(a, LOG2E);
+  // a score in base 2 of head i at distance dj
+  auto windowed = [&](int i, float x, float dj) {
+    const int d = min((int)dj, a.n_bias - 1);
+    const float b = (bias_lds ? bias_s[i][d] : bias_g[i][d]) * LOG2E;
+    if constexpr (!F32) return cap(x) + b;
+    x *= a.scale;
+    if (a.softcap > 0.f) x = a.softcap * tanhf(x / a.softcap);
+    return fmaf(x, LOG2E, b);
+  };
+
   // kf: scale of a key's scores, dj: its distance
   auto fold = [&](const auto& k, const auto& v, const bool (&ok)[KB],
                   const float (&kf)[KB], const float (&dj)[KB]) {
@@ -165,7 +212,9 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
         float d = 0.f;
         #pragma unroll
         for (int j = 0; j < 8; ++j) d = fmaf(q[i][j], k[u][j], d);
-        d = group_sum<LPK>(d) * kf[u] - slope2[i] * dj[u];
+        d = group_sum<LPK>(d);
+        if constexpr (WIN) d = windowed(i, d, dj[u]);
+        else d = d * kf[u] - slope2[i] * dj[u];
         sc[u] = ok[u] ? d : NEG;
         mx = fmaxf(mx, sc[u]);
       }
@@ -189,11 +238,11 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
   };
 
   const int jc = min(je, p + 1);              // p itself is not cached yet
-  const int pg0 = jb / LM_PAGE;
-  const int npg = jc > jb ? (jc - 1) / LM_PAGE - pg0 + 1 : 0;
+  const int pg0 = max(jb, cs) / LM_PAGE;      // pages of kept keys aside
+  const int npg = jc > max(jb, cs) ? (jc - 1) / LM_PAGE - pg0 + 1 : 0;
   const bool in_lds = npg <= TABS;
-  if (in_lds) {
-    for (int i = tid; i < npg; i += 256) tab_s[i] = tab[pg0 + i];
+  if (in_lds || WIN) {
+    for (int i = tid; in_lds && i < npg; i += 256) tab_s[i] = tab[pg0 + i];
     __syncthreads();
   }
   // the new token's key and value, in every lane group of the split that
@@ -206,6 +255,16 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
       vnew.load(qkv + (long)(a.H + a.G) * a.dim + (long)g * a.vdim + c,
                 a.vdim - c, aligned);
       head_norm<F32, LPK>(k0, a.kw, c, a.dim, a.eps);
+      if constexpr (WIN) {
+        if (a.v_norm) {
+          float v0[8];
+          #pragma unroll
+          for (int j = 0; j < 8; ++j) v0[j] = vnew[j];
+          unit_norm<F32, LPK>(v0, a.vdim, a.eps);
+          #pragma unroll
+          for (int j = 0; j < 8; ++j) vnew.e[j] = N::down(v0[j]);
+        }
+      }
     }
     #pragma unroll
     for (int j = 0; j < 8; ++j) knew.e[j] = N::down(k0[j]);
@@ -229,12 +288,13 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
   auto fetch = [&](int j0) {
     #pragma unroll
     for (int u = 0; u < KB; ++u) {
-      const int j = j0 + (u * 4 + w) * KPW + grp;
-      okn[u] = j < jc;
-      const bool cached = j < min(jc, p);
+      const int v = j0 + (u * 4 + w) * KPW + grp, j = place(v);
+      okn[u] = v < jc;
+      const bool cached = v < min(jc, p);
       long cell = 0, tok = 0;
       if (cached) {
-        const int page = in_lds ? tab_s[j / LM_PAGE - pg0] : tab[j / LM_PAGE];
+        const int page = in_lds && v >= cs ? tab_s[j / LM_PAGE - pg0]
+                                           : tab[j / LM_PAGE];
         cell = ((long)page * a.G + g) * LM_PAGE + j % LM_PAGE;
         tok = (long)page * LM_PAGE + j % LM_PAGE;
       }
@@ -247,7 +307,7 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
       } else {
         vn[u].load((const E*)a.vc + cell * a.vdim + c, cached ? a.vdim - c : 0, aligned);
       }
-      if (j == p && okn[u]) {
+      if (v == p && okn[u]) {
         kn[u] = knew;
         if constexpr (!TIED) vn[u] = vnew;
       }
@@ -306,7 +366,7 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
       if (a.gate)
         av *= sigmoid(N::up(((const E*)a.gate)[(long)row * a.ld +
                                                (long)(h0 + i) * a.vdim + d]));
-      out[(long)(h0 + i) * a.vdim + d] = N::down(av / lt);
+      out[(long)(h0 + i) * a.vdim + d] = N::down(av / lt * a.out_scale);
     } else {
       float* o = ws + (((long)row * a.H + h0 + i) * nsplit + split) * (a.vdim + 2);
       o[2 + d] = av;
@@ -346,7 +406,7 @@ attn_decode_tied_kernel(AttnArgs a, const int* __restrict__ pos,
   const int nh = min(16, hg - hc * 16), h0 = g * hg + hc * 16;
   const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
   const int lr = l & 15, lg = l >> 4;
-  short* out = (short*)a.out + (long)row * a.H * a.dim;
+  short* out = (short*)a.out + (long)row * a.ldo;
 
   const int s = slot[row];
   if (s < 0) {                        // idle row: a defined, unused output
@@ -538,7 +598,7 @@ attn_decode_tied_kernel(AttnArgs a, const int* __restrict__ pos,
       if (a.gate)
         av *= sigmoid(bf2f(((const short*)a.gate)[(long)row * a.ld +
                                                   (long)(h0 + i) * a.dim + d]));
-      out[(long)(h0 + i) * a.dim + d] = cvt_bf16(av / lt);
+      out[(long)(h0 + i) * a.dim + d] = cvt_bf16(av / lt * a.out_scale);
     } else {
       float* q = ws + (((long)row * a.H + h0 + i) * nsplit + split) * (a.dim + 2);
       q[2 + d] = av;
@@ -589,15 +649,16 @@ attn_combine_kernel(AttnArgs a, const int* __restrict__ slot, int nsplit,
   __syncthreads();
   if (!mine) return;
   for (int i = 1; i < parts; ++i) av += part_s[i * nd + d];
-  ((E*)a.out)[((long)row * a.H + h) * a.vdim + d] = N::down(av * inv * gate);
+  ((E*)a.out)[(long)row * a.ldo + (long)h * a.vdim + d] =
+      N::down(av * inv * gate * a.out_scale);
 }
 
-template <bool F32, int LPK, bool TIED>
+template <bool F32, int LPK, int FORM>
 void pick_heads(const AttnArgs& a, const int* pos, const int* slot, int R,
                 int nsplit, float* ws, hipStream_t st) {
   const int hg = a.H / a.G;
   #define AD_GO(HGC)                                                           \
-    hipLaunchKernelGGL((attn_decode_kernel<F32, LPK, HGC, TIED>),                    \
+    hipLaunchKernelGGL((attn_decode_kernel<F32, LPK, HGC, FORM>),              \
                        dim3(nsplit, a.G * ((hg + HGC - 1) / HGC), R),          \
                        dim3(256), 0, st, a, pos, slot, nsplit, ws)
   if (hg == 1) AD_GO(1);
@@ -609,8 +670,9 @@ void pick_heads(const AttnArgs& a, const int* pos, const int* slot, int R,
 template <bool F32, int LPK>
 void pick_form(const AttnArgs& a, const int* pos, const int* slot, int R,
                int nsplit, float* ws, hipStream_t st) {
-  if (a.ks) pick_heads<F32, LPK, true>(a, pos, slot, R, nsplit, ws, st);
-  else pick_heads<F32, LPK, false>(a, pos, slot, R, nsplit, ws, st);
+  if (a.ks) pick_heads<F32, LPK, TIED_KV>(a, pos, slot, R, nsplit, ws, st);
+  else if (a.bias) pick_heads<F32, LPK, WINDOW>(a, pos, slot, R, nsplit, ws, st);
+  else pick_heads<F32, LPK, PLAIN>(a, pos, slot, R, nsplit, ws, st);
 }
 
 template <bool F32>

@@ -17,6 +17,9 @@
 //    rows for the scores, transpose reads for the values; the swizzle keeps
 //    both free of conflicts.  A key's factor and its distance bias join the
 //    score in one multiply-add each.
+//  * Window form: soft cap by one exponential and one reciprocal, the bias by
+//    distance from LDS (a page whose every distance is beyond the table's
+//    last adds a constant), kept first pages before the window's.
 //  * Pages that no row of a wave sees are skipped by that wave; masks are
 //    applied only on pages that a chunk edge or the diagonal crosses.
 
@@ -63,19 +66,23 @@ DEVINL int chunk_at(int j, int cb) {
   else return cb ^ (j & 7);
 }
 
-// FORM 0: as stored; 1: with a bias by distance; 2: tied, with one
+constexpr int BIAS_LDS = 512;          // entries of a head's bias kept in LDS
+
+// FORM 0: as stored; 1: with a bias by distance; 2: tied, with one; 3: window
 template <int DK, int DV, int HPB, int FORM>
 __global__ void __launch_bounds__(HPB * 128, 2)
 attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
                          int n_tiles) {
   constexpr int NT = HPB * 128;
   constexpr int NSL = DK / 16, NDT = DV / 32;
-  constexpr bool TIED = FORM == 2, BIAS = FORM != 0;
+  constexpr bool TIED = FORM == 2, BIAS = FORM == 1 || FORM == 2;
+  constexpr bool WIN = FORM == 3;
   static_assert(!TIED || DK == DV, "one image");
   constexpr int BUF = 64 * (DK + (TIED ? 0 : DV));  // K image + V tr-image
   constexpr int KC = 64 * DK / 8 / NT, VC = 64 * DV / 8 / NT;
   __shared__ __attribute__((aligned(16))) short lds[2 * BUF];
   __shared__ __attribute__((aligned(16))) float kfs[TIED ? 2 * 64 : 4];
+  __shared__ float bias_s[WIN ? HPB * BIAS_LDS : 1];
 
   const int tid = threadIdx.x, l = tid & 63, wid = tid >> 6;
   const int lq = l & 31, half = l >> 5;
@@ -89,8 +96,7 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
   const int row = 32 * (wid & 1) + lq;
   const int rowc = min(row, t.y - 1);
   const int ip = t.z + rowc;
-  const int size = a.size;
-  const int cs = size ? ip - ip % size : 0;
+  const int cs = first_seen(a, ip), keep = WIN ? a.keep : 0;
 
   bf16x8 qf[NSL];
   {
@@ -103,15 +109,14 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
   }
 
   const int p_last = t.z + t.y - 1;
-  const int j_first = size ? t.z - t.z % size : 0;
-  const int pg0 = j_first / LM_PAGE, pg1 = p_last / LM_PAGE;
+  const PageList pages(a, t.z, p_last);
   const int* tab = a.table + (long)t.w * a.max_pages;
 
   // this wave's rows: first and last position, and their chunk starts
   const int w0 = t.z + min(32 * (wid & 1), t.y - 1);
   const int w1 = t.z + min(32 * (wid & 1) + 31, t.y - 1);
   const bool w_any = 32 * (wid & 1) < t.y;
-  const int wcs0 = size ? w0 - w0 % size : 0, wcs1 = size ? w1 - w1 % size : 0;
+  const int wcs0 = first_seen(a, w0), wcs1 = first_seen(a, w1);
 
   bf16x8 kr[KC], vr[TIED ? 1 : VC];
   float kf = 0.f;
@@ -176,14 +181,30 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
   #pragma unroll
   for (int i = 0; i < NDT; ++i) o[i] = {};
 
-  stage_load(pg0);
+  // window form: this head's bias in base 2
+  const int n_bias = WIN ? a.n_bias : 0;
+  const bool bias_lds = n_bias <= BIAS_LDS;
+  const float* bias_g = nullptr;
+  const float* bias_h = bias_s + (wid >> 1) * BIAS_LDS;
+  float bias_far = 0.f;
+  if constexpr (WIN) {
+    bias_g = a.bias + (long)h * n_bias;
+    bias_far = bias_g[n_bias - 1] * LOG2E;
+    if (bias_lds)
+      for (int i = tid % 128; i < n_bias; i += 128)
+        bias_s[(wid >> 1) * BIAS_LDS + i] = bias_g[i] * LOG2E;
+  }
+  const SoftCap cap(a, LOG2E);
+
+  stage_load(pages[0]);
   stage_write(0);
   __syncthreads();
   int cur = 0;
-  for (int pg = pg0; pg <= pg1; ++pg) {
-    if (pg < pg1) stage_load(pg + 1);
+  for (int it = 0; it < pages.n; ++it) {
+    const int pg = pages[it];
+    if (it + 1 < pages.n) stage_load(pages[it + 1]);
     const int j0 = pg * LM_PAGE;
-    if (w_any && j0 <= w1 && j0 + LM_PAGE > wcs0) {
+    if (w_any && j0 <= w1 && (j0 + LM_PAGE > wcs0 || j0 < keep)) {
       const short* kimg = lds + cur * BUF;
       f32x16 s[2];
       s[0] = {};
@@ -200,6 +221,27 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
       const bool edge = j0 + LM_PAGE - 1 > w0 || j0 < wcs1;
       float mt = -1e30f;
       const float d0 = slope2 * (float)(j0 + 4 * half - ip);
+      if constexpr (WIN) {
+        const int last = n_bias - 1, dist = ip - j0 - 4 * half;
+        #pragma unroll
+        for (int sub = 0; sub < 2; ++sub)
+          #pragma unroll
+          for (int r = 0; r < 16; ++r) s[sub][r] = cap(s[sub][r]);
+        if (w0 - j0 - (LM_PAGE - 1) >= last) {         // uniform in the wave
+          #pragma unroll
+          for (int sub = 0; sub < 2; ++sub)
+            #pragma unroll
+            for (int r = 0; r < 16; ++r) s[sub][r] += bias_far;
+        } else {
+          #pragma unroll
+          for (int sub = 0; sub < 2; ++sub)
+            #pragma unroll
+            for (int r = 0; r < 16; ++r) {
+              const int d = min(max(dist - (sub * 32 + (r & 3) + 8 * (r >> 2)), 0), last);
+              s[sub][r] += bias_lds ? bias_h[d] : bias_g[d] * LOG2E;
+            }
+        }
+      }
       #pragma unroll
       for (int sub = 0; sub < 2; ++sub)
         #pragma unroll
@@ -207,11 +249,11 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
           const int jr = sub * 32 + (r & 3) + 8 * (r >> 2);
           float x = s[sub][r];
           if constexpr (TIED) x *= kfs[cur * 64 + jr + 4 * half];
-          else x *= scale2;
+          else if constexpr (!WIN) x *= scale2;
           if constexpr (BIAS) x += fmaf(slope2, (float)jr, d0);
           if (edge) {
             const int j = j0 + jr + 4 * half;
-            x = j <= ip && j >= cs ? x : -1e30f;
+            x = j <= ip && (j >= cs || (WIN && j < keep)) ? x : -1e30f;
           }
           s[sub][r] = x;
           mt = fmaxf(mt, x);
@@ -286,14 +328,14 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
       }
     }
     // the other buffer's readers passed the barrier of the last page
-    if (pg < pg1) stage_write(cur ^ 1);
+    if (it + 1 < pages.n) stage_write(cur ^ 1);
     __syncthreads();
     cur ^= 1;
   }
 
   if (row < t.y) {
-    const float inv = l_run > 0.f ? 1.0f / l_run : 0.f;
-    short* dst = (short*)a.out + (long)(t.x + row) * a.H * a.vdim + (long)h * a.vdim;
+    const float inv = l_run > 0.f ? a.out_scale / l_run : 0.f;
+    short* dst = (short*)a.out + (long)(t.x + row) * a.ldo + (long)h * a.vdim;
     const short* gate = a.gate ? (const short*)a.gate + (long)(t.x + row) * a.ld +
                                      (long)h * a.vdim : nullptr;
     #pragma unroll
@@ -329,14 +371,17 @@ void launch(const AttnArgs& a, const int4* tiles, int n, hipStream_t st) {
 
 template <int DK, int DV>
 void pick_form(const AttnArgs& a, const int4* tiles, int n, hipStream_t st) {
-  if (a.slopes) launch<DK, DV, 1>(a, tiles, n, st);
+  if (a.bias) launch<DK, DV, 3>(a, tiles, n, st);
+  else if (a.slopes) launch<DK, DV, 1>(a, tiles, n, st);
   else launch<DK, DV, 0>(a, tiles, n, st);
 }
 
 }  // namespace
 
 bool lm_attn_mfma_ok(const AttnArgs& a) {
-  return a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 128 && a.vdim <= 128;
+  // rows of out that vectors can be stored to
+  return a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 128 && a.vdim <= 128 &&
+         a.ldo % 4 == 0 && (size_t)a.out % 8 == 0;
 }
 
 void lm_attn_prefill_mfma(const AttnArgs& a, const int4* tiles, int n_tiles,

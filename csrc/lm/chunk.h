@@ -40,15 +40,6 @@ template <bool F32, int D> struct RowStage {
   }
 };
 
-// value rows of a tile, zeros past its end
-template <bool F32, int DV>
-DEVINL void stage_v(const ColTile<F32, DV>& V, const typename Num<F32>::E* v0,
-                    long ld, int rows, int width, bool aligned) {
-  RowStage<F32, DV> r;
-  r.load(v0, ld, rows, width, aligned);
-  r.put(V, rows, width);
-}
-
 // dst [dv][dk] = sum_j v_j k_j^T.  Wave w owns DV/4 state rows, in groups
 // of 16; 64 columns at a time.
 template <bool F32, int DK, int DV>

@@ -58,7 +58,13 @@ void width_ok(long W) {
 LmNorm norm_of(const OptTensor& w, const OptTensor& b, const OptTensor& alpha,
                bool rms, long W, c10::ScalarType type, const char* name) {
   LmNorm n{};
-  n.w = opt_vec(w, W, type, name);
+  n.one = w.has_value() && w->dim() == 0;      // one number for all columns
+  if (n.one) {
+    shaped(*w, {}, type, name);
+    n.w = w->data_ptr();
+  } else {
+    n.w = opt_vec(w, W, type, name);
+  }
   n.b = opt_vec(b, W, type, name);
   n.rms = rms;
   if (alpha.has_value()) {
@@ -231,8 +237,26 @@ Tensor grouped_rms(Tensor y, Tensor w, long parts, double eps) {
   shaped(w, {y.size(1)}, y.scalar_type(), "norm weight");
   TORCH_CHECK(y.size(0) * parts < (1L << 31), "too many rows");
   auto out = torch::empty_like(y);
-  lm_grouped_rms(y.data_ptr(), w.data_ptr(), out.data_ptr(), y.size(0),
-                 (int)parts, (int)(y.size(1) / parts), (float)eps, is_f32(y),
+  lm_grouped_rms(y.data_ptr(), w.data_ptr(), nullptr, 0, out.data_ptr(),
+                 y.size(0), (int)parts, (int)(y.size(1) / parts), (float)eps,
+                 is_f32(y), cur_stream());
+  launched();
+  return out;
+}
+
+// RMS norm of whole rows, times the sigmoid of p's columns from `col` on
+Tensor gated_rms(Tensor y, Tensor w, Tensor p, long col, double eps) {
+  dense(y, "y"); dense(p, "p");
+  const long n = y.size(1);
+  shaped(w, {n}, y.scalar_type(), "norm weight");
+  TORCH_CHECK(y.dim() == 2 && p.dim() == 2 && p.size(0) == y.size(0) &&
+              p.scalar_type() == y.scalar_type() && col >= 0 &&
+              col + n <= p.size(1), "gates");
+  TORCH_CHECK(y.size(0) < (1L << 31), "too many rows");
+  auto out = torch::empty_like(y);
+  lm_grouped_rms(y.data_ptr(), w.data_ptr(),
+                 (const char*)p.data_ptr() + col * p.element_size(), p.size(1),
+                 out.data_ptr(), y.size(0), 1, (int)n, (float)eps, is_f32(y),
                  cur_stream());
   launched();
   return out;
@@ -277,11 +301,12 @@ AttnArgs attn_args(const Tensor& qkv, const Tensor& kc, const Tensor& vc,
   a.table = ints(table, 1, "page table");
   a.max_pages = (int)table.size(1);
   a.size = (int)size; a.scale = (float)scale; a.eps = (float)eps;
+  a.out_scale = 1.f;
   return a;
 }
 
 // Rows [0, n_dec) of a.qkv are single new tokens, the rest prompt portions
-// described by `tiles`; returns (T, heads * vdim).
+// described by `tiles`; returns (T, heads * vdim), or fills a.out if it is set.
 Tensor attend(AttnArgs& a, const Tensor& qkv, const Tensor& pos,
               const Tensor& slot, const Tensor& tiles, long n_dec,
               long max_len) {
@@ -292,8 +317,12 @@ Tensor attend(AttnArgs& a, const Tensor& qkv, const Tensor& pos,
   const int* sp = ints(slot, T, "slots");
   const long nt = tiles.numel() / 4;
   const int4* tp = (const int4*)ints(tiles, 4 * nt, "tiles");
-  auto out = torch::empty({T, (long)a.H * a.vdim}, qkv.options());
-  a.out = out.data_ptr();
+  Tensor out;
+  if (!a.out) {
+    out = torch::empty({T, (long)a.H * a.vdim}, qkv.options());
+    a.out = out.data_ptr();
+    a.ldo = out.size(1);
+  }
   auto st = cur_stream();
   if (n_dec > 0) {
     TORCH_CHECK(n_dec <= 65535, "too many decode rows");
@@ -302,7 +331,7 @@ Tensor attend(AttnArgs& a, const Tensor& qkv, const Tensor& pos,
     const long hg = a.H / a.G;
     const long hc = !f32 && lm_attn_decode_tied_mfma(a) ? 16 : hg <= 2 ? hg : 4;
     const long blocks = n_dec * a.G * ((hg + hc - 1) / hc);
-    const long keys = a.size > 0 ? std::min<long>(a.size, max_len) : max_len;
+    const long keys = a.size > 0 ? std::min<long>(a.size + a.keep, max_len) : max_len;
     long ns = std::min((512 + blocks - 1) / blocks, (keys + 127) / 128);
     ns = std::max<long>(1, std::min<long>(ns, 64));
     Tensor ws;
@@ -330,6 +359,55 @@ Tensor paged_attention(Tensor qkv, Tensor kc, Tensor vc, Tensor table,
   AttnArgs a = attn_args(qkv, kc, vc, table, qw, kw, sink, slopes, heads, size,
                          scale, eps);
   return attend(a, qkv, pos, slot, tiles, n_dec, max_len);
+}
+
+// columns [col, ...) of x: [q | k | v | gate]; result into columns
+// [out_col, ...) of out
+void window_attention(Tensor x, long col, Tensor out, long out_col, Tensor kc,
+                      Tensor vc, Tensor table, Tensor pos, Tensor slot,
+                      Tensor tiles, long n_dec, Tensor bias, double softcap,
+                      long heads, long size, long keep, double scale,
+                      double out_scale, double eps, long max_len) {
+  const auto ty = x.scalar_type();
+  is_f32(x);
+  dense(x, "rows"); dense(out, "out"); dense(kc, "key cache");
+  dense(vc, "value cache"); dense(table, "page table"); dense(bias, "bias");
+  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && kc.dim() == 4 && vc.dim() == 4 &&
+              table.dim() == 2 && bias.dim() == 2, "ranks");
+  AttnArgs a{};
+  a.H = (int)heads;
+  a.G = (int)kc.size(1);
+  a.dim = (int)kc.size(3);
+  a.vdim = (int)vc.size(3);
+  TORCH_CHECK(a.G >= 1 && a.H >= 1 && a.H % a.G == 0, "kv heads must divide heads");
+  TORCH_CHECK(a.dim >= 1 && a.dim <= 256 && a.vdim >= 1 && a.vdim <= 256,
+              "head sizes 1..256 are supported");
+  TORCH_CHECK(kc.size(2) == LM_PAGE && kc.scalar_type() == ty, "key cache");
+  shaped(vc, {kc.size(0), a.G, LM_PAGE, a.vdim}, ty, "value cache");
+  a.ld = x.size(1);
+  const long qk = (long)(a.H + a.G) * a.dim, g0 = qk + (long)a.G * a.vdim;
+  TORCH_CHECK(col >= 0 && col % 8 == 0 && a.ld % 8 == 0 &&
+              col + g0 + (long)a.H * a.vdim <= a.ld, "row length ", a.ld);
+  a.ldo = out.size(1);
+  TORCH_CHECK(out.size(0) == x.size(0) && out.scalar_type() == ty &&
+              out_col >= 0 && out_col + (long)a.H * a.vdim <= a.ldo, "out");
+  shaped(bias, {a.H, bias.size(1)}, torch::kFloat32, "bias");
+  TORCH_CHECK(bias.size(1) >= 1 && size >= 0 && keep >= 0 && softcap >= 0,
+              "window, bias, soft cap");
+  const size_t es = x.element_size();
+  a.qkv = (char*)x.data_ptr() + col * es;
+  a.gate = (const char*)a.qkv + g0 * es;
+  a.out = (char*)out.data_ptr() + out_col * es;
+  a.kc = kc.data_ptr(); a.vc = vc.data_ptr();
+  a.bias = bias.data_ptr<float>();
+  a.n_bias = (int)bias.size(1);
+  a.softcap = (float)softcap;
+  a.v_norm = true;
+  a.table = ints(table, 1, "page table");
+  a.max_pages = (int)table.size(1);
+  a.size = (int)size; a.keep = size > 0 ? (int)keep : 0;
+  a.scale = (float)scale; a.eps = (float)eps; a.out_scale = (float)out_scale;
+  attend(a, x, pos, slot, tiles, n_dec, max_len);
 }
 
 // rows [q | k | gate, the last if `gated`]; kc (pages, kv, 64, dim) takes k,
@@ -364,6 +442,7 @@ Tensor tied_attention(Tensor x, Tensor kc, Tensor ks, Tensor table, Tensor pos,
   a.qw = qw.data_ptr(); a.kw = kw.data_ptr();
   a.slopes = (const float*)opt_vec(slopes, a.H, torch::kFloat32, "slopes");
   a.has_sink = sink.has_value();
+  a.out_scale = 1.f;
   a.sink0 = (float)sink.value_or(0.0);
   a.t_coef = (float)t_coef; a.t_every = (int)t_every;
   a.table = ints(table, 1, "page table");
@@ -374,7 +453,8 @@ Tensor tied_attention(Tensor x, Tensor kc, Tensor ks, Tensor table, Tensor pos,
 
 Tensor retention(Tensor qkvg, Tensor state, Tensor pos, Tensor slot,
                  Tensor tiles, Tensor seqs, long n_dec, Tensor pows, Tensor dec,
-                 OptTensor cos_t, OptTensor sin_t, double kscale, double eps) {
+                 OptTensor cos_t, OptTensor sin_t, double kscale, double eps,
+                 bool light) {
   const bool f32 = is_f32(qkvg);
   dense(qkvg, "qkvg"); dense(state, "state");
   TORCH_CHECK(state.dim() == 4 && state.scalar_type() == torch::kFloat32, "state");
@@ -410,6 +490,7 @@ Tensor retention(Tensor qkvg, Tensor state, Tensor pos, Tensor slot,
   a.out = out.data_ptr(); a.pows = pows.data_ptr<float>();
   a.dec = dec.data_ptr<float>();
   a.kscale = (float)kscale; a.eps = (float)eps;
+  a.silu = a.raw = light;
   auto st = cur_stream();
   if (n_dec > 0) lm_ret_decode(a, pp, sp, (int)n_dec, f32, st);
   if (nt > 0) {
@@ -447,6 +528,127 @@ Plan plan_of(const Tensor& pos, const Tensor& slot, const Tensor& tiles,
 
 const void* at(const Tensor& t, long i) {
   return (const char*)t.data_ptr() + i * t.element_size();
+}
+
+RaggedRows ragged(const Plan& g, long T) {
+  return RaggedRows{g.pos, g.slot, g.tiles, g.seqs, g.n_seqs, g.n_dec, (int)T};
+}
+
+// tokens (T,) -> float stream x (T, W); last (slots,) the tokens before
+Tensor stream_embed(Tensor tokens, Tensor embed, Tensor pos, Tensor slot,
+                    Tensor tiles, Tensor seqs, long n_dec, OptTensor rates,
+                    OptTensor pairs, long mul_prev, long mul_cur,
+                    OptTensor last) {
+  dense(embed, "embed");
+  const bool f32 = is_f32(embed);
+  const long T = tokens.numel(), W = embed.size(1);
+  width_ok(W);
+  EmbedArgs a{};
+  a.tokens = token_ids(tokens, T);
+  a.embed = embed.data_ptr(); a.vocab = embed.size(0); a.W = (int)W;
+  if (rates.has_value()) {
+    shaped(*rates, {(W + 1) / 2}, torch::kFloat64, "turn rates");
+    a.rates = rates->data_ptr<double>();
+  }
+  if (pairs.has_value()) {
+    TORCH_CHECK(pairs->dim() == 2 && pairs->size(0) >= 2 && last.has_value(), "pairs");
+    a.buckets = pairs->size(0) - 1;
+    shaped(*pairs, {a.buckets + 1, W}, embed.scalar_type(), "pairs");
+    dense(*last, "last tokens");
+    TORCH_CHECK(last->dim() == 1 && last->scalar_type() == torch::kInt64, "last tokens");
+    a.pairs = pairs->data_ptr();
+    a.mul_prev = mul_prev; a.mul_cur = mul_cur;
+    a.last = (long*)last->data_ptr<int64_t>();
+  }
+  const Plan g = plan_of(pos, slot, tiles, seqs, n_dec, T);
+  auto x = torch::empty({T, W}, embed.options().dtype(torch::kFloat32));
+  a.x = x.data_ptr<float>();
+  lm_stream_embed(a, ragged(g, T), f32, cur_stream());
+  launched();
+  return x;
+}
+
+// {x + mult * y + add + step, its norm blended with the row before}
+std::vector<Tensor> shift_norm(Tensor x, OptTensor y, OptTensor weights,
+                               double mult, Tensor nw, OptTensor nb,
+                               OptTensor na, bool n_rms, double eps, Tensor pos,
+                               Tensor slot, Tensor tiles, Tensor seqs,
+                               long n_dec, OptTensor shift, OptTensor state,
+                               OptTensor add, OptTensor step) {
+  const bool f32 = is_f32(nw);
+  const auto ty = nw.scalar_type();
+  ShiftArgs a{};
+  a.x = stream_x(x);
+  const long T = x.size(0), W = x.size(1);
+  TORCH_CHECK(!na.has_value(), "a dynamic tanh is not served here");
+  a.y = sum_of(y, weights, T, W, ty);
+  a.mult = (float)mult;
+  a.nxt = norm_of(nw, nb, na, n_rms, W, ty, "norm");
+  a.W = (int)W; a.eps = (float)eps;
+  if (shift.has_value()) {
+    TORCH_CHECK(state.has_value() && state->dim() == 2, "state of the shift");
+    a.shift = opt_vec(shift, W, ty, "shift");
+    shaped(*state, {state->size(0), W}, torch::kFloat32, "state of the shift");
+    a.state = state->data_ptr<float>();
+  }
+  if (add.has_value()) {
+    shaped(*add, {T, W}, torch::kFloat32, "added stream");
+    a.add = add->data_ptr<float>();
+  }
+  a.step = opt_vec(step, W, ty, "step");
+  const Plan g = plan_of(pos, slot, tiles, seqs, n_dec, T);
+  auto xo = torch::empty_like(x);
+  auto h = torch::empty({T, W}, nw.options());
+  a.xo = xo.data_ptr<float>(); a.h = h.data_ptr();
+  lm_shift_norm(a, ragged(g, T), f32, cur_stream());
+  launched();
+  return {xo, h};
+}
+
+// columns [col, ...) of x: [q | k | v | gate | what makes the decays]; result
+// into columns [out_col, ...) of out
+void gla(Tensor x, long col, Tensor out, long out_col, Tensor state, Tensor pos,
+         Tensor slot, Tensor tiles, Tensor seqs, long n_dec, Tensor a2,
+         Tensor a2b, double tau, Tensor norm, double out_scale, double eps) {
+  const bool f32 = is_f32(x);
+  const auto ty = x.scalar_type();
+  dense(x, "rows"); dense(out, "out"); dense(state, "state"); dense(a2, "a2");
+  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && a2.dim() == 2, "ranks");
+  TORCH_CHECK(state.dim() == 4 && state.scalar_type() == torch::kFloat32, "state");
+  GlaArgs a{};
+  a.H = (int)state.size(1);
+  a.dv = (int)state.size(2);
+  a.dk = (int)state.size(3);
+  a.rank = (int)a2.size(1);
+  TORCH_CHECK(a.dk >= 1 && a.dk <= 256 && a.dv >= 1 && a.dv <= 256,
+              "head sizes 1..256 are supported");
+  TORCH_CHECK(a.H >= 1 && a.H <= 65535 && a.rank >= 1, "heads, rank");
+  TORCH_CHECK(tau > 0, "tau");
+  const long qk = (long)a.H * a.dk, vv = (long)a.H * a.dv, T = x.size(0);
+  a.ld = x.size(1); a.ldo = out.size(1);
+  TORCH_CHECK(col >= 0 && col % 8 == 0 && a.ld % 8 == 0 &&
+              col + 2 * (qk + vv) + a.rank <= a.ld, "row length ", a.ld);
+  TORCH_CHECK(out.size(0) == T && out.scalar_type() == ty && out_col >= 0 &&
+              out_col + vv <= a.ldo, "out");
+  shaped(a2, {qk, a.rank}, ty, "decay matrix");
+  shaped(a2b, {qk}, ty, "decay bias");
+  shaped(norm, {a.dv}, ty, "norm weight");
+  const Plan g = plan_of(pos, slot, tiles, seqs, n_dec, T);
+  a.q = at(x, col); a.k = at(x, col + qk); a.v = at(x, col + 2 * qk);
+  a.gate = at(x, col + 2 * qk + vv); a.u = at(x, col + 2 * (qk + vv));
+  a.a2 = a2.data_ptr(); a.a2b = a2b.data_ptr(); a.norm = norm.data_ptr();
+  a.state = state.data_ptr<float>();
+  a.out = (char*)out.data_ptr() + out_col * out.element_size();
+  a.qscale = 1.0f / std::sqrt((float)a.dk); a.inv_tau = (float)(1.0 / tau);
+  a.out_scale = (float)out_scale; a.eps = (float)eps;
+  auto st = cur_stream();
+  lm_gla_decode(a, g.pos, g.slot, g.n_dec, f32, st);
+  if (g.n_tiles > 0) {
+    auto ws = torch::empty({lm_gla_scratch(a, g.n_tiles)}, state.options());
+    lm_gla_prefill(a, g.tiles, g.n_tiles, g.seqs, g.n_seqs,
+                   ws.data_ptr<float>(), f32, st);
+  }
+  launched();
 }
 
 // convolution and silu over columns [col, col + channels) of p
@@ -688,18 +890,15 @@ Tensor router_logits(Tensor x, Tensor r) {
   return z;
 }
 
-// z (T, >= E + 1 with a shared expert) router logits, x (T, W); returns the
-// places' outputs y (T, K, W) and their weights (T, K)
-std::vector<Tensor> moe(Tensor x, Tensor z, Tensor gu, Tensor down,
-                        OptTensor sgu, OptTensor sdown, long top, long groups,
-                        long keep, double scale) {
+// sizes and operands of a routed feed-forward without what chooses
+MoeArgs moe_args(const Tensor& x, const Tensor& gu, const Tensor& down,
+                 const OptTensor& sgu, const OptTensor& sdown, long top) {
   const auto ty = x.scalar_type();
-  const bool f32 = is_f32(x);
-  dense(x, "x"); dense(z, "router logits"); dense(gu, "gate and up"); dense(down, "down");
-  TORCH_CHECK(x.dim() == 2 && z.dim() == 2 && gu.dim() == 3, "ranks");
+  dense(x, "x"); dense(gu, "gate and up"); dense(down, "down");
+  TORCH_CHECK(x.dim() == 2 && gu.dim() == 3, "ranks");
   MoeArgs a{};
-  const long T = x.size(0);
-  a.T = (int)T; a.W = (int)x.size(1);
+  TORCH_CHECK(x.size(0) < (1L << 30), "too many tokens");
+  a.T = (int)x.size(0); a.W = (int)x.size(1);
   a.E = (int)gu.size(0);
   a.ff = (int)gu.size(1) / 2;
   shaped(gu, {a.E, 2L * a.ff, a.W}, ty, "gate and up");
@@ -714,27 +913,27 @@ std::vector<Tensor> moe(Tensor x, Tensor z, Tensor gu, Tensor down,
     a.K = a.top + 1;
   }
   TORCH_CHECK(a.E >= 1 && a.E <= LM_MOE_EXPERTS && a.ff >= 1, "experts");
-  TORCH_CHECK(groups >= 1 && groups <= LM_MOE_GROUPS && a.E % groups == 0 &&
-              keep >= 1 && keep <= groups, "expert groups");
-  TORCH_CHECK(top >= 1 && top <= LM_MOE_TOP && top <= keep * (a.E / groups),
-              "too few experts to choose from");
-  TORCH_CHECK(T * a.K < (1L << 30), "too many tokens");
-  a.ldz = (int)z.size(1);
-  TORCH_CHECK(z.size(0) == T && a.ldz >= a.E + (a.K - a.top) &&
-              z.scalar_type() == torch::kFloat32, "router logits");
-  a.groups = (int)groups; a.keep = (int)keep; a.scale = (float)scale;
-  a.z = z.data_ptr<float>();
+  TORCH_CHECK(top >= 1 && top <= LM_MOE_TOP, "experts per token");
+  TORCH_CHECK((long)a.T * a.K < (1L << 30), "too many tokens");
   a.x = x.data_ptr(); a.gu = gu.data_ptr(); a.down = down.data_ptr();
+  return a;
+}
+
+// chooses and runs; returns the places' outputs y (T, K, W) and their weights
+// (T, K)
+std::vector<Tensor> moe_run(MoeArgs& a, const Tensor& x) {
+  const bool f32 = is_f32(x);
+  const long T = a.T;
   a.lda = (std::max(a.ff, a.ffs) + 7) / 8 * 8;
   a.rows = lm_moe_rows(a, f32);
   // each expert's last tile may be short
-  const long nt = (T * top + a.rows - 1) / a.rows + std::min<long>(a.E, T * top) +
+  const long nt = (T * a.top + a.rows - 1) / a.rows + std::min<long>(a.E, T * a.top) +
                   (a.K > a.top ? (T + a.rows - 1) / a.rows : 0);
   TORCH_CHECK(nt <= 65535, "too many tiles");
   a.n_tiles = (int)nt;
-  auto ints32 = x.options().dtype(torch::kInt32);
-  auto wts = torch::empty({T, a.K}, z.options());
-  auto plan = torch::empty({4 * nt + T * a.K + T * top}, ints32);
+  auto wts = torch::empty({T, a.K}, x.options().dtype(torch::kFloat32));
+  auto plan = torch::empty({4 * nt + T * a.K + T * a.top},
+                           x.options().dtype(torch::kInt32));
   auto act = torch::empty({T * a.K, (long)a.lda}, x.options());
   auto y = torch::empty({T, (long)a.K, (long)a.W}, x.options());
   a.wts = wts.data_ptr<float>();
@@ -748,6 +947,35 @@ std::vector<Tensor> moe(Tensor x, Tensor z, Tensor gu, Tensor down,
   return {y, wts};
 }
 
+// z (T, >= E + 1 with a shared expert) router logits, x (T, W)
+std::vector<Tensor> moe(Tensor x, Tensor z, Tensor gu, Tensor down,
+                        OptTensor sgu, OptTensor sdown, long top, long groups,
+                        long keep, double scale) {
+  MoeArgs a = moe_args(x, gu, down, sgu, sdown, top);
+  dense(z, "router logits");
+  TORCH_CHECK(z.dim() == 2, "ranks");
+  TORCH_CHECK(groups >= 1 && groups <= LM_MOE_GROUPS && a.E % groups == 0 &&
+              keep >= 1 && keep <= groups, "expert groups");
+  TORCH_CHECK(top <= keep * (a.E / groups), "too few experts to choose from");
+  a.ldz = (int)z.size(1);
+  TORCH_CHECK(z.size(0) == a.T && a.ldz >= a.E + (a.K - a.top) &&
+              z.scalar_type() == torch::kFloat32, "router logits");
+  a.groups = (int)groups; a.keep = (int)keep; a.scale = (float)scale;
+  a.z = z.data_ptr<float>();
+  return moe_run(a, x);
+}
+
+// table (vocab, top): the experts of each token id
+std::vector<Tensor> table_moe(Tensor x, Tensor tokens, Tensor table, Tensor gu,
+                              Tensor down) {
+  TORCH_CHECK(table.dim() == 2 && table.size(0) >= 1, "table");
+  MoeArgs a = moe_args(x, gu, down, c10::nullopt, c10::nullopt, table.size(1));
+  a.tokens = token_ids(tokens, a.T);
+  a.vocab = table.size(0);
+  a.table = ints(table, table.numel(), "table");
+  return moe_run(a, x);
+}
+
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -759,6 +987,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gelu_erf", &gelu_erf, "exact GELU");
   m.def("paged_attention", &paged_attention,
         "chunked causal attention with sink over a paged cache");
+  m.def("window_attention", &window_attention,
+        "window attention with kept first tokens over a paged cache");
+  m.def("gla", &gla, "gated linear attention over state slots");
+  m.def("gated_rms", &gated_rms, "RMS norm of rows behind a sigmoid gate");
+  m.def("stream_embed", &stream_embed, "embeddings, positions and pairs");
+  m.def("shift_norm", &shift_norm,
+        "residual add and a norm blended with the token before");
+  m.def("table_moe", &table_moe, "experts by token id");
   m.def("retention", &retention, "retention over state slots");
   m.def("residual_concat", &residual_concat,
         "residual add, then the stream beside the embeddings");

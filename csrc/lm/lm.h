@@ -22,6 +22,7 @@ struct LmNorm {
   const void* b;      // or null
   const void* alpha;  // one element, or null
   bool rms;
+  bool one;           // w is one element, for all columns
 };
 // a sublayer's output: y [T][W] (or null), or with weights w [T][n] the
 // weighted sum over n of y [T][n][W]
@@ -57,9 +58,49 @@ void lm_gated_act(const void* in, void* out, long rows, int n, int act,
                   hipStream_t stream);
 void lm_softcap(const void* in, float* out, long n, float cap, bool f32,
                 hipStream_t stream);
-// RMS norm of each of a row's `parts` spans of n elements, times w
-void lm_grouped_rms(const void* y, const void* w, void* out, long rows,
-                    int parts, int n, float eps, bool f32, hipStream_t stream);
+// RMS norm of each of a row's `parts` spans of n elements, times w and, if
+// there is a gate (rows of stride ldg), its sigmoid
+void lm_grouped_rms(const void* y, const void* w, const void* gate, long ldg,
+                    void* out, long rows, int parts, int n, float eps, bool f32,
+                    hipStream_t stream);
+
+// ---- stream.hip: the start of a stream, and norms that look a token back
+struct RaggedRows {   // where the rows of a batch lie (see StepPlan)
+  const int* pos;
+  const int* slot;
+  const int4* tiles;  // first row, rows, position, slot
+  const int4* seqs;   // first tile, tiles, position, slot
+  int n_seqs, n_dec, T;
+};
+struct EmbedArgs {
+  const long* tokens;
+  const void* embed;
+  long vocab;
+  const double* rates;  // [(W + 1) / 2] turns per position, or null
+  const void* pairs;    // [buckets + 1][W] or null
+  long buckets, mul_prev, mul_cur;
+  long* last;           // [slots] the token before
+  float* x;
+  int W;
+};
+void lm_stream_embed(const EmbedArgs& a, const RaggedRows& r, bool f32,
+                     hipStream_t stream);
+struct ShiftArgs {
+  const float* x;
+  LmSum y;
+  float mult;
+  const float* add;     // [T][W] or null
+  const void* step;     // [W] or null
+  LmNorm nxt;           // no alpha
+  const void* shift;    // [W] or null
+  float* state;         // [slots][W], with shift
+  float* xo;            // x + mult * y + add + step; not x
+  void* h;              // its norm, blended with the row before
+  int W;
+  float eps;
+};
+void lm_shift_norm(const ShiftArgs& a, const RaggedRows& r, bool f32,
+                   hipStream_t stream);
 
 // ---- attn.hip / attn_decode.hip
 struct AttnArgs {
@@ -74,6 +115,16 @@ struct AttnArgs {
   const void* sink;   // [heads] or null: every head's is sink0
   float sink0;
   bool has_sink;
+  long ldo;           // row stride of out
+  float out_scale;    // multiplies out
+  bool v_norm;        // each head's value over its root mean square
+  // window form (bias not null): `size` is a sliding window, beside which the
+  // first `keep` tokens stay visible; softcap * tanh(score / softcap)
+  // (softcap 0: the score), then bias[h][min(distance, n_bias - 1)]
+  const float* bias;  // [heads][n_bias]
+  int n_bias;
+  int keep;
+  float softcap;
   const float* slopes;  // [heads] taken off a score per step of distance, or null
   // tied form (ks not null): the cached rows are the keys before their norm
   // and the values as well; token j's score takes the factor ks[j].  Norms
@@ -86,7 +137,7 @@ struct AttnArgs {
   const int* table;
   int max_pages;
   int H, G, dim, vdim;
-  int size;           // chunk length in tokens; 0 = plain causal
+  int size;           // chunk or window length in tokens; 0 = plain causal
   float scale;
   float eps;
 };
@@ -118,12 +169,39 @@ struct RetArgs {
   int H, dk, dv, rd;
   float kscale;
   float eps;
+  bool silu;          // of q, k and v as they are read
+  bool raw;           // out takes S^T q as it is, without norm and gate
 };
 // cs [n_tiles][H][dv][dk] scratch; seqs int4 {first tile, tiles, pos0, slot}
 void lm_ret_prefill(const RetArgs& a, const int4* tiles, int n_tiles,
                     const int4* seqs, int n_seqs, float* cs, bool f32,
                     hipStream_t stream);
 void lm_ret_decode(const RetArgs& a, const int* pos, const int* slot, int R,
+                   bool f32, hipStream_t stream);
+
+// ---- gla.hip: a decay per key channel and token
+struct GlaArgs {
+  const void* q;      // rows of stride ld: q, k [H][dk], v, gate [H][dv], u
+  const void* k;
+  const void* v;
+  const void* gate;
+  const void* u;      // [rank]
+  long ld;
+  const void* a2;     // [H * dk][rank], [H * dk]: what makes the decay of u
+  const void* a2b;
+  const void* norm;   // [dv]
+  float* state;       // [slots][H][dv][dk]
+  void* out;          // rows of stride ldo, [H][dv]
+  long ldo;
+  int H, dk, dv, rank;
+  float qscale, inv_tau, out_scale, eps;
+};
+// floats of scratch that a prompt of n_tiles tiles needs
+long lm_gla_scratch(const GlaArgs& a, int n_tiles);
+void lm_gla_prefill(const GlaArgs& a, const int4* tiles, int n_tiles,
+                    const int4* seqs, int n_seqs, float* ws, bool f32,
+                    hipStream_t stream);
+void lm_gla_decode(const GlaArgs& a, const int* pos, const int* slot, int R,
                    bool f32, hipStream_t stream);
 
 // ---- mamba2.hip / mlstm.hip: recurrences with a decay per head and token
@@ -221,6 +299,9 @@ struct MoeArgs {
   int ff, ffs;           // inner widths of experts and shared expert (0: none)
   const float* z;        // router logits [T][ldz], the shared gate's after E
   int ldz;
+  const int* table;      // null, or [vocab][top]: a token's experts, no router
+  const long* tokens;    // [T]
+  long vocab;
   int groups, keep;
   float scale;
   float* wts;            // [T][K]

@@ -1,5 +1,5 @@
-// Routed feed-forward: sigmoid router with expert groups, gated experts and
-// a shared expert.
+// Routed feed-forward: sigmoid router with expert groups, or a table of token
+// ids, gated experts and a shared expert.
 //
 // One plan kernel chooses the experts, sorts the (token, place) entries by
 // expert and cuts them into tiles; two grouped products follow,
@@ -142,7 +142,9 @@ moe_route_kernel(MoeArgs a) {
   if (t < a.T) route_token<NPL>(a, t, sc[w], threadIdx.x & 63);
 }
 
-// One block sorts the entries; ROUTE: and routes the tokens before that.
+// One block sorts the entries; ROUTE: and routes the tokens before that.  With
+// a table nothing is routed: a token's experts are read there and have equal
+// weights.
 template <int NPL, bool ROUTE>
 __global__ void __launch_bounds__(1024)
 moe_plan_kernel(MoeArgs a) {
@@ -152,9 +154,15 @@ moe_plan_kernel(MoeArgs a) {
   for (int e = tid; e < NPL * 64; e += 1024) cnt[e] = 0;
   if constexpr (ROUTE)
     for (int t = w; t < a.T; t += 16) route_token<NPL>(a, t, sc[w], l);
+  const int n = a.T * a.top;
+  if (a.table)
+    for (int i = tid; i < n; i += 1024) {
+      const long tok = min(max(a.tokens[i / a.top], 0l), a.vocab - 1);
+      a.ids[i] = min(max(a.table[tok * a.top + i % a.top], 0), a.E - 1);
+      a.wts[i] = 1.0f / (float)a.top;
+    }
   __threadfence_block();
   __syncthreads();
-  const int n = a.T * a.top;
   for (int i = tid; i < n; i += 1024) atomicAdd(&cnt[a.ids[i]], 1);
   __syncthreads();
   if (w == 0) {                        // entries and tiles before each expert
@@ -499,7 +507,9 @@ Kind pick(const MoeArgs& a, bool f32) {
 
 template <int NPL>
 void plan(const MoeArgs& a, hipStream_t st) {
-  if (a.T <= 32) {
+  if (a.table) {
+    hipLaunchKernelGGL((moe_plan_kernel<NPL, false>), dim3(1), dim3(1024), 0, st, a);
+  } else if (a.T <= 32) {
     hipLaunchKernelGGL((moe_plan_kernel<NPL, true>), dim3(1), dim3(1024), 0, st, a);
   } else {
     hipLaunchKernelGGL((moe_route_kernel<NPL>), dim3((a.T + 3) / 4), dim3(256), 0, st, a);

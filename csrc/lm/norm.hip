@@ -10,115 +10,11 @@
 // with the tokens' embeddings e, and x <- y + step.
 //
 // Rows up to 2048 wide take one wave each (4 rows a block, shuffles
-// only); wider rows, and few rows that are not narrow, take a 4-wave block.  Row values stay in registers
-// between the mean and the variance pass.
+// only); wider rows, and few rows that are not narrow, take a 4-wave block.
 
-#include "lm.h"
-#include "tile.h"
+#include "norm.h"
 
 namespace {
-
-template <int VEC> struct Pack { float v[VEC]; };
-
-template <bool F32, int VEC>
-DEVINL Pack<VEC> ldv(const void* base, long i) {
-  Pack<VEC> p;
-  if constexpr (F32) {
-    const float* s = (const float*)base + i;
-    if constexpr (VEC == 4) *(f32x4*)p.v = *(const f32x4*)s;
-    else p.v[0] = s[0];
-  } else {
-    const short* s = (const short*)base + i;
-    if constexpr (VEC == 4) {
-      const bf16x4 t = *(const bf16x4*)s;
-      #pragma unroll
-      for (int j = 0; j < 4; ++j) p.v[j] = bf2f(t[j]);
-    } else {
-      p.v[0] = bf2f(s[0]);
-    }
-  }
-  return p;
-}
-
-// VEC elements as stored (half the registers of their float form in bf16)
-template <bool F32, int VEC> struct Held {
-  typename Num<F32>::E e[VEC];
-  DEVINL void load(const void* base, long i) {
-    const auto* s = (const typename Num<F32>::E*)base + i;
-    if constexpr (VEC == 4 && F32) *(f32x4*)e = *(const f32x4*)s;
-    else if constexpr (VEC == 4) *(bf16x4*)e = *(const bf16x4*)s;
-    else e[0] = s[0];
-  }
-  DEVINL Pack<VEC> up() const {
-    Pack<VEC> p;
-    #pragma unroll
-    for (int j = 0; j < VEC; ++j) p.v[j] = Num<F32>::up(e[j]);
-    return p;
-  }
-};
-
-template <bool F32, int VEC>
-DEVINL void stv(void* base, long i, const Pack<VEC>& p) {
-  if constexpr (F32) {
-    float* s = (float*)base + i;
-    if constexpr (VEC == 4) *(f32x4*)s = *(const f32x4*)p.v;
-    else s[0] = p.v[0];
-  } else {
-    short* s = (short*)base + i;
-    if constexpr (VEC == 4) {
-      bf16x4 t;
-      #pragma unroll
-      for (int j = 0; j < 4; ++j) t[j] = cvt_bf16(p.v[j]);
-      *(bf16x4*)s = t;
-    } else {
-      s[0] = cvt_bf16(p.v[0]);
-    }
-  }
-}
-
-template <int TPR>
-DEVINL float row_sum(float v, float* red) {
-  v = group_sum<64>(v);
-  if constexpr (TPR == 256) {
-    const int w = threadIdx.x >> 6;
-    __syncthreads();             // the previous use of red is over
-    if ((threadIdx.x & 63) == 0) red[w] = v;
-    __syncthreads();
-    v = red[0] + red[1] + red[2] + red[3];
-  }
-  return v;
-}
-
-// rms: without taking the mean off
-template <int TPR, int VEC, int NV>
-DEVINL void layer_norm_rows(Pack<VEC> (&v)[NV], int tid, int W, float eps,
-                            bool rms, float* red) {
-  float mean = 0.f;
-  if (!rms) {
-    float s = 0.f;
-    #pragma unroll
-    for (int i = 0; i < NV; ++i)
-      #pragma unroll
-      for (int j = 0; j < VEC; ++j) s += v[i].v[j];  // lanes past W hold 0
-    mean = row_sum<TPR>(s, red) / (float)W;
-  }
-  float q = 0.f;
-  #pragma unroll
-  for (int i = 0; i < NV; ++i) {
-    const bool ok = (i * TPR + tid) * VEC < W;
-    #pragma unroll
-    for (int j = 0; j < VEC; ++j) {
-      const float d = v[i].v[j] - mean;
-      v[i].v[j] = d;
-      q += ok ? d * d : 0.f;
-    }
-  }
-  const float inv = 1.0f / sqrtf(row_sum<TPR>(q, red) / (float)W + eps);
-  #pragma unroll
-  for (int i = 0; i < NV; ++i)
-    #pragma unroll
-    for (int j = 0; j < VEC; ++j) v[i].v[j] *= inv;
-}
 
 // tanh(alpha * v), what a dynamic tanh has in place of statistics
 template <int VEC, int NV>
@@ -143,7 +39,7 @@ struct NormArgs {
   const void* pw;       // its norm (null: y is added as it is)
   const void* pb;
   const void* pa;       // its alpha: dynamic tanh (null: layer or RMS norm)
-  bool p_rms;
+  bool p_rms, p_one, n_one;   // *_one: a single weight for all columns
   float mult;
   const void* nw;       // next norm or null
   const void* nb;
@@ -181,9 +77,9 @@ residual_norm_kernel(NormArgs a) {
       const int c = (i * TPR + tid) * VEC;
       wp[i] = bp[i] = wn[i] = bn[i] = Held<F32, VEC>{};
       if (c < W) {
-        if (a.pw) wp[i].load(a.pw, c);
+        if (a.pw) wp[i].load_weight(a.pw, c, a.p_one);
         if (a.pb) bp[i].load(a.pb, c);
-        if (a.nw) wn[i].load(a.nw, c);
+        if (a.nw) wn[i].load_weight(a.nw, c, a.n_one);
         if (a.nb) bn[i].load(a.nb, c);
       }
     }
@@ -282,7 +178,9 @@ residual_norm_kernel(NormArgs a) {
             w = wp[i].up();
             b = bp[i].up();
           } else {
-            w = ldv<F32, VEC>(a.pw, c);
+            Held<F32, VEC> t;
+            t.load_weight(a.pw, c, a.p_one);
+            w = t.up();
             if (a.pb) b = ldv<F32, VEC>(a.pb, c);
           }
           #pragma unroll
@@ -323,7 +221,9 @@ residual_norm_kernel(NormArgs a) {
           w = wn[i].up();
           b = bn[i].up();
         } else {
-          w = ldv<F32, VEC>(a.nw, c);
+          Held<F32, VEC> t;
+          t.load_weight(a.nw, c, a.n_one);
+          w = t.up();
           if (a.nb) b = ldv<F32, VEC>(a.nb, c);
         }
         #pragma unroll
@@ -437,14 +337,17 @@ softcap_kernel(const void* in, float* out, long n4, long n, float cap) {
   }
 }
 
-// y * inv_rms(y) * w over equal parts of a row, one block per (row, part)
+// y * inv_rms(y) * w (* sigmoid(gate)) over equal parts of a row, one block
+// per (row, part); gate: rows of stride ldg, or null
 template <bool F32, int VEC>
 __global__ void __launch_bounds__(256)
 grouped_rms_kernel(const void* __restrict__ y, const void* __restrict__ w,
+                   const void* __restrict__ gate, long ldg,
                    void* __restrict__ out, int parts, int n, float eps) {
   __shared__ float red[4];
   const long off = (long)blockIdx.x * n;
   const long woff = (long)(blockIdx.x % parts) * n;
+  const long goff = blockIdx.x / parts * ldg + woff;
   float q = 0.f;
   for (int c = threadIdx.x * VEC; c < n; c += 256 * VEC) {
     const Pack<VEC> v = ldv<F32, VEC>(y, off + c);
@@ -455,8 +358,13 @@ grouped_rms_kernel(const void* __restrict__ y, const void* __restrict__ w,
   for (int c = threadIdx.x * VEC; c < n; c += 256 * VEC) {
     Pack<VEC> v = ldv<F32, VEC>(y, off + c);
     const Pack<VEC> g = ldv<F32, VEC>(w, woff + c);
+    Pack<VEC> z;
+    if (gate) z = ldv<F32, VEC>(gate, goff + c);
     #pragma unroll
-    for (int j = 0; j < VEC; ++j) v.v[j] *= inv * g.v[j];
+    for (int j = 0; j < VEC; ++j) {
+      v.v[j] *= inv * g.v[j];
+      if (gate) v.v[j] /= 1.0f + expf(-z.v[j]);
+    }
     stv<F32, VEC>(out, off + c, v);
   }
 }
@@ -470,7 +378,7 @@ void lm_embed_norm(const long* tokens, const void* embed, const int* pos,
   NormArgs a{};
   a.tokens = tokens; a.embed = embed; a.vocab = vocab;
   a.pos = pos; a.ptab = ptab; a.n_pos = n_pos;
-  a.x = x; a.nw = nxt.w; a.nb = nxt.b; a.na = nxt.alpha; a.n_rms = nxt.rms;
+  a.x = x; a.nw = nxt.w; a.nb = nxt.b; a.na = nxt.alpha; a.n_rms = nxt.rms; a.n_one = nxt.one;
   a.h = h; a.T = T; a.W = W; a.eps = eps;
   dispatch_norm(a, f32, stream);
 }
@@ -479,8 +387,8 @@ void lm_residual_norm(float* x, LmSum y, LmNorm post, float mult,
                       LmNorm nxt, void* h, const int* rows, int T, int W,
                       float eps, bool store_x, bool f32, hipStream_t stream) {
   NormArgs a{};
-  a.x = x; a.y = y.y; a.mw = y.w; a.mix = y.n; a.pw = post.w; a.pb = post.b; a.pa = post.alpha; a.p_rms = post.rms;
-  a.mult = mult; a.nw = nxt.w; a.nb = nxt.b; a.na = nxt.alpha; a.n_rms = nxt.rms;
+  a.x = x; a.y = y.y; a.mw = y.w; a.mix = y.n; a.pw = post.w; a.pb = post.b; a.pa = post.alpha; a.p_rms = post.rms; a.p_one = post.one;
+  a.mult = mult; a.nw = nxt.w; a.nb = nxt.b; a.na = nxt.alpha; a.n_rms = nxt.rms; a.n_one = nxt.one;
   a.h = h; a.rows = rows; a.T = T; a.W = W; a.eps = eps; a.store_x = store_x;
   dispatch_norm(a, f32, stream);
 }
@@ -490,7 +398,7 @@ void lm_residual_concat(float* x, LmSum y, LmNorm post, float mult,
                         int W, long vocab, float eps, bool f32,
                         hipStream_t stream) {
   NormArgs a{};
-  a.x = x; a.y = y.y; a.mw = y.w; a.mix = y.n; a.pw = post.w; a.pb = post.b; a.pa = post.alpha; a.p_rms = post.rms;
+  a.x = x; a.y = y.y; a.mw = y.w; a.mix = y.n; a.pw = post.w; a.pb = post.b; a.pa = post.alpha; a.p_rms = post.rms; a.p_one = post.one;
   a.mult = mult; a.tokens = tokens; a.embed = embed; a.vocab = vocab;
   a.cat = true; a.h = h; a.T = T; a.W = W; a.eps = eps; a.store_x = true;
   dispatch_norm(a, f32, stream);
@@ -501,7 +409,7 @@ void lm_replace_norm(float* x, const void* y, bool y_f32, const void* step,
                      hipStream_t stream) {
   NormArgs a{};
   a.x = x; a.y = y; a.y_f32 = y_f32; a.step = step;
-  a.nw = nxt.w; a.nb = nxt.b; a.na = nxt.alpha; a.n_rms = nxt.rms;
+  a.nw = nxt.w; a.nb = nxt.b; a.na = nxt.alpha; a.n_rms = nxt.rms; a.n_one = nxt.one;
   a.h = h; a.T = T; a.W = W; a.eps = eps;
   dispatch_norm(a, f32, stream);
 }
@@ -550,16 +458,19 @@ void lm_softcap(const void* in, float* out, long n, float cap, bool f32,
     hipLaunchKernelGGL((softcap_kernel<false>), grid, dim3(256), 0, stream, in, out, n4, n, cap);
 }
 
-void lm_grouped_rms(const void* y, const void* w, void* out, long rows,
-                    int parts, int n, float eps, bool f32, hipStream_t stream) {
+void lm_grouped_rms(const void* y, const void* w, const void* gate, long ldg,
+                    void* out, long rows, int parts, int n, float eps, bool f32,
+                    hipStream_t stream) {
   if (rows <= 0) return;
   const dim3 grid((unsigned)(rows * parts));
+  // vectors need every row's start aligned
+  const bool v4 = n % 4 == 0 && (!gate || (ldg % 4 == 0 && (size_t)gate % 16 == 0));
   #define GR_GO(F, V)                                                          \
     hipLaunchKernelGGL((grouped_rms_kernel<F, V>), grid, dim3(256), 0, stream, \
-                       y, w, out, parts, n, eps)
-  if (f32 && n % 4 == 0) GR_GO(true, 4);
+                       y, w, gate, ldg, out, parts, n, eps)
+  if (f32 && v4) GR_GO(true, 4);
   else if (f32) GR_GO(true, 1);
-  else if (n % 4 == 0) GR_GO(false, 4);
+  else if (v4) GR_GO(false, 4);
   else GR_GO(false, 1);
   #undef GR_GO
 }

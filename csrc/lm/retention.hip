@@ -15,10 +15,16 @@
 // q and k are rotated while they are staged; from there on they, the decay
 // powers and the state are float (in bf16 mode the matrix products take
 // them as two bf16 parts, see tile.h).
+//
+// Linear attention with the same recurrence is served as well: silu of q, k
+// and v as they are read (v is rounded to the model's type after it), and raw
+// outputs for a norm over all heads.
 
 #include "chunk.h"
 
 namespace {
+
+DEVINL float silu(float z) { return z / (1.0f + expf(-z)); }
 
 // Rotated q or k elements c..c+7 of one head, times `mul`.  Element i of
 // the first half of the rotated span pairs with i + rd/2.
@@ -53,6 +59,10 @@ DEVINL void load_rot8(const typename Num<F32>::E* head, int c, const RetArgs& a,
         }
       }
     }
+  }
+  if (a.silu) {
+    #pragma unroll
+    for (int j = 0; j < 8; ++j) out[j] = silu(out[j]);
   }
   #pragma unroll
   for (int j = 0; j < 8; ++j) out[j] *= mul;
@@ -101,7 +111,7 @@ DEVINL void stage_rot(const typename Num<F32>::E* head0, const RetArgs& a,
           const float w = low ? -y : y;
           r = in ? x * cv[it][i] + w * sv[it][i] : x;
         }
-        v[i] = r * f;
+        v[i] = (a.silu ? silu(r) : r) * f;
       }
       put(j, c, v);
     }
@@ -114,6 +124,21 @@ DEVINL void stage_rot(const typename Num<F32>::E* head0, const RetArgs& a,
       put(j, c, v);
     }
   }
+}
+
+// value rows of a tile
+template <bool F32, int DV>
+DEVINL void ret_values(const ColTile<F32, DV>& V, const typename Num<F32>::E* v0,
+                       const RetArgs& a, int rows, bool aligned) {
+  RowStage<F32, DV> r;
+  r.load(v0, a.ld, rows, a.dv, aligned);
+  if (!a.silu) return r.put(V, rows, a.dv);
+  r.visit(rows, a.dv, [&](int j, int c, const Raw8<F32>& x) {
+    float v[8];
+    #pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = silu(x[i]);
+    V.put8(j, c, v);
+  });
 }
 
 DEVINL bool ret_aligned(const RetArgs& a) {
@@ -147,8 +172,8 @@ ret_chunk_state_kernel(RetArgs a, const int4* __restrict__ tiles,
           Kl.put8(j, c, v);
         }
       });
-  stage_v<F32, DV>(V, base + (long)2 * a.H * a.dk + (long)h * a.dv, a.ld,
-                   t.y, a.dv, aligned);
+  ret_values<F32, DV>(V, base + (long)2 * a.H * a.dk + (long)h * a.dv, a, t.y,
+                      aligned);
   __syncthreads();
 
   tile_outer<F32, DK, DV>(V, Kh, Kl, a.dv, a.dk,
@@ -210,8 +235,8 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
                        [&](int j, int c, float* v) { X.put8(j * LDK + c, v); });
   };
   stage_qk((long)h * a.dk, 1.f);
-  stage_v<F32, DV>(V, base + (long)2 * a.H * a.dk + (long)h * a.dv, a.ld,
-                   t.y, a.dv, aligned);
+  ret_values<F32, DV>(V, base + (long)2 * a.H * a.dk + (long)h * a.dv, a, t.y,
+                      aligned);
   __syncthreads();
   typename Split<F32>::Frag qf[DK / 32];
   #pragma unroll
@@ -245,13 +270,15 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
       });
   // gates: all in flight here, used in the epilogue
   E gz[4][DV / 16];
-  #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const E* gate = base + (long)min(16 * w + 4 * lg + r, t.y - 1) * a.ld +
-                    (long)2 * a.H * a.dk + (long)(a.H + h) * a.dv;
+  if (!a.raw) {
     #pragma unroll
-    for (int i = 0; i < DV / 16; ++i)
-      gz[r][i] = gate[min(i * 16 + lr, a.dv - 1)];
+    for (int r = 0; r < 4; ++r) {
+      const E* gate = base + (long)min(16 * w + 4 * lg + r, t.y - 1) * a.ld +
+                      (long)2 * a.H * a.dk + (long)(a.H + h) * a.dv;
+      #pragma unroll
+      for (int i = 0; i < DV / 16; ++i)
+        gz[r][i] = gate[min(i * 16 + lr, a.dv - 1)];
+    }
   }
   float ss[4] = {0.f, 0.f, 0.f, 0.f};
   #pragma unroll
@@ -271,6 +298,18 @@ ret_chunk_out_kernel(RetArgs a, const int4* __restrict__ tiles,
       #pragma unroll
       for (int x = 0; x < 4; ++x) o[i + x] = mma_sp<F32>(pf, vf[x], o[i + x]);
     }
+  }
+  if (a.raw) {
+    #pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = 16 * w + 4 * lg + r;
+      if (row >= t.y) continue;
+      E* dst = (E*)a.out + ((long)(t.x + row) * a.H + h) * a.dv;
+      #pragma unroll
+      for (int i = 0; i < DV / 16; ++i)
+        if (i * 16 + lr < a.dv) dst[i * 16 + lr] = N::down(o[i][r]);
+    }
+    return;
   }
   #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -327,10 +366,15 @@ ret_decode_kernel(RetArgs a, const int* __restrict__ pos,
       const float cv = a.cos_t[(long)p * half + i], sv = a.sin_t[(long)p * half + i];
       x = low ? x * cv - y * sv : x * cv + y * sv;
     }
+    if (a.silu) x = silu(x);
     (isk ? k_s : q_s)[c] = isk ? x * a.kscale : x;
   }
   __syncthreads();
 
+  auto value = [&](int r) {
+    const float v = N::up(vrow[r]);
+    return a.silu ? N::up(N::down(silu(v))) : v;
+  };
   const float dh = a.dec[2 * h], dl = a.dec[2 * h + 1];
   float* S = a.state + ((long)s * a.H + h) * a.dv * a.dk;
   const bool fresh = p == 0;
@@ -359,7 +403,7 @@ ret_decode_kernel(RetArgs a, const int* __restrict__ pos,
         const int r = r0 + u * rstep;
         float d = 0.f;
         if (in && r < a.dv) {
-          const float v = N::up(vrow[r]);
+          const float v = value(r);
           #pragma unroll
           for (int j = 0; j < 4; ++j) {
             x[u][j] = fmaf(x[u][j], dh, fmaf(x[u][j], dl, kv[j] * v));
@@ -374,7 +418,7 @@ ret_decode_kernel(RetArgs a, const int* __restrict__ pos,
   } else {
     const int w = tid >> 6, l = tid & 63;
     for (int r = w; r < a.dv; r += NT / 64) {
-      const float v = N::up(vrow[r]);
+      const float v = value(r);
       float d = 0.f;
       for (int c = l; c < a.dk; c += 64) {
         float* e = S + (long)r * a.dk + c;
@@ -388,6 +432,10 @@ ret_decode_kernel(RetArgs a, const int* __restrict__ pos,
     }
   }
   __syncthreads();
+  if (a.raw) {
+    for (int c = tid; c < a.dv; c += NT) dst[c] = N::down(o_s[c]);
+    return;
+  }
   float qd = 0.f;
   for (int c = tid; c < a.dv; c += NT) qd += o_s[c] * o_s[c];
   qd = wave_reduce_sum(qd);

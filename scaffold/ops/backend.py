@@ -49,10 +49,12 @@ _SOURCES = [
 _LM_SOURCES = [
     "lm/ext.cpp",
     "lm/norm.hip",
+    "lm/stream.hip",
     "lm/attn.hip",
     "lm/attn_mfma.hip",
     "lm/attn_decode.hip",
     "lm/retention.hip",
+    "lm/gla.hip",
     "lm/mamba2.hip",
     "lm/mlstm.hip",
     "lm/latent.hip",

@@ -459,7 +459,7 @@ def retention(qkvg, cache, run, plan, *, pows, dec, rope, kscale, eps):
         cos, sin = rope if rope is not None else (None, None)
         return require_lm_ext().retention(
             qkvg, st, plan.pos, plan.slot, plan.tiles, plan.seqs, plan.n_dec,
-            pows, dec, cos, sin, kscale, eps)
+            pows, dec, cos, sin, kscale, eps, False)
     H, dv, dk = st.shape[1:]
     q, k, v, g = (t.reshape(qkvg.shape[0], H, -1).float() for t in
                   torch.split(qkvg, [H * dk, H * dk, H * dv, H * dv], dim=1))
