@@ -124,13 +124,13 @@ def main() -> int:
     ap.add_argument("--warmup", type=int, default=20)
     ap.add_argument("--model", type=str, default="resnet50",
                     choices=["resnet50", "gpt2", "llama3_8b", "mlp",
-                             "lasezen", "nekozen", "babodra"],
-                    help="lasezen, nekozen, babodra: serving throughput "
-                         "(prefill, decode) beside llama or lasezen at equal "
-                         "size, one JSON line each")
+                             "lasezen", "nekozen", "babodra", "tilivik"],
+                    help="lasezen, nekozen, babodra, tilivik: serving "
+                         "throughput (prefill, decode) beside the closest "
+                         "models at equal size, one JSON line each")
     ap.add_argument("--sizes", type=str, default="",
-                    help="lasezen, nekozen, babodra: comma-separated sizes (default "
-                         "all)")
+                    help="lasezen, nekozen, babodra, tilivik: comma-separated "
+                         "sizes (default all)")
     ap.add_argument("--batch-size", type=int, default=0, help="per-rank; 0=config default")
     ap.add_argument("--bucket-mb", type=float, default=0.0, help="bucket override")
     ap.add_argument("--sweep-buckets", type=str, default="",
@@ -139,7 +139,7 @@ def main() -> int:
     ap.add_argument("overrides", nargs="*", help="section.key=value overrides")
     args = ap.parse_args()
 
-    if args.model in ("lasezen", "nekozen", "babodra"):
+    if args.model in ("lasezen", "nekozen", "babodra", "tilivik"):
         from benchmarks import stack_bench
 
         stack_bench.run(args.steps, args.warmup,

@@ -3,9 +3,10 @@ model it is closest to (random weights): Lasezen beside Llama at equal
 width, heads, feed-forward width and depth; Nekozen beside Lasezen at
 equal width, heads and depth, its feed-forwards two thirds as wide because
 they have three matrices; Babodra beside Lasezen at equal width, heads and
-depth, with as many feed-forward weights active per token.
+depth, with as many feed-forward weights active per token; Tilivik beside
+Babodra at equal width, heads, depth, experts and active feed-forward weights.
 
-Run through bench.py: `python bench.py --model lasezen|nekozen|babodra
+Run through bench.py: `python bench.py --model lasezen|nekozen|babodra|tilivik
 [--steps K] [--warmup W]`.  One JSON line per size and phase; decode steps are
 hipGraph replays of the serving step for all models.
 """
@@ -32,7 +33,8 @@ SIZES = {
 MAX_LEN = 8192 + 512
 # what a benchmark of a design measures
 BESIDE = {"lasezen": ("lasezen", "llama"), "nekozen": ("nekozen", "lasezen"),
-          "babodra": ("babodra", "lasezen")}
+          "babodra": ("babodra", "lasezen"),
+          "tilivik": ("tilivik", "lasezen", "babodra")}
 
 
 def lasezen_config(s: dict) -> TrainConfig:
@@ -107,6 +109,36 @@ def babodra_config(s: dict) -> TrainConfig:
     return cfg
 
 
+def tilivik_config(s: dict) -> TrainConfig:
+    """Every fourth layer lightning, the others window attention beside gated
+    linear attention with a quarter of its heads; in every layer 32 experts of
+    which a token id takes 5, as wide as Babodra's.  The second half of the
+    stack is the loop's span, run once."""
+    H, n = s["heads"], s["layers"]
+    moe = {"kind": "table_moe", "router": {"experts": 32, "top": 5},
+           "expert": {"ff": s["ff"] * 2 // 15 // 64 * 64}}
+    light = {"type": "lightning", "mlp": moe, "mixer": {
+        "heads": H, "dim": s["dim"], "vdim": s["dim"],
+        "decay": [1 - 2.0 ** (-5 - 3 * h / H) for h in range(H)]}}
+    both = {"type": "parallel", "mlp": moe, "mixer": {
+        "left": {"type": "window_attention", "heads": H, "kv_heads": s["kv"],
+                 "dim": s["dim"], "vdim": s["dim"], "buckets": 32,
+                 "bias_max": 128, "scale": s["dim"] ** -0.5, "softcap": 50.0,
+                 "mask": {"size": s["chunk"], "keep_first": 4}},
+        "right": {"type": "gla", "heads": H // 4, "dim": s["dim"],
+                  "vdim": s["dim"], "rank": 16, "tau": 16.0},
+        "left_scale": 0.7, "right_scale": 1.0}}
+    cfg = load_config(None, ["model.name=tilivik",
+                             f"model.vocab_size={s['vocab']}",
+                             f"model.d_model={s['width']}",
+                             f"model.max_seq_len={MAX_LEN}"])
+    cfg.model.bigram = {"buckets": s["vocab"], "mul_prev": 8191,
+                        "mul_cur": 127}
+    cfg.model.layers = [both if i % 4 else light for i in range(n)]
+    cfg.model.loop = {"start": n // 2, "stop": n, "times": 1}
+    return cfg
+
+
 def llama_config(s: dict) -> TrainConfig:
     return load_config(None, [
         "model.name=llama", f"model.vocab_size={s['vocab']}",
@@ -118,7 +150,8 @@ def llama_config(s: dict) -> TrainConfig:
 def build(name: str, s: dict, dtype=torch.bfloat16):
     torch.manual_seed(0)
     cfg = {"lasezen": lasezen_config, "nekozen": nekozen_config,
-           "babodra": babodra_config, "llama": llama_config}[name](s)
+           "babodra": babodra_config, "tilivik": tilivik_config,
+           "llama": llama_config}[name](s)
     with torch.device("cuda"):       # random init on the GPU
         model = build_model(cfg)
     # llama builds its rotary tables on the host: move what is left
