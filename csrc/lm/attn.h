@@ -35,20 +35,34 @@ struct PageList {
   DEVINL int operator[](int i) const { return i < kept ? i : first + i - kept; }
 };
 
-// A score times `scale` through the soft cap and to base 2, bias aside:
-// c tanh(x / c) = c - 2 c / (exp(2 x / c) + 1).
+// A score times `scale` through the soft cap c tanh(x / c), in base 2, plus an
+// addend.  Where every score of a wave is below 0.4 c (small(max |score|)) a
+// polynomial in the square serves, four multiply-adds, relative error 1e-7
+// (fitted to tanh(y) / y on [0, 0.4]); else c - 2 c / (exp(2 x / c) + 1).
 struct SoftCap {
-  float in, out, c2;     // exponent's factor, factors of the result
-  bool on;
-  DEVINL explicit SoftCap(const AttnArgs& a, float log2e) {
-    on = a.softcap > 0.f;
-    in = on ? 2.f * log2e * a.scale / a.softcap : 0.f;
-    out = on ? a.softcap * log2e : a.scale * log2e;
+  float in, out, c2, limit;       // limit: of the polynomial, for a raw score
+  float p0, p1, p2, p3;
+  DEVINL SoftCap(const AttnArgs& a, float log2e) {
+    const bool on = a.softcap > 0.f;
+    const float r = on ? a.scale / a.softcap : 0.f, r2 = r * r;
+    in = 2.f * log2e * r;
+    out = a.softcap * log2e;
     c2 = -2.f * out;
+    limit = on ? 0.4f / fabsf(r) : INFINITY;
+    const float f = a.scale * log2e;          // no cap: this alone
+    p0 = on ? f * 0.999999904f : f;
+    p1 = -0.333313902f * f * r2;
+    p2 = 0.132714383f * f * r2 * r2;
+    p3 = -0.0475728106f * f * r2 * r2 * r2;
   }
-  DEVINL float operator()(float s) const {
-    if (!on) return s * out;
-    return fmaf(c2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * in) + 1.f), out);
+  DEVINL bool small(float most) const { return !__any(most > limit); }
+  DEVINL float near(float s, float b) const {
+    const float t = s * s;
+    return fmaf(s, fmaf(t, fmaf(t, fmaf(t, p3, p2), p1), p0), b);
+  }
+  DEVINL float any(float s, float b) const {
+    const float e = __builtin_amdgcn_exp2f(s * in);
+    return fmaf(c2, __builtin_amdgcn_rcpf(e + 1.f), out + b);
   }
 };
 

@@ -191,14 +191,29 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
     }
   }
   const SoftCap cap(a, LOG2E);
-  // a score in base 2 of head i at distance dj
-  auto windowed = [&](int i, float x, float dj) {
-    const int d = min((int)dj, a.n_bias - 1);
-    const float b = (bias_lds ? bias_s[i][d] : bias_g[i][d]) * LOG2E;
-    if constexpr (!F32) return cap(x) + b;
-    x *= a.scale;
-    if (a.softcap > 0.f) x = a.softcap * tanhf(x / a.softcap);
-    return fmaf(x, LOG2E, b);
+  // scores of head i in base 2, at distances dj
+  auto windowed = [&](int i, float (&x)[KB], const float (&dj)[KB]) {
+    float b[KB], most = 0.f;
+    #pragma unroll
+    for (int u = 0; u < KB; ++u) {
+      const int d = min((int)dj[u], a.n_bias - 1);
+      b[u] = (bias_lds ? bias_s[i][d] : bias_g[i][d]) * LOG2E;
+      most = fmaxf(most, fabsf(x[u]));
+    }
+    if constexpr (F32) {
+      #pragma unroll
+      for (int u = 0; u < KB; ++u) {
+        float y = x[u] * a.scale;
+        if (a.softcap > 0.f) y = a.softcap * tanhf(y / a.softcap);
+        x[u] = fmaf(y, LOG2E, b[u]);
+      }
+    } else if (cap.small(most)) {
+      #pragma unroll
+      for (int u = 0; u < KB; ++u) x[u] = cap.near(x[u], b[u]);
+    } else {
+      #pragma unroll
+      for (int u = 0; u < KB; ++u) x[u] = cap.any(x[u], b[u]);
+    }
   };
 
   // kf: scale of a key's scores, dj: its distance
@@ -212,10 +227,13 @@ attn_decode_kernel(AttnArgs a, const int* __restrict__ pos,
         float d = 0.f;
         #pragma unroll
         for (int j = 0; j < 8; ++j) d = fmaf(q[i][j], k[u][j], d);
-        d = group_sum<LPK>(d);
-        if constexpr (WIN) d = windowed(i, d, dj[u]);
-        else d = d * kf[u] - slope2[i] * dj[u];
-        sc[u] = ok[u] ? d : NEG;
+        sc[u] = group_sum<LPK>(d);
+      }
+      if constexpr (WIN) windowed(i, sc, dj);
+      #pragma unroll
+      for (int u = 0; u < KB; ++u) {
+        if constexpr (!WIN) sc[u] = sc[u] * kf[u] - slope2[i] * dj[u];
+        sc[u] = ok[u] ? sc[u] : NEG;
         mx = fmaxf(mx, sc[u]);
       }
       const float al = exp2f(m[i] - mx);

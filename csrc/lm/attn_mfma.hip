@@ -223,23 +223,39 @@ attn_prefill_mfma_kernel(AttnArgs a, const int4* __restrict__ tiles,
       const float d0 = slope2 * (float)(j0 + 4 * half - ip);
       if constexpr (WIN) {
         const int last = n_bias - 1, dist = ip - j0 - 4 * half;
+        const bool far = w0 - j0 - (LM_PAGE - 1) >= last;     // of all rows
+        float most = 0.f;
         #pragma unroll
         for (int sub = 0; sub < 2; ++sub)
           #pragma unroll
-          for (int r = 0; r < 16; ++r) s[sub][r] = cap(s[sub][r]);
-        if (w0 - j0 - (LM_PAGE - 1) >= last) {         // uniform in the wave
-          #pragma unroll
-          for (int sub = 0; sub < 2; ++sub)
-            #pragma unroll
-            for (int r = 0; r < 16; ++r) s[sub][r] += bias_far;
-        } else {
+          for (int r = 0; r < 16; ++r) most = fmaxf(most, fabsf(s[sub][r]));
+        const bool small = cap.small(most);
+        // both are uniform in the wave
+        auto scores = [&](auto bias) {
           #pragma unroll
           for (int sub = 0; sub < 2; ++sub)
             #pragma unroll
             for (int r = 0; r < 16; ++r) {
-              const int d = min(max(dist - (sub * 32 + (r & 3) + 8 * (r >> 2)), 0), last);
-              s[sub][r] += bias_lds ? bias_h[d] : bias_g[d] * LOG2E;
+              const float b = bias(sub * 32 + (r & 3) + 8 * (r >> 2));
+              s[sub][r] = small ? cap.near(s[sub][r], b) : cap.any(s[sub][r], b);
             }
+        };
+        if (far) {
+          if (small) {
+            #pragma unroll
+            for (int sub = 0; sub < 2; ++sub)
+              #pragma unroll
+              for (int r = 0; r < 16; ++r) s[sub][r] = cap.near(s[sub][r], bias_far);
+          } else {
+            #pragma unroll
+            for (int sub = 0; sub < 2; ++sub)
+              #pragma unroll
+              for (int r = 0; r < 16; ++r) s[sub][r] = cap.any(s[sub][r], bias_far);
+          }
+        } else if (bias_lds) {
+          scores([&](int j) { return bias_h[min(max(dist - j, 0), last)]; });
+        } else {
+          scores([&](int j) { return bias_g[min(max(dist - j, 0), last)] * LOG2E; });
         }
       }
       #pragma unroll

@@ -30,55 +30,86 @@ namespace {
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr float LIMIT = 60.f;
 
+DEVINL float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
 DEVINL float silu(float z) { return z / (1.0f + expf(-z)); }
 
-// log2 of a channel's decay
+// log2 of a channel's decay.  log(1 + t) as log(u) t / (u - 1), u the rounded
+// 1 + t: the rounding of u cancels (Higham, "Accuracy and Stability of
+// Numerical Algorithms").
+template <bool F32>
 DEVINL float log_decay(const GlaArgs& a, float z) {
-  return -(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)))) * (LOG2E * a.inv_tau);
+  if constexpr (F32)
+    return -(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)))) * (LOG2E * a.inv_tau);
+  const float t = pow2(-fabsf(z) * LOG2E), u = 1.f + t;
+  const float l = u == 1.f ? t * LOG2E
+                           : __builtin_amdgcn_logf(u) * t * __builtin_amdgcn_rcpf(u - 1.f);
+  return -fmaf(fmaxf(-z, 0.f), LOG2E, l) * a.inv_tau;
 }
 
 // Log decays of a tile: F [64][DK] from the start of a token's sub-tile up to
-// it, tot [4][DK] those of whole sub-tiles.  Wave w has sub-tile w.
+// it, tot [4][DK] those of whole sub-tiles.  Wave w has sub-tile w, eight
+// 16-channel tiles at a time; the first 32 columns of the sum over the rank
+// (all of them, as a rule) have their loads in flight together.
 template <bool F32, int DK>
 DEVINL void tile_decays(const GlaArgs& a, int row0, int rows, int h, float* F,
                         float* tot) {
   using N = Num<F32>;
   using E = typename N::E;
+  constexpr int CT = DK / 16 < 8 ? DK / 16 : 8;
   const int w = threadIdx.x >> 6, l = threadIdx.x & 63;
   const int lr = l & 15, lg = l >> 4;
   const bool al = a.rank % 8 == 0, u_al = al && a.dk % 8 == 0 && a.dv % 8 == 0;
   const E* u = (const E*)a.u + (long)(row0 + min(16 * w + lr, rows - 1)) * a.ld;
-  for (int ct = 0; ct * 16 < a.dk; ++ct) {
-    const int c = min(ct * 16 + lr, a.dk - 1);
-    const E* m = (const E*)a.a2 + ((long)h * a.dk + c) * a.rank;
-    f32x4 z = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k0 = 0; k0 < a.rank; k0 += 32) {
-      const int k = k0 + 8 * lg;
-      Raw8<F32> x, y;
-      x.load(u + k, a.rank - k, u_al);
-      y.load(m + k, a.rank - k, al);
-      z = N::mma(N::load(x.e, 0), N::load(y.e, 0), z);
-    }
-    const float b = N::up(((const E*)a.a2b)[(long)h * a.dk + c]);
-    float f[4], s = 0.f;
+  const E* m0 = (const E*)a.a2 + (long)h * a.dk * a.rank;
+  Raw8<F32> x;
+  x.load(u + 8 * lg, a.rank - 8 * lg, u_al);
+  for (int c0 = 0; c0 < a.dk; c0 += 16 * CT) {
+    Raw8<F32> y[CT];
+    E b[CT];
     #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      s += 16 * w + 4 * lg + r < rows ? log_decay(a, z[r] + b) : 0.f;
-      f[r] = s;
+    for (int i = 0; i < CT; ++i) {
+      const int c = min(c0 + i * 16 + lr, a.dk - 1);
+      y[i].load(m0 + (long)c * a.rank + 8 * lg, a.rank - 8 * lg, al);
+      b[i] = ((const E*)a.a2b)[(long)h * a.dk + c];
     }
-    // tokens 4 lg .. of the sub-tile: add what the lane groups before have
-    float before = 0.f;
+    f32x4 z[CT];
     #pragma unroll
-    for (int g = 0; g < 3; ++g) {
-      const float o = __shfl(s, g * 16 + lr, 64);
-      before += g < lg ? o : 0.f;
+    for (int i = 0; i < CT; ++i)
+      z[i] = N::mma(N::load(x.e, 0), N::load(y[i].e, 0), f32x4{0.f, 0.f, 0.f, 0.f});
+    for (int k = 32 + 8 * lg; k - 8 * lg < a.rank; k += 32) {
+      Raw8<F32> v;
+      v.load(u + k, a.rank - k, u_al);
+      #pragma unroll
+      for (int i = 0; i < CT; ++i) {
+        y[i].load(m0 + (long)min(c0 + i * 16 + lr, a.dk - 1) * a.rank + k,
+                  a.rank - k, al);
+        z[i] = N::mma(N::load(v.e, 0), N::load(y[i].e, 0), z[i]);
+      }
     }
     #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      f[r] += before;
-      F[(16 * w + 4 * lg + r) * DK + ct * 16 + lr] = f[r];
+    for (int i = 0; i < CT; ++i) {
+      if (c0 + i * 16 >= a.dk) continue;      // uniform
+      float f[4], s = 0.f;
+      #pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float d = log_decay<F32>(a, z[i][r] + N::up(b[i]));
+        s += 16 * w + 4 * lg + r < rows ? d : 0.f;
+        f[r] = s;
+      }
+      // tokens 4 lg .. of the sub-tile: add what the lane groups before have
+      float before = 0.f;
+      #pragma unroll
+      for (int g = 0; g < 3; ++g) {
+        const float o = __shfl(s, g * 16 + lr, 64);
+        before += g < lg ? o : 0.f;
+      }
+      #pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        f[r] += before;
+        F[(16 * w + 4 * lg + r) * DK + c0 + i * 16 + lr] = f[r];
+      }
+      if (lg == 3) tot[w * DK + c0 + i * 16 + lr] = f[3];
     }
-    if (lg == 3) tot[w * DK + ct * 16 + lr] = f[3];
   }
 }
 
@@ -92,10 +123,9 @@ gla_chunk_state_kernel(GlaArgs a, const int4* __restrict__ tiles,
   using E = typename Num<F32>::E;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   __shared__ float tot[4 * DK], tail[4 * DK];
+  float* F = (float*)smem;                    // first F, then the operands
   const ColTile<F32, DK> Kh{(E*)smem}, Kl{Kh.p + Kh.SIZE};
-  E* rest = Kh.p + (F32 ? 1 : 2) * Kh.SIZE;   // first F, then the values
-  float* F = (float*)rest;
-  const ColTile<F32, DV> V{rest};
+  const ColTile<F32, DV> V{Kh.p + (F32 ? 1 : 2) * Kh.SIZE};
 
   const int4 t = tiles[blockIdx.y];
   const int h = blockIdx.x;
@@ -116,26 +146,32 @@ gla_chunk_state_kernel(GlaArgs a, const int4* __restrict__ tiles,
       tail[i * DK + c] = s;
       s += tot[i * DK + c];
     }
-    cd[cell * a.dk + c] = __builtin_amdgcn_exp2f(s);
+    cd[cell * a.dk + c] = pow2(s);
   }
   __syncthreads();
+  float wk[RowStage<F32, DK>::N][8];          // weighted keys
+  int n = 0;
   ks.visit(t.y, a.dk, [&](int j, int c, const Raw8<F32>& x) {
-    float v[8];
     const float* f = F + j * DK + c;
     const int sub = (j >> 4) * DK + c;
     #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      const bool on = c + i < a.dk;
-      v[i] = on ? x[i] * exp2f((tot[sub + i] - f[i]) + tail[sub + i]) : 0.f;
+      const float d = pow2((tot[sub + i] - f[i]) + tail[sub + i]);
+      wk[n][i] = c + i < a.dk ? x[i] * d : 0.f;
     }
-    Kh.put8(j, c, v);
-    if constexpr (!F32) {
-      #pragma unroll
-      for (int i = 0; i < 8; ++i) v[i] -= bf2f(cvt_bf16(v[i]));
-      Kl.put8(j, c, v);
-    }
+    ++n;
   });
   __syncthreads();                            // F is done with
+  n = 0;
+  ks.visit(t.y, a.dk, [&](int j, int c, const Raw8<F32>&) {
+    Kh.put8(j, c, wk[n]);
+    if constexpr (!F32) {
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) wk[n][i] -= bf2f(cvt_bf16(wk[n][i]));
+      Kl.put8(j, c, wk[n]);
+    }
+    ++n;
+  });
   vs.put(V, t.y, a.dv);
   __syncthreads();
   tile_outer<F32, DK, DV>(V, Kh, Kl, a.dv, a.dk, cs + cell * a.dv * a.dk);
@@ -220,7 +256,7 @@ gla_chunk_out_kernel(GlaArgs a, const int4* __restrict__ tiles,
     const int sub = (j >> 4) * DK + c;
     #pragma unroll
     for (int i = 0; i < 8; ++i)
-      v[i] = c + i < a.dk ? x[i] * exp2f(tot[sub + i] - f[i]) : 0.f;
+      v[i] = c + i < a.dk ? x[i] * pow2(tot[sub + i] - f[i]) : 0.f;
     X.put8(j * LDK + c, v);
   });
 
@@ -253,8 +289,8 @@ gla_chunk_out_kernel(GlaArgs a, const int4* __restrict__ tiles,
       const float d = on ? tot[w * DK + c + i] : 0.f;
       const float q = on ? qr[kb][i] * a.qscale : 0.f;
       steep |= d < -LIMIT;
-      qd[kb][i] = q * exp2f(f);
-      qi[i] = q * exp2f(fminf(f - d, LIMIT));
+      qd[kb][i] = q * pow2(f);
+      qi[i] = q * pow2(fminf(f - d, LIMIT));
     }
     qs[kb] = frag(kb, qi);
   }
@@ -287,7 +323,7 @@ gla_chunk_out_kernel(GlaArgs a, const int4* __restrict__ tiles,
       if (lr <= 4 * lg + r)
         for (int c = 0; c < a.dk; ++c)
           s = fmaf(N::up(qi[c]) * a.qscale * N::up(kj[c]),
-                   exp2f(F[i * DK + c] - Fj[c]), s);
+                   pow2(F[i * DK + c] - Fj[c]), s);
       own[r] = s;
     }
   }
@@ -302,7 +338,7 @@ gla_chunk_out_kernel(GlaArgs a, const int4* __restrict__ tiles,
         qs[kb] = frag(kb, qd[kb]);
         #pragma unroll
         for (int i = 0; i < 8; ++i)
-          qd[kb][i] *= c + i < a.dk ? exp2f(tot[b * DK + c + i]) : 0.f;
+          qd[kb][i] *= c + i < a.dk ? pow2(tot[b * DK + c + i]) : 0.f;
       }
     }
     if (b < w) sc[b] = against(b);
@@ -402,7 +438,8 @@ gla_decode_kernel(GlaArgs a, const int* __restrict__ pos,
     }
     z = group_sum<4>(z);
     if (c < a.dk && (tid & 3) == 0)
-      d_s[c] = exp2f(log_decay(a, z + N::up(((const E*)a.a2b)[(long)h * a.dk + c])));
+      d_s[c] = pow2(log_decay<F32>(
+          a, z + N::up(((const E*)a.a2b)[(long)h * a.dk + c])));
   }
   for (int c = tid; c < a.dk; c += NT) {
     q_s[c] = N::up(((const E*)a.q)[at + (long)h * a.dk + c]) * a.qscale;
@@ -488,8 +525,8 @@ void launch_prefill(const GlaArgs& a, const int4* tiles, int n_tiles,
   constexpr size_t es = sizeof(typename N::E);
   constexpr int LDJ = LM_TILE + N::PAD;
   constexpr size_t f = sizeof(float) * LM_TILE * DK;
-  constexpr size_t lds1 = es * S::PARTS * ColTile<F32, DK>::SIZE +
-                          std::max(f, es * V::SIZE);
+  constexpr size_t lds1 =
+      std::max(f, es * (S::PARTS * ColTile<F32, DK>::SIZE + V::SIZE));
   constexpr size_t lds2 =
       es * S::PARTS * LM_TILE * (DK + N::PAD) +
       std::max(f, es * (S::PARTS * LM_TILE * LDJ + V::SIZE));

@@ -142,9 +142,22 @@ moe_route_kernel(MoeArgs a) {
   if (t < a.T) route_token<NPL>(a, t, sc[w], threadIdx.x & 63);
 }
 
-// One block sorts the entries; ROUTE: and routes the tokens before that.  With
-// a table nothing is routed: a token's experts are read there and have equal
-// weights.
+// With a table nothing is routed: entry i's expert is read there, and all of
+// a token's have equal weights.
+DEVINL void look_up(const MoeArgs& a, int i) {
+  const long tok = min(max(a.tokens[i / a.top], 0l), a.vocab - 1);
+  a.ids[i] = min(max(a.table[tok * a.top + i % a.top], 0), a.E - 1);
+  a.wts[i] = 1.0f / (float)a.top;
+}
+
+__global__ void __launch_bounds__(256)
+moe_table_kernel(MoeArgs a) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i < a.T * a.top) look_up(a, i);
+}
+
+// One block sorts the entries; ROUTE: and routes the tokens (or looks them up)
+// before that.
 template <int NPL, bool ROUTE>
 __global__ void __launch_bounds__(1024)
 moe_plan_kernel(MoeArgs a) {
@@ -152,15 +165,13 @@ moe_plan_kernel(MoeArgs a) {
   __shared__ float sc[ROUTE ? 16 : 1][NPL * 64];
   const int tid = threadIdx.x, w = tid >> 6, l = tid & 63;
   for (int e = tid; e < NPL * 64; e += 1024) cnt[e] = 0;
-  if constexpr (ROUTE)
-    for (int t = w; t < a.T; t += 16) route_token<NPL>(a, t, sc[w], l);
   const int n = a.T * a.top;
-  if (a.table)
-    for (int i = tid; i < n; i += 1024) {
-      const long tok = min(max(a.tokens[i / a.top], 0l), a.vocab - 1);
-      a.ids[i] = min(max(a.table[tok * a.top + i % a.top], 0), a.E - 1);
-      a.wts[i] = 1.0f / (float)a.top;
-    }
+  if constexpr (ROUTE) {
+    if (a.table)
+      for (int i = tid; i < n; i += 1024) look_up(a, i);
+    else
+      for (int t = w; t < a.T; t += 16) route_token<NPL>(a, t, sc[w], l);
+  }
   __threadfence_block();
   __syncthreads();
   for (int i = tid; i < n; i += 1024) atomicAdd(&cnt[a.ids[i]], 1);
@@ -507,12 +518,14 @@ Kind pick(const MoeArgs& a, bool f32) {
 
 template <int NPL>
 void plan(const MoeArgs& a, hipStream_t st) {
-  if (a.table) {
-    hipLaunchKernelGGL((moe_plan_kernel<NPL, false>), dim3(1), dim3(1024), 0, st, a);
-  } else if (a.T <= 32) {
+  if (a.T <= 32 || (a.table && a.T * a.top <= 1024)) {
     hipLaunchKernelGGL((moe_plan_kernel<NPL, true>), dim3(1), dim3(1024), 0, st, a);
   } else {
-    hipLaunchKernelGGL((moe_route_kernel<NPL>), dim3((a.T + 3) / 4), dim3(256), 0, st, a);
+    if (a.table)
+      hipLaunchKernelGGL(moe_table_kernel, dim3((a.T * a.top + 255) / 256),
+                         dim3(256), 0, st, a);
+    else
+      hipLaunchKernelGGL((moe_route_kernel<NPL>), dim3((a.T + 3) / 4), dim3(256), 0, st, a);
     hipLaunchKernelGGL((moe_plan_kernel<NPL, false>), dim3(1), dim3(1024), 0, st, a);
   }
 }

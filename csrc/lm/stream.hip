@@ -89,7 +89,9 @@ __global__ void __launch_bounds__(256)
 shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
   __shared__ float red[4];
   const int tid = threadIdx.x % TPR, W = a.W;
-  const int task = blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
+  // with a block per row everything that depends on the row alone is uniform
+  const int task = TPR == 256 ? blockIdx.x
+                              : blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
   int row0, rows;
   if (task < r.n_dec) {
     row0 = task;
@@ -113,7 +115,7 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
 
   // a row's new stream and its norm
   auto make = [&](long row, bool store, Pack<VEC> (&h)[NV]) {
-    constexpr int CH = NV <= 4 ? 4 : 2;
+    constexpr int CH = NV <= 4 ? 6 : 2;       // parts with loads in flight
     Held<F32, VEC> t[CH][NV];
     const int n = a.y.y ? (a.y.w ? a.y.n : 1) : 0;
     float wt[CH];
@@ -122,7 +124,8 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
       for (int k = 0; k < CH; ++k) {
         const bool on = k0 + k < n;
         const long part = row * n + (on ? k0 + k : 0);
-        wt[k] = on ? (a.y.w ? a.y.w[part] : 1.f) * a.mult : 0.f;
+        wt[k] = a.y.w ? a.y.w[part] : 1.f;
+        wt[k] = on ? wt[k] * a.mult : 0.f;
         #pragma unroll
         for (int i = 0; i < NV; ++i) {
           const int c = (i * TPR + tid) * VEC;
@@ -131,7 +134,7 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
         }
       }
     };
-    fetch(0);
+    if (n > 0) fetch(0);
     #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int c = (i * TPR + tid) * VEC;
