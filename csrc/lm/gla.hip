@@ -117,7 +117,7 @@ DEVINL bool gla_aligned(const GlaArgs& a) { return a.dk % 8 == 0 && a.dv % 8 == 
 
 // contribution of one tile and head to the state, and its channels' decays
 template <bool F32, int DK, int DV>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, !F32 && DK <= 128 && DV <= 128 ? 3 : 1)
 gla_chunk_state_kernel(GlaArgs a, const int4* __restrict__ tiles,
                        float* __restrict__ cs, float* __restrict__ cd) {
   using E = typename Num<F32>::E;

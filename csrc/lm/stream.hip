@@ -4,10 +4,11 @@
 //    neighbouring tokens.  Angles are turns in double, reduced before they
 //    become float, so a position's vector does not lose digits with distance.
 //  shift: x' = x + mult * y + add + step, h = norm(x'), and the output
-//    h + (h_before - h) * shift.  A thread group walks some consecutive rows
-//    and carries the last h in registers; its first row's predecessor it
-//    computes once more.  The new stream goes to another buffer, so that this
-//    never meets a row that its own group has already replaced.
+//    h + (h_before - h) * shift.  In prompts a thread group walks some
+//    consecutive rows and carries the last h in registers; its first row's
+//    predecessor it computes once more.  The new stream goes to another buffer,
+//    so that this never meets a row that its own group has already replaced.
+//    A single token's predecessor is what its slot keeps.
 //
 // What a sequence keeps for its next step (its last token, its last h) is
 // read and replaced by whoever has the first row of its portion: that group
@@ -84,7 +85,8 @@ stream_embed_kernel(EmbedArgs a, RaggedRows r) {
   }
 }
 
-template <bool F32, int TPR, int VEC, int NV>
+// WALK: groups of `per` rows of the portions; else a single token each
+template <bool F32, int TPR, int VEC, int NV, bool WALK>
 __global__ void __launch_bounds__(256)
 shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
   __shared__ float red[4];
@@ -92,14 +94,8 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
   // with a block per row everything that depends on the row alone is uniform
   const int task = TPR == 256 ? blockIdx.x
                               : blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
-  int row0, rows;
-  if (task < r.n_dec) {
-    row0 = task;
-    rows = 1;
-  } else {
-    row0 = r.n_dec + (task - r.n_dec) * per;
-    rows = min(per, r.T - row0);
-  }
+  const int row0 = WALK ? r.n_dec + task * per : task;
+  const int rows = WALK ? min(per, r.T - row0) : task < r.n_dec;
   if (rows <= 0) return;              // whole wave (TPR 64) or whole block
 
   Held<F32, VEC> wn[NV], mix[NV];
@@ -113,9 +109,9 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
     }
   }
 
-  // a row's new stream and its norm
-  auto make = [&](long row, bool store, Pack<VEC> (&h)[NV]) {
-    constexpr int CH = NV <= 4 ? 6 : 2;       // parts with loads in flight
+  // a row's new stream and its norm; also() is called when the loads are out
+  auto make = [&](long row, bool store, Pack<VEC> (&h)[NV], auto also) {
+    constexpr int CH = NV <= 4 ? 6 : NV <= 8 ? 2 : 1;  // loads in flight
     Held<F32, VEC> t[CH][NV];
     const int n = a.y.y ? (a.y.w ? a.y.n : 1) : 0;
     float wt[CH];
@@ -141,6 +137,7 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
       h[i] = Pack<VEC>{};
       if (c < W) h[i] = ldv<true, VEC>(a.x, row * W + c);
     }
+    also();
     for (int k0 = 0; k0 < n; k0 += CH) {
       if (k0) fetch(k0);
       #pragma unroll
@@ -183,39 +180,24 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
     }
   };
 
-  auto keep = [&](int s, const Pack<VEC> (&h)[NV]) {
+  Pack<VEC> before[NV], h[NV];
+  auto recall = [&](int row, int s) {
+    const bool old = s >= 0 && r.pos[row] > 0;
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * TPR + tid) * VEC;
+      before[i] = Pack<VEC>{};
+      if (old && c < W) before[i] = ldv<true, VEC>(a.state, (long)s * W + c);
+    }
+  };
+  auto keep = [&](int s) {
     #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int c = (i * TPR + tid) * VEC;
       if (c < W) stv<true, VEC>(a.state, (long)s * W + c, h[i]);
     }
   };
-
-  Pack<VEC> before[NV], h[NV];
-  #pragma unroll
-  for (int i = 0; i < NV; ++i) before[i] = Pack<VEC>{};
-  if (a.shift && !starts(r, row0)) make(row0 - 1, false, before);
-  for (int k = 0; k < rows; ++k) {
-    const int row = row0 + k;
-    if (a.shift && starts(r, row)) {
-      const int s = r.slot[row];
-      const bool old = s >= 0 && r.pos[row] > 0;
-      #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int c = (i * TPR + tid) * VEC;
-        before[i] = Pack<VEC>{};
-        if (old && c < W) before[i] = ldv<true, VEC>(a.state, (long)s * W + c);
-      }
-      if (row >= r.n_dec && s >= 0) {
-        const int end = last_row(r, s);
-        if (end >= 0) {
-          make(end, false, h);
-          keep(s, h);
-        }
-      }
-    }
-    make(row, true, h);
-    if (a.shift && row < r.n_dec && r.slot[row] >= 0) keep(r.slot[row], h);
+  auto blend = [&](int row) {
     #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int c = (i * TPR + tid) * VEC;
@@ -228,6 +210,46 @@ shift_norm_kernel(ShiftArgs a, RaggedRows r, int per) {
       }
       if (c < W) stv<F32, VEC>(a.h, (long)row * W + c, o);
     }
+  };
+  if constexpr (!WALK) {
+    const int s = a.shift ? r.slot[row0] : -1;
+    make(row0, true, h, [&] { recall(row0, s); });
+    if (s >= 0) keep(s);
+    blend(row0);
+  } else {
+    // k -1: the row before the first, nothing but its norm.  A portion's last
+    // row comes before its first one (`ahead`), for what the slot keeps.
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) before[i] = Pack<VEC>{};
+    bool ahead = false;
+    int k = a.shift && !starts(r, row0) ? -1 : 0;
+    while (k < rows) {
+      const int row = row0 + k;
+      int s = -1, at = row;
+      if (k >= 0 && a.shift && starts(r, row)) {
+        s = r.slot[row];
+        if (!ahead) {
+          recall(row, s);
+          const int end = s >= 0 ? last_row(r, s) : -1;
+          ahead = end >= 0;
+          if (ahead) at = end;
+        } else {
+          ahead = false;
+        }
+      }
+      make(at, k >= 0 && !ahead, h, [] {});
+      if (ahead) {
+        keep(s);
+        continue;
+      }
+      if (k >= 0) {
+        blend(row);
+      } else {
+        #pragma unroll
+        for (int i = 0; i < NV; ++i) before[i] = h[i];
+      }
+      ++k;
+    }
   }
 }
 
@@ -236,17 +258,22 @@ void launch_shift(const ShiftArgs& a, const RaggedRows& r, hipStream_t st) {
   // more rows a group: less work done twice; fewer: more groups
   const int rest = r.T - r.n_dec;
   const int per = !a.shift || rest <= 512 ? 1 : rest <= 2048 ? 2 : rest <= 4096 ? 4 : 8;
-  const int tasks = r.n_dec + (rest + per - 1) / per;
+  const int tasks = (rest + per - 1) / per;
+  #define SN_ONE(TPR, NV, WALK, N)                                             \
+    if (N > 0)                                                                 \
+      hipLaunchKernelGGL((shift_norm_kernel<F32, TPR, VEC, NV, WALK>),         \
+                         dim3((unsigned)(((long)(N) * TPR + 255) / 256)),      \
+                         dim3(256), 0, st, a, r, per)
   #define SN_GO(TPR, NV)                                                       \
-    hipLaunchKernelGGL((shift_norm_kernel<F32, TPR, VEC, NV>),                 \
-                       dim3((tasks * TPR + 255) / 256), dim3(256), 0, st, a, r, per)
-  if (a.W <= 64 * VEC) SN_GO(64, 1);
-  else if (a.W <= 256 * VEC) SN_GO(256, 1);
-  else if (a.W <= 512 * VEC) SN_GO(256, 2);
-  else if (a.W <= 1024 * VEC) SN_GO(256, 4);
-  else if (a.W <= 2048 * VEC) SN_GO(256, 8);
-  else SN_GO(256, 16);            // up to 4096 * VEC (checked by the caller)
+    { SN_ONE(TPR, NV, false, r.n_dec); SN_ONE(TPR, NV, true, tasks); }
+  if (a.W <= 64 * VEC) SN_GO(64, 1)
+  else if (a.W <= 256 * VEC) SN_GO(256, 1)
+  else if (a.W <= 512 * VEC) SN_GO(256, 2)
+  else if (a.W <= 1024 * VEC) SN_GO(256, 4)
+  else if (a.W <= 2048 * VEC) SN_GO(256, 8)
+  else SN_GO(256, 16)             // up to 4096 * VEC (checked by the caller)
   #undef SN_GO
+  #undef SN_ONE
 }
 
 }  // namespace
