@@ -581,6 +581,109 @@ def test_experts_by_token(dev, dt, T, E, top, ff, W):
     close(parts.total(), O.table_moe(h, w, "", tokens.tolist()), dt)
 
 
+# ----------------------------------------------------- parts of other stacks
+@place
+def test_parallel_is_the_sum_of_its_sides(dev, dt):
+    """Each side also stands alone, with matrices of its own."""
+    from scaffold.cache import PagedStateCache
+    from scaffold.models import mixers as M
+
+    left = {"type": "window_attention", "heads": 4, "kv_heads": 2, "dim": 16,
+            "vdim": 9, "scale": 0.3, "softcap": 5.0, "buckets": 9,
+            "bias_max": 30, "mask": {"size": 20, "keep_first": 2}}
+    right = {"type": "gla", "heads": 3, "dim": 8, "vdim": 5, "rank": 6,
+             "tau": 4.0}
+    W, T, eps = 40, 90, 1e-4
+    torch.manual_seed(0)
+    both = M.Parallel(W, {"left": left, "right": right, "left_scale": 0.6,
+                          "right_scale": -1.5}, eps)
+    sides = [M.WindowAttention(W, left, eps),
+             M.GatedLinearAttention(W, right, eps)]
+    with torch.no_grad():
+        for i, side in enumerate(sides):
+            own = dict(side.packed())
+            for n, t in both.packed():
+                if n.startswith(("left.", "right.")[i]):
+                    t.copy_(rnd(*t.shape, seed=len(n) + i) * t.shape[-1] ** -0.5)
+                    own[n.split(".", 1)[1]].copy_(t)
+    mods = [m.to(dev, dt) for m in (both, *sides)]
+    cache = PagedStateCache([m.cache_spec() for m in mods], 2, 256, 256, dev,
+                            dt)
+    slot, h = cache.open(), rnd(T, W, seed=3).to(dev, dt)
+    with torch.no_grad():
+        a, b, c = feed(T, [40, 1, 49], cache, slot, [0] * T, lambda plan, i, j: [
+            m.step(h[i:j].contiguous(), plan, cache, run)
+            for run, m in enumerate(mods)])
+    close(a, (0.6 * b.double() - 1.5 * c.double()).cpu(), dt)
+    with pytest.raises(ValueError, match="retention"):
+        M.Parallel(W, {"left": left, "right": {"type": "retention"},
+                       "left_scale": 1, "right_scale": 1}, eps)
+
+
+@pytest.mark.parametrize("dev", ["cpu", pytest.param("cuda", marks=gpu)])
+@pytest.mark.parametrize("shift", [False, True])
+@pytest.mark.parametrize("start", [False, True])
+@pytest.mark.parametrize("loop", [False, True])
+def test_every_choice_of_a_stack_alone(dev, shift, start, loop):
+    """Token shift, embeddings and added loop inputs do not need each other:
+    any cut gives the same logits, and a shift by nothing is no shift."""
+    from scaffold.config import load_config
+    from scaffold.generate import Generator
+    from scaffold.models import build_model
+    from tests.oracle.cases import attn, poison, ret
+
+    def make(shift):
+        cfg = load_config(None, ["model.name=lasezen", "model.vocab_size=31",
+                                 "model.d_model=20", "model.norm=rms_norm",
+                                 "model.post_norm=false"])
+        m = cfg.model
+        m.layers = [attn(), ret(ff=None)]
+        m.token_shift, m.loop_add = shift, loop
+        m.loop = {"start": 1, "stop": 2, "times": 3} if loop else None
+        if start:
+            m.sinusoid_base = 500.0
+            m.bigram = {"buckets": 7, "mul_prev": 3, "mul_cur": 2}
+        torch.manual_seed(1)
+        model = build_model(cfg)
+        with torch.no_grad():
+            for n, p in model.named_parameters():
+                if p.dim() > 1:
+                    p.copy_(torch.randn(p.shape) * p.shape[-1] ** -0.5)
+                elif n.endswith("shift"):
+                    p.zero_()
+        return model.to(dev).eval()
+
+    t = torch.randint(0, 31, (70,), generator=torch.Generator().manual_seed(2))
+    t = t.tolist()
+
+    def logits(model, parts):
+        cache, out, at = poison(model.new_cache(2, 256, 128)), [], 0
+        s = cache.open()
+        for n in parts:
+            out.append(Generator(model).step(cache, [(s, t[at:at + n], range(n))]))
+            at += n
+        return torch.cat(out).double().cpu()
+
+    model = make(shift)
+    torch.manual_seed(1)
+    plain = make(False)
+    with torch.no_grad():
+        sd = model.state_dict()
+        plain.load_state_dict({k: v for k, v in sd.items()
+                               if not k.endswith("shift")})
+    want = logits(plain, [70])
+    for parts in ([70], [1] * 70, cuts(70, [2, 33])):
+        close(logits(model, parts), want, torch.float32, 5)
+    if shift:
+        with torch.no_grad():
+            for b in model.blocks:
+                b.shift.fill_(0.4)
+        want = logits(model, [70])
+        assert (want - logits(plain, [70])).abs().max() > 1e-2
+        for parts in ([1] * 70, cuts(70, [2, 33])):
+            close(logits(model, parts), want, torch.float32, 5)
+
+
 # ------------------------------------------------------------------- checks
 @gpu
 def test_bindings_refuse_bad_operands():
